@@ -2,10 +2,10 @@
 count of tokens whose keys and values are stored, and the rules by which pages are taken,
 shared, and given back.
 
-Layers whose mixers have the same need (all earlier keys; or a window of a given length)
-form a *group*: one page pool and one block table per request serve all layers of the
+Layers whose mixers have the same need (all earlier keys; a window of a given length; or the keys of
+the query's own block of a given number of positions) form a *group*: one page pool and one block table per request serve all layers of the
 group, each layer having page storage of its own.  Pages of a window group are given back
-as soon as the window has passed them; all pages and the slot are given back when the
+as soon as the window has passed them, those of a block group when the next token begins another block; all pages and the slot are given back when the
 request ends.  Full pages of the all-keys group are hashed by content (chained over the
 prefix) so that a later request with the same prefix takes them instead of recomputing.
 
@@ -26,13 +26,22 @@ from .state_slots import StateSlotPool
 
 @dataclass
 class CacheGroup:
-    key: tuple                 # ("full",) or ("window", W)
+    key: tuple                 # ("full",), ("window", W) or ("chunk", C)
     runs: list                 # schedule entries whose own cache lives in this group
     pool: PagePool
 
     @property
-    def window(self) -> Optional[int]:
-        return self.key[1] if self.key[0] == "window" else None
+    def keeps_all(self) -> bool:
+        """Whether a request's pages stay until it ends."""
+        return self.key[0] == "full"
+
+    def first_needed(self, position: int) -> int:
+        """The earliest position whose key the query at ``position``, or any later one, still reads."""
+        if self.key[0] == "window":
+            return max(0, position - self.key[1] + 1)
+        if self.key[0] == "chunk":
+            return position - position % self.key[1]
+        return 0
 
 
 @dataclass
@@ -54,7 +63,7 @@ class RequestCache:
 class CacheManager:
     def __init__(self, group_keys: Sequence[tuple], page_size: int, num_pages, max_num_seqs: int,
                  enable_prefix_cache: bool = True, has_state: bool = False):
-        """``group_keys``: the distinct cache needs in the model, e.g. [("full",), ("window", 128)].
+        """``group_keys``: the distinct cache needs in the model, e.g. [("full",), ("window", 128), ("chunk", 512)].
         ``num_pages``: usable pages per group (an int for all, or one per group)."""
         self.page_size = int(page_size)
         if isinstance(num_pages, int):
@@ -193,12 +202,10 @@ class CacheManager:
                 pool.register_hash(table[i], h)
                 rc.hashes.append(h)
         for gi, (g, table) in enumerate(zip(self.groups, rc.tables)):
-            w = g.window
-            if w is None:
+            # the next query sits at position ctx: pages that end at or before its first key are dead
+            dead_pages = g.first_needed(ctx) // ps
+            if not dead_pages:
                 continue
-            # the next query sits at position ctx and reads keys > ctx - w: pages that end at or
-            # before ctx - w + 1 are dead
-            dead_pages = max(0, ctx - w + 1) // ps
             gone = [i for i in range(min(dead_pages, len(table))) if table[i] != NULL_PAGE]
             g.pool.release([table[i] for i in gone])
             for i in gone:

@@ -10,17 +10,27 @@ from __future__ import annotations
 
 import torch
 
-from ..parts.spec import LayerMemory, state_specs_of
+from ..parts.spec import LayerMemory, state_specs_of, widest_need
 
 _STATE_DTYPES = {"float32": torch.float32, "bfloat16": torch.bfloat16, "int32": torch.int32}
+
+
+def needs_of(plan) -> dict:
+    """Run -> group key of every run with a cache of its own: the widest of its own need and those of the runs that
+    read its cache."""
+    needs: dict = {}
+    for p in plan:
+        if p.cache is not None:
+            needs.setdefault(p.run if p.cache_of is None else p.cache_of, []).append(p.cache.group_key)
+    return {run: widest_need(keys) for run, keys in needs.items()}
 
 
 def group_keys_of(plan) -> list:
     """Distinct cache needs in schedule order of first appearance."""
     keys = []
-    for p in plan:
-        if p.cache is not None and p.cache_of is None and p.cache.group_key not in keys:
-            keys.append(p.cache.group_key)
+    for key in needs_of(plan).values():
+        if key not in keys:
+            keys.append(key)
     return keys
 
 
@@ -33,11 +43,12 @@ def allocate_memories(plan, group_keys, num_pages, page_size: int, max_num_seqs:
     if isinstance(num_pages, int):
         num_pages = [num_pages] * len(group_keys)
     memories = []
+    needs = needs_of(plan)
     for p in plan:
         mem = LayerMemory()
         if p.cache is not None:
             if p.cache_of is None:
-                g = group_keys.index(p.cache.group_key)
+                g = group_keys.index(needs[p.run])
                 for t in p.cache.tensors:
                     kind = dtype if t.dtype is None else _STATE_DTYPES[t.dtype]
                     mem.pages[t.name] = torch.zeros((num_pages[g] + 1, *t.page_shape(page_size)), dtype=kind, device=device)
@@ -51,10 +62,6 @@ def allocate_memories(plan, group_keys, num_pages, page_size: int, max_num_seqs:
                     raise ValueError(f"run {p.run} cannot read run {p.cache_of}'s cache: they declare different tensors "
                                      f"({[(t.name, t.token_shape) for t in own.tensors]} against "
                                      f"{[(t.name, t.token_shape) for t in other.tensors]})")
-                if other.window is not None and (own.window is None or own.window > other.window):
-                    raise ValueError(
-                        f"run {p.run} cannot read run {p.cache_of}'s cache: it needs keys that the owner's "
-                        f"window of {other.window} has already given back")
                 mem.pages, mem.group, mem.writes = owner.pages, owner.group, False
         for st in state_specs_of(p.state):
             # one row per slot and a spare one that belongs to no request

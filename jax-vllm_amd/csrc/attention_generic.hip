@@ -5,7 +5,8 @@
 // with a running (max, sum) softmax.
 //
 //   query token t of request r = token_req[t] sits at absolute position p = positions[t]
-//   and sees keys j with  max(0, p - window + 1) <= j <= p   (window <= 0: all j <= p);
+//   and sees keys j with  max(0, p - window + 1) <= j <= p   (window 0: all j <= p; window < 0: those of
+//   its own block of -window positions, counted from position 0);
 //   key j lives in page block_tables[r, j / page_size] at slot j % page_size;
 //   q head h reads kv head h / (nq / nkv).
 // With `sinks` (one float per q head) every row's softmax denominator also holds exp(sinks[h]).
@@ -32,7 +33,7 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
   const int kvh = h / (nq / nkv);
   const int r = token_req[t];
   const int pos = positions[t];
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = window < 0 ? pos - pos % -window : (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
   const int* table = block_tables + (long long)r * table_stride;
   const T* qv = q + t * q_row_stride + (long long)h * D;
   for (int d = lane; d < D; d += 64) qs[d] = to_f32(qv[d]);

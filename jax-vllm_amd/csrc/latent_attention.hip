@@ -37,7 +37,8 @@ extern "C" int jv_rope_table_amp(float* cos_sin, const int* positions, const flo
 //            token's slot (slot_mapping[t] < 0: nothing is stored)
 // rotate: element i < half pairs with i + half (half = rot_dims / 2), or (interleaved) element 2i with 2i + 1,
 // both by the angle of frequency i; elements from rot_dims on pass.  q_rank may be 0 (queries that are projected
-// directly: no query latent, cq null); the kv latent begins at column kv_off of the row.
+// directly: no query latent, cq null); the kv latent begins at column kv_off of the row.  rank may be 0 (a layer that
+// reads another layer's cache: the query latent alone).
 // One block per token.
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -53,8 +54,8 @@ latent_prepare_kernel(const T* __restrict__ proj, long long ld, int q_rank, long
   for (int c = threadIdx.x; c < q_rank; c += blockDim.x) { const float v = to_f32(x[c]); sq += v * v; }
   for (int c = threadIdx.x; c < rank; c += blockDim.x) { const float v = to_f32(x[kv_off + c]); sk += v * v; }
   if (q_rank) sq = block_sum(sq, red);
-  sk = block_sum(sk, red);
-  const float inv_q = q_rank ? rsqrtf(sq / (float)q_rank + eps) : 0.f, inv_k = rsqrtf(sk / (float)rank + eps);
+  if (rank) sk = block_sum(sk, red);
+  const float inv_q = q_rank ? rsqrtf(sq / (float)q_rank + eps) : 0.f, inv_k = rank ? rsqrtf(sk / (float)rank + eps) : 0.f;
   for (int c = threadIdx.x; c < q_rank; c += blockDim.x)
     cq[t * q_rank + c] = from_f32<T>(to_f32(x[c]) * inv_q * wq[c]);
   const long long slot = slot_mapping ? (long long)slot_mapping[t] : -1;
@@ -276,7 +277,7 @@ extern "C" int jv_head_linear_mfma_bf16(void* y, long long ldy, int ys, const vo
                                          void* cq, void* k_pages, void* v_pages, int page_size,            \
                                          void* stream) {                                                   \
     if (n <= 0) return 0;                                                                                  \
-    if (q_rank < 0 || kv_off < 0 || rank <= 0 || rot < 0 || rot_dims < 0 || rot_dims > rot || rot_dims % 2 || \
+    if (q_rank < 0 || kv_off < 0 || rank < 0 || (!rank && k_pages) || rot < 0 || rot_dims < 0 || rot_dims > rot || rot_dims % 2 || \
         (q_rank && (!wq || !cq)))                                                                          \
       return (int)hipErrorInvalidValue;                                                                    \
     hipLaunchKernelGGL(latent_prepare_kernel<T>, dim3(n), dim3(256), 0, (hipStream_t)stream,               \

@@ -5,11 +5,13 @@
 //   route:   z = router logits (float, plus an optional bias per expert) -> the `top` largest per token
 //            (lowest index among equals), weight = sigmoid(z), or the softmax over the chosen logits alone, or
 //            ("sigmoid_normed") the largest sigmoid(z) + correction chosen, weight = sigmoid(z) over the sum of the
-//            chosen sigmoids (+ 1e-20) times a constant
+//            chosen sigmoids (+ 1e-20) times a constant, or ("softmax") the softmax over ALL logits, as it is.
+//            Experts may form equal groups of neighbours: only those of the `keep` groups with the largest logits
+//            (lowest group among equals) can then be chosen
 //   group:   entry s = token * top + kk  ->  position in a list ordered by expert; tiles of MOE_TM rows
 //            that never straddle two experts
 //   gate/up: z[pos] = act(w g) * (w u),  g = Wg[e] x[token], u = Wu[e] x[token]      (w = the entry's weight
-//            when it scales the expert's INPUT: w (W x) = W (w x); else 1)
+//            when it scales the expert's INPUT: w (W x) = W (w x); else 1); experts without a gate: act(w u)
 //   down:    y[kk][token] = (Wd[e] z[pos]) * (w if it scales the OUTPUT else 1)        float
 // The order of rows inside an expert's group depends on timing; no result does: every output row is a
 // sum over the inner size in ascending order, alone.
@@ -24,10 +26,36 @@
 #define MOE_SCORE_SIGMOID 0          // weight = sigmoid(logit)
 #define MOE_SCORE_SOFTMAX_CHOSEN 1   // weight = exp(logit) / sum of exp over the token's chosen logits
 #define MOE_SCORE_SIGMOID_NORMED 2   // chosen by sigmoid(logit) + correction; weight = sigmoid(logit) / (sum over the chosen + 1e-20) * scale
+#define MOE_SCORE_SOFTMAX 3          // weight = exp(logit) / sum of exp over all of the token's logits
+#define MOE_MAX_GROUPS 64
 __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int lane, int* ids, float* weights,
-                                         int score, const float* __restrict__ correction = nullptr,
-                                         float weight_scale = 1.f) {
+                                         int score, const float* __restrict__ correction, float weight_scale,
+                                         int groups, int keep) {
   const bool normed = score == MOE_SCORE_SIGMOID_NORMED;
+  float zmax = 0.f, inv_sum = 0.f;
+  if (score == MOE_SCORE_SOFTMAX) {      // over all experts, before any is left out
+    float m = -INFINITY, sum = 0.f;
+    for (int e = lane; e < experts; e += JV_WAVE) m = fmaxf(m, zt[e]);
+    zmax = wave_max(m);
+    for (int e = lane; e < experts; e += JV_WAVE) sum += expf(zt[e] - zmax);
+    inv_sum = 1.f / wave_sum(sum);
+  }
+  if (groups > 1 && keep < groups) {
+    // lane g ranks group g by its largest logit; every lane then takes the lost groups' experts out of those it scans
+    const int size = experts / groups;
+    float best = -INFINITY;
+    if (lane < groups)
+      for (int i = 0; i < size; ++i) best = fmaxf(best, zt[lane * size + i]);
+    int ahead = 0;
+    for (int g = 0; g < groups; ++g) {
+      const float other = __shfl(best, g, JV_WAVE);
+      if (other > best || (other == best && g < lane)) ++ahead;
+    }
+    const unsigned long long kept = __ballot(lane < groups && ahead < keep);
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // the groups are read before their entries change
+    for (int e = lane; e < experts; e += JV_WAVE)
+      if (!((kept >> (e / size)) & 1)) zt[e] = -INFINITY;
+  }
   for (int kk = 0; kk < top; ++kk) {
     float bv = -INFINITY;
     int bi = 0x7fffffff;
@@ -47,7 +75,8 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
     if (lane == 0) {
       ids[kk] = bi;
       const float z = normed ? zt[bi] : bv;          // the logit itself: the correction takes part in the choice only
-      weights[kk] = score == MOE_SCORE_SOFTMAX_CHOSEN ? bv : 1.f / (1.f + expf(-z));
+      weights[kk] = score == MOE_SCORE_SOFTMAX_CHOSEN ? bv : score == MOE_SCORE_SOFTMAX ? expf(z - zmax) * inv_sum
+                                                                                        : 1.f / (1.f + expf(-z));
     }
     if ((bi & (JV_WAVE - 1)) == lane) zt[bi] = -INFINITY;
   }
@@ -75,14 +104,15 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ bias, int n, int experts, int top,
                  int score, int* __restrict__ ids, float* __restrict__ weights, const float* __restrict__ correction,
-                 float weight_scale) {
+                 float weight_scale, int groups, int keep) {
   extern __shared__ float zs[];      // [4][experts]
   const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE;
   const long long t = (long long)blockIdx.x * 4 + wid;
   if (t >= n) return;
   float* zt = zs + wid * experts;
   for (int e = lane; e < experts; e += JV_WAVE) zt[e] = logits[t * experts + e] + (bias ? bias[e] : 0.f);
-  moe_pick(zt, experts, top, lane, ids + t * top, weights + t * top, score, correction, weight_scale);
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");        // a group's lane reads what other lanes wrote
+  moe_pick(zt, experts, top, lane, ids + t * top, weights + t * top, score, correction, weight_scale, groups, keep);
 }
 
 // Router and choice in one launch: a block takes up to MOE_RT tokens, their rows in LDS as floats; a wave per
@@ -95,7 +125,8 @@ template <typename T>
 __global__ void __launch_bounds__(1024)
 moe_router_kernel(const T* __restrict__ x, const T* __restrict__ W, const float* __restrict__ bias, int n, int hidden,
                   int experts, int top, int tb, int score, int* __restrict__ ids, float* __restrict__ weights,
-                  float* __restrict__ logits_out, const float* __restrict__ correction, float weight_scale) {
+                  float* __restrict__ logits_out, const float* __restrict__ correction, float weight_scale, int groups,
+                  int keep) {
   extern __shared__ float rs[];      // x [tb][hidden] | z [tb][experts]
   float* xs = rs;
   float* z = rs + tb * hidden;
@@ -143,7 +174,7 @@ moe_router_kernel(const T* __restrict__ x, const T* __restrict__ W, const float*
   __syncthreads();
   for (int t = wid; t < nt; t += nw)
     moe_pick(z + t * experts, experts, top, lane, ids + (t0 + t) * top, weights + (t0 + t) * top, score, correction,
-             weight_scale);
+             weight_scale, groups, keep);
 }
 
 // One block.  meta: [0] number of tiles; offsets [experts + 1]; tile_expert / tile_row0 [max_tiles];
@@ -183,8 +214,8 @@ moe_group_kernel(const int* __restrict__ ids, int entries, int experts, int tile
 }
 
 // grid (max tiles, column tiles of the expert width).  x [tokens, hidden]; Wg, Wu [experts, ff, hidden];
-// z [entries, ff] by position.
-template <typename T>
+// z [entries, ff] by position.  Without GATED there is no Wg and the activation stands alone.
+template <typename T, bool GATED>
 __global__ void __launch_bounds__(256)
 moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restrict__ Wg, const T* __restrict__ Wu,
                    const int* __restrict__ meta, const int* __restrict__ offsets, const int* __restrict__ tile_expert,
@@ -192,7 +223,7 @@ moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restri
                    int top, int hidden, int ff, int act, int scale_input) {
   if ((int)blockIdx.x >= meta[0]) return;
   __shared__ float As[MOE_BK][MOE_TM + 4];
-  __shared__ float Gs[MOE_BK][MOE_TN + 4];
+  __shared__ float Gs[GATED ? MOE_BK : 1][MOE_TN + 4];
   __shared__ float Us[MOE_BK][MOE_TN + 4];
   __shared__ int tok[MOE_TM];
   __shared__ float wgt[MOE_TM];
@@ -206,7 +237,7 @@ moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restri
     wgt[tid] = (s < 0 || !scale_input) ? 1.f : weights[s];
   }
   __syncthreads();
-  const T* G = Wg + (long long)e * ff * hidden;
+  const T* G = GATED ? Wg + (long long)e * ff * hidden : nullptr;
   const T* U = Wu + (long long)e * ff * hidden;
   float ag[4][4] = {}, au[4][4] = {};
   for (int k0 = 0; k0 < hidden; k0 += MOE_BK) {
@@ -217,7 +248,7 @@ moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restri
       const int tk = tok[r], wn = n0 + r;
       As[kk][r] = (tk >= 0 && k < hidden) ? to_f32(x[(long long)tk * hidden + k]) : 0.f;
       const bool in = wn < ff && k < hidden;
-      Gs[kk][r] = in ? to_f32(G[(long long)wn * hidden + k]) : 0.f;
+      if (GATED) Gs[kk][r] = in ? to_f32(G[(long long)wn * hidden + k]) : 0.f;
       Us[kk][r] = in ? to_f32(U[(long long)wn * hidden + k]) : 0.f;
     }
     __syncthreads();
@@ -227,12 +258,12 @@ moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restri
 #pragma unroll
       for (int i = 0; i < 4; ++i) a[i] = As[kk][ty * 4 + i];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) { g[j] = Gs[kk][tx * 4 + j]; u[j] = Us[kk][tx * 4 + j]; }
+      for (int j = 0; j < 4; ++j) { g[j] = GATED ? Gs[GATED ? kk : 0][tx * 4 + j] : 0.f; u[j] = Us[kk][tx * 4 + j]; }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          ag[i][j] = fmaf(a[i], g[j], ag[i][j]);
+          if (GATED) ag[i][j] = fmaf(a[i], g[j], ag[i][j]);
           au[i][j] = fmaf(a[i], u[j], au[i][j]);
         }
     }
@@ -246,7 +277,7 @@ moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restri
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < ff) z[(long long)(row0 + m) * ff + n] = from_f32<T>(jv_gated(act, ag[i][j] * w, au[i][j] * w));
+      if (n < ff) z[(long long)(row0 + m) * ff + n] = from_f32<T>(GATED ? jv_gated(act, ag[i][j] * w, au[i][j] * w) : jv_act(act, au[i][j] * w));
     }
   }
 }
@@ -339,14 +370,22 @@ row_gate_vec_kernel(float* __restrict__ out, const T* __restrict__ y, const T* _
 
 extern "C" int jv_moe_tile_rows() { return MOE_TM; }
 
+// equal groups of neighbours, the kept ones with enough experts for the choice (groups <= 1: none)
+static bool moe_groups_ok(int experts, int top, int groups, int keep) {
+  return groups <= 1 || (groups <= MOE_MAX_GROUPS && experts % groups == 0 && keep >= 1 && keep <= groups &&
+                         (long long)keep * (experts / groups) >= top);
+}
+
 extern "C" int jv_moe_route(const float* logits, const float* bias, int n, int experts, int top, int score, int* ids,
-                            float* weights, const float* correction, float weight_scale, void* stream) {
+                            float* weights, const float* correction, float weight_scale, int groups, int keep,
+                            void* stream) {
   if (n <= 0) return 0;
-  if (experts <= 0 || top <= 0 || top > experts || score < 0 || score > MOE_SCORE_SIGMOID_NORMED)
+  if (experts <= 0 || top <= 0 || top > experts || score < 0 || score > MOE_SCORE_SOFTMAX)
     return (int)hipErrorInvalidValue;
+  if (!moe_groups_ok(experts, top, groups, keep)) return (int)hipErrorInvalidValue;
   if (experts > 3840) return (int)hipErrorInvalidValue;
   hipLaunchKernelGGL(moe_route_kernel, dim3((n + 3) / 4), dim3(256), 4 * experts * sizeof(float), (hipStream_t)stream,
-                     logits, bias, n, experts, top, score, ids, weights, correction, weight_scale);
+                     logits, bias, n, experts, top, score, ids, weights, correction, weight_scale, groups, keep);
   return JV_LAUNCH_CHECK();
 }
 
@@ -362,11 +401,11 @@ extern "C" int jv_moe_group(const int* ids, int entries, int experts, int tile_r
 #define DEFINE_MOE(SUF, T)                                                                                        \
   extern "C" int jv_moe_router_##SUF(const void* x, const void* W, const float* bias, int n, int hidden,          \
                                      int experts, int top, int score, int* ids, float* weights,                   \
-                                     float* logits_out, const float* correction, float weight_scale,              \
-                                     void* stream) {                                                              \
+                                     float* logits_out, const float* correction, float weight_scale, int groups,  \
+                                     int keep, void* stream) {                                                    \
     if (n <= 0) return 0;                                                                                         \
     if (experts <= 0 || top <= 0 || top > experts || hidden <= 0 || (hidden + experts) > 15000 || score < 0 ||    \
-        score > MOE_SCORE_SIGMOID_NORMED)                                                                         \
+        score > MOE_SCORE_SOFTMAX || !moe_groups_ok(experts, top, groups, keep))                                  \
       return (int)hipErrorInvalidValue;                                                                           \
     int tb = 15000 / (hidden + experts);             /* tokens of a block: their rows and logits in 60 KB */      \
     tb = tb > MOE_RT ? MOE_RT : tb;                                                                               \
@@ -374,7 +413,7 @@ extern "C" int jv_moe_group(const int* ids, int entries, int experts, int tile_r
     hipLaunchKernelGGL(moe_router_kernel<T>, dim3((n + tb - 1) / tb), dim3(1024),                                  \
                        (size_t)tb * (hidden + experts) * sizeof(float), (hipStream_t)stream, (const T*)x,         \
                        (const T*)W, bias, n, hidden, experts, top, tb, score, ids, weights, logits_out,           \
-                       correction, weight_scale);                                                                 \
+                       correction, weight_scale, groups, keep);                                                   \
     return JV_LAUNCH_CHECK();                                                                                     \
   }                                                                                                               \
   extern "C" int jv_row_gate_##SUF(float* out, const void* y, const void* g, long long ldg, long long n,         \
@@ -395,8 +434,10 @@ extern "C" int jv_moe_group(const int* ids, int entries, int experts, int tile_r
                                       const int* order, const float* weights, int max_tiles, int top, int hidden, \
                                       int ff, int act, int scale_input, void* stream) {                           \
     if (max_tiles <= 0 || ff <= 0) return 0;                                                                      \
-    if (!jv_act_known(act) || (ff + MOE_TN - 1) / MOE_TN > 65535) return (int)hipErrorInvalidValue;               \
-    hipLaunchKernelGGL(moe_gate_up_kernel<T>, dim3(max_tiles, (ff + MOE_TN - 1) / MOE_TN), dim3(256), 0,          \
+    if (!(Wg ? jv_act_known(act) : jv_plain_act_known(act)) || (ff + MOE_TN - 1) / MOE_TN > 65535)                \
+      return (int)hipErrorInvalidValue;                                                                           \
+    auto kernel = Wg ? moe_gate_up_kernel<T, true> : moe_gate_up_kernel<T, false>;                                \
+    hipLaunchKernelGGL(kernel, dim3(max_tiles, (ff + MOE_TN - 1) / MOE_TN), dim3(256), 0,          \
                        (hipStream_t)stream, (T*)z, (const T*)x, (const T*)Wg, (const T*)Wu, meta, offsets,        \
                        tile_expert, tile_row0, order, weights, top, hidden, ff, act, scale_input);                \
     return JV_LAUNCH_CHECK();                                                                                     \

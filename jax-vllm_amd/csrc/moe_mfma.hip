@@ -7,25 +7,29 @@
 // multiplied.  v_mfma_f32_16x16x32_bf16 with A = 16 rows of W (wave w owns rows 16 w .. 16 w + 15 of the
 // tile), B = 16 rows of x: the accumulator of row tile mt holds y^T[n = 4 lc + e][m = 16 mt + li].
 // Each output row is a sum over the inner size in a fixed order, whatever else is in the step.
-//   GATED:  z[pos] = act(w g) * (w u), g = Wg[e] x[token], u = Wu[e] x[token]       (bf16)
-//   else:   y[kk][token] = (Wd[e] z[pos]) * w_out                                   (float)
+//   MM_GATED:  z[pos] = act(w g) * (w u), g = Wg[e] x[token], u = Wu[e] x[token]    (bf16)
+//   MM_PLAIN:  z[pos] = act(w u), u = Wu[e] x[token]: experts without a gate        (bf16)
+//   MM_DOWN:   y[kk][token] = (Wd[e] z[pos]) * w_out                                (float)
 #include "common.h"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+enum { MM_DOWN = 0, MM_GATED = 1, MM_PLAIN = 2 };
 
 #define MM_T 64            // rows of a tile, rows of W of a block, columns of a chunk
 #define MM_S 80            // LDS row length: 40 dwords, 8 mod 16: 16-byte reads of 16 rows are conflict-free
 
 // MT: row tiles of 16 a block takes (a tile of the grouping has 16 MT rows).  Without a grouping
 // (tile_expert null) the product is a plain one: rows in order, one weight matrix, float output [rows, N].
-template <bool GATED, int MT>
+template <int MODE, int MT>
 __global__ void __launch_bounds__(256)
 moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const bf16_t* __restrict__ W0,
                 const bf16_t* __restrict__ W1, const int* __restrict__ meta, const int* __restrict__ offsets,
                 const int* __restrict__ tile_expert, const int* __restrict__ tile_row0, const int* __restrict__ order,
                 const float* __restrict__ weights, int top, int n_tokens, int K, int N, int act, int use_weight) {
   constexpr int TM = 16 * MT;
+  constexpr bool GATED = MODE == MM_GATED, BY_TOKEN = MODE != MM_DOWN;
   if (tile_expert && (int)blockIdx.x >= meta[0]) return;
   __shared__ __attribute__((aligned(16))) bf16_t xs[TM * MM_S];
   __shared__ __attribute__((aligned(16))) bf16_t w0s[MM_T * MM_S];
@@ -46,7 +50,7 @@ moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const
 #pragma unroll
   for (int q = 0; q < XQ; ++q) {
     const int r = pr + 32 * q;
-    const long long src = GATED ? (long long)(ent[r] / top) : (long long)(row0 + min(r, rows - 1));
+    const long long src = BY_TOKEN ? (long long)(ent[r] / top) : (long long)(row0 + min(r, rows - 1));
     xrow[q] = a_rows + src * K;
   }
 #pragma unroll
@@ -114,6 +118,11 @@ moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const
 #pragma unroll
       for (int c = 0; c < 4; ++c)
         if (nb + c < N) z[nb + c] = from_f32<bf16_t>(jv_gated(act, acc0[mt][c] * w, acc1[mt][c] * w));
+    } else if (MODE == MM_PLAIN) {
+      bf16_t* z = (bf16_t*)out + (long long)(row0 + m) * N;
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+        if (nb + c < N) z[nb + c] = from_f32<bf16_t>(jv_act(act, acc0[mt][c] * w));
     } else {
       const int token = s / top, kk = s - token * top;
       float* y = (float*)out + ((long long)kk * n_tokens + token) * N;
@@ -124,16 +133,16 @@ moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const
   }
 }
 
-template <bool GATED>
+template <int MODE>
 static int launch_moe_mfma(int tile_rows, dim3 grid, hipStream_t stream, void* out, const bf16_t* a, const bf16_t* W0,
                            const bf16_t* W1, const int* meta, const int* offsets, const int* tile_expert,
                            const int* tile_row0, const int* order, const float* weights, int top, int n_tokens, int K,
                            int N, int act, int use_weight) {
   if (tile_rows == 128)
-    hipLaunchKernelGGL((moe_mfma_kernel<GATED, 8>), grid, dim3(256), 0, stream, out, a, W0, W1, meta, offsets, tile_expert,
+    hipLaunchKernelGGL((moe_mfma_kernel<MODE, 8>), grid, dim3(256), 0, stream, out, a, W0, W1, meta, offsets, tile_expert,
                        tile_row0, order, weights, top, n_tokens, K, N, act, use_weight);
   else if (tile_rows == 64)
-    hipLaunchKernelGGL((moe_mfma_kernel<GATED, 4>), grid, dim3(256), 0, stream, out, a, W0, W1, meta, offsets, tile_expert,
+    hipLaunchKernelGGL((moe_mfma_kernel<MODE, 4>), grid, dim3(256), 0, stream, out, a, W0, W1, meta, offsets, tile_expert,
                        tile_row0, order, weights, top, n_tokens, K, N, act, use_weight);
   else
     return (int)hipErrorInvalidValue;
@@ -141,14 +150,18 @@ static int launch_moe_mfma(int tile_rows, dim3 grid, hipStream_t stream, void* o
 }
 
 // gate/up: x [tokens, hidden], Wg, Wu [experts, ff, hidden] -> z [entries, ff] bf16 by position; tile_rows (64 or
-// 128) is what the grouping was made with
+// 128) is what the grouping was made with.  Wg null: experts without a gate, act one that stands alone.
 extern "C" int jv_moe_gate_up_mfma_bf16(void* z, const void* x, const void* Wg, const void* Wu, const int* meta,
                                         const int* offsets, const int* tile_expert, const int* tile_row0,
                                         const int* order, const float* weights, int max_tiles, int top, int hidden,
                                         int ff, int act, int scale_input, int tile_rows, void* stream) {
   if (max_tiles <= 0 || ff <= 0) return 0;
-  if (!jv_act_known(act) || hidden < 8 || hidden % 8 || (ff + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
-  return launch_moe_mfma<true>(tile_rows, dim3(max_tiles, (ff + MM_T - 1) / MM_T), (hipStream_t)stream, z, (const bf16_t*)x,
+  if (!(Wg ? jv_act_known(act) : jv_plain_act_known(act)) || hidden < 8 || hidden % 8 || (ff + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
+  if (!Wg)
+    return launch_moe_mfma<MM_PLAIN>(tile_rows, dim3(max_tiles, (ff + MM_T - 1) / MM_T), (hipStream_t)stream, z,
+                                     (const bf16_t*)x, (const bf16_t*)Wu, nullptr, meta, offsets, tile_expert, tile_row0,
+                                     order, weights, top, 0, hidden, ff, act, scale_input);
+  return launch_moe_mfma<MM_GATED>(tile_rows, dim3(max_tiles, (ff + MM_T - 1) / MM_T), (hipStream_t)stream, z, (const bf16_t*)x,
                                (const bf16_t*)Wg, (const bf16_t*)Wu, meta, offsets, tile_expert, tile_row0, order,
                                weights, top, 0, hidden, ff, act, scale_input);
 }
@@ -160,7 +173,7 @@ extern "C" int jv_moe_down_mfma_bf16(float* y, const void* z, const void* Wd, co
                                      int scale_output, int tile_rows, void* stream) {
   if (max_tiles <= 0 || hidden <= 0) return 0;
   if (ff < 8 || ff % 8 || (hidden + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
-  return launch_moe_mfma<false>(tile_rows, dim3(max_tiles, (hidden + MM_T - 1) / MM_T), (hipStream_t)stream, y,
+  return launch_moe_mfma<MM_DOWN>(tile_rows, dim3(max_tiles, (hidden + MM_T - 1) / MM_T), (hipStream_t)stream, y,
                                 (const bf16_t*)z, (const bf16_t*)Wd, nullptr, meta, offsets, tile_expert, tile_row0, order,
                                 weights, top, n_tokens, ff, hidden, 0, scale_output);
 }
@@ -170,6 +183,6 @@ extern "C" int jv_moe_down_mfma_bf16(float* y, const void* z, const void* Wd, co
 extern "C" int jv_gemm_rows_f32out_bf16(float* y, const void* x, const void* W, int M, int N, int K, void* stream) {
   if (M <= 0 || N <= 0) return 0;
   if (K < 8 || K % 8 || (N + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
-  return launch_moe_mfma<false>(128, dim3((M + 127) / 128, (N + MM_T - 1) / MM_T), (hipStream_t)stream, y, (const bf16_t*)x,
+  return launch_moe_mfma<MM_DOWN>(128, dim3((M + 127) / 128, (N + MM_T - 1) / MM_T), (hipStream_t)stream, y, (const bf16_t*)x,
                                 (const bf16_t*)W, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 1, M, K, N, 0, 0);
 }

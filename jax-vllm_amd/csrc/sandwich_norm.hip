@@ -88,14 +88,24 @@ template <typename T> __device__ __forceinline__ void sn_store4(T* p, float4 v) 
 }
 template <> __device__ __forceinline__ void sn_store4<float>(float* p, float4 v) { *(float4*)p = v; }
 
+// A causal filter over time behind the next norm, for steps with one token a request (row i is request i): with
+// x the normed row, out = x + sum_j wt[lags - j] * (the input j tokens back), the last `lags` inputs read from and left
+// in the request's state row [lags][hidden] (token_filter.hip has the form for any step).
+struct SnFilter {
+  const float* wt;         // [lags + 1][hidden]
+  float* state;            // [slots + 1][lags][hidden]
+  const int* slot_ids;
+  int lags;
+};
+
 #define SN_V 4      // 16-byte pieces a thread: rows of up to 4 * SN_V * 256 = 4,096 floats
-template <typename T>
+template <typename T, bool FILTER>
 __global__ void __launch_bounds__(256)
 postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, const float* __restrict__ parts,
                                 int n_parts, long long part_stride, const float* __restrict__ bias,
                                 const float* __restrict__ wb,
                                 const float* __restrict__ w, T* __restrict__ out, const int* __restrict__ rows,
-                                int hidden, float eps, float eps_out, float plain_scale) {
+                                int hidden, float eps, float eps_out, float plain_scale, SnFilter f) {
   __shared__ float red[32];
   const long long i = blockIdx.x;
   const long long r = rows ? (long long)rows[i] : i;
@@ -157,7 +167,22 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
     const int c = (threadIdx.x + q * 256) * 4;
     if (c < hidden) {
       const float4 g = *(const float4*)(w + c);
-      sn_store4<T>(out + i * hidden + c, float4{x[q].x * inv * g.x, x[q].y * inv * g.y, x[q].z * inv * g.z, x[q].w * inv * g.w});
+      const float4 o = float4{x[q].x * inv * g.x, x[q].y * inv * g.y, x[q].z * inv * g.z, x[q].w * inv * g.w};
+      if constexpr (FILTER) {
+        // the input in the activation type, as a later step reads it
+        const float4 u = float4{to_f32(from_f32<T>(o.x)), to_f32(from_f32<T>(o.y)), to_f32(from_f32<T>(o.z)), to_f32(from_f32<T>(o.w))};
+        float* st = f.state + (long long)f.slot_ids[r] * f.lags * hidden + c;
+        float4 acc = float4{0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j <= f.lags; ++j) {
+          const float4 in = j < f.lags ? *(const float4*)(st + (long long)j * hidden) : u;
+          const float4 k = *(const float4*)(f.wt + (long long)j * hidden + c);
+          acc = float4{fmaf(k.x, in.x, acc.x), fmaf(k.y, in.y, acc.y), fmaf(k.z, in.z, acc.z), fmaf(k.w, in.w, acc.w)};
+          if (j > 0) *(float4*)(st + (long long)(j - 1) * hidden) = in;
+        }
+        sn_store4<T>(out + i * hidden + c, float4{acc.x + u.x, acc.y + u.y, acc.z + u.z, acc.w + u.w});
+      } else {
+        sn_store4<T>(out + i * hidden + c, o);
+      }
     }
   }
 }
@@ -172,15 +197,29 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
     if (n_out <= 0 || hidden <= 0) return 0;                                                             \
     if ((!y && n_parts <= 0) || hidden > 16384) return (int)hipErrorInvalidValue;                        \
     if (hidden % 4 == 0 && hidden <= 4 * SN_V * 256) {                                                   \
-      hipLaunchKernelGGL(postnorm_add_rmsnorm_vec_kernel<T>, dim3(n_out), dim3(256), 0,                  \
+      hipLaunchKernelGGL((postnorm_add_rmsnorm_vec_kernel<T, false>), dim3(n_out), dim3(256), 0,         \
                          (hipStream_t)stream, h, (const T*)y, parts, n_parts, part_stride, bias, wb, w,  \
-                         (T*)out, rows, hidden, eps, eps_out, plain_scale);                              \
+                         (T*)out, rows, hidden, eps, eps_out, plain_scale, SnFilter{});                  \
       return JV_LAUNCH_CHECK();                                                                          \
     }                                                                                                    \
     hipLaunchKernelGGL(postnorm_add_rmsnorm_kernel<T>, dim3(n_out), dim3(256), hidden * sizeof(float),   \
                        (hipStream_t)stream, h, (const T*)y, parts, n_parts, part_stride, bias, wb, w,    \
                        (T*)out,                                                                          \
                        rows, hidden, eps, eps_out, plain_scale);                                         \
+    return JV_LAUNCH_CHECK();                                                                            \
+  }                                                                                                      \
+  extern "C" int jv_norm_filter_##SUF(float* h, const void* y, const float* parts, int n_parts,           \
+                                      long long part_stride, const float* wb, const float* w, void* out,  \
+                                      int n, int hidden, float eps, float eps_out, const float* wt,        \
+                                      float* state, const int* slot_ids, int taps, void* stream) {         \
+    if (n <= 0 || hidden <= 0) return 0;                                                                 \
+    if (hidden % 4 || hidden > 4 * SN_V * 256 || !w || !out || !wt || taps < 1 ||                        \
+        (taps > 1 && (!state || !slot_ids)))                                                             \
+      return (int)hipErrorInvalidValue;                                                                  \
+    hipLaunchKernelGGL((postnorm_add_rmsnorm_vec_kernel<T, true>), dim3(n), dim3(256), 0,                \
+                       (hipStream_t)stream, h, (const T*)y, parts, n_parts, part_stride,                 \
+                       (const float*)nullptr, wb, w, (T*)out, (const int*)nullptr, hidden, eps, eps_out,  \
+                       1.f, SnFilter{wt, state, slot_ids, taps - 1});                                    \
     return JV_LAUNCH_CHECK();                                                                            \
   }                                                                                                      \
   extern "C" int jv_gated_rmsnorm_##SUF(void* out, const float* o, const void* g, long long g_stride,    \

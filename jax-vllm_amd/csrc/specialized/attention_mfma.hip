@@ -63,6 +63,15 @@ struct PageSplit {
   __device__ __forceinline__ int slot(int j) const { return shift >= 0 ? (j & (P - 1)) : j % P; }
 };
 
+// The first key that the query at position `pos` sees: all of them (0), the last `window` (> 0), or those of its
+// own block of -window positions counted from position 0 (< 0).  It never falls as pos rises, so a group of rows
+// begins at its first row's first key, and from its last row's on every row sees every key up to itself.
+__device__ __forceinline__ int first_key(int pos, int window) {
+  if (window == 0) return 0;
+  if (window < 0) return pos - pos % -window;
+  return pos - window + 1 > 0 ? pos - window + 1 : 0;
+}
+
 struct AttnArgs {
   bf16_t* out;                // [tokens, nq * D]
   const bf16_t* q;            // row t at q + t * q_row_stride, head h at + h * D
@@ -76,7 +85,7 @@ struct AttnArgs {
   const int* work;            // prefill: [n_work][3] = (request, first row of group 0, first row of group 1 or -1); decode: [n_work] = request
   int page_size, page_shift, nq, nkv;   // page_shift: log2(page_size) or -1
   float scale_log2;           // softmax scale * log2(e)
-  int window;                 // <= 0: none
+  int window;                 // which keys a row sees, see first_key()
   const float* sinks;         // [nq] or null: exp(sinks[h]) joins every row's softmax denominator (no key, no value, unscaled)
   // decode only
   int num_splits;
@@ -131,7 +140,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
 
   // this lane's rows (one per group), and per group the key ranges of the block and of the wave
-  int qi[RT], hg[RT], pos[RT];
+  int qi[RT], hg[RT], pos[RT], row_first[RT];
   bool row_ok[RT];
   bf16x8 qf[RT][NKS];
   int blk_begin[RT], blk_end[RT];          // keys [begin, end) some row of the block's group sees; empty if no group
@@ -146,6 +155,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
     qi[t] = row_ok[t] ? row / G : 0;
     hg[t] = row_ok[t] ? row - qi[t] * G : 0;
     pos[t] = ctx + qi[t];
+    row_first[t] = first_key(pos[t], p.window);
     const bf16_t* qrow = p.q + (long long)(q_start + qi[t]) * p.q_row_stride + (long long)(g * G + hg[t]) * D;
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks) {
@@ -156,10 +166,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
     if (m0 >= 0 && m0 < M) {
       const int last_row = (M < m0 + GROUP_ROWS ? M : m0 + GROUP_ROWS) - 1;
       blk_end[t] = ctx + last_row / G + 1;
-      if (p.window > 0) {
-        blk_begin[t] = ctx + m0 / G - p.window + 1;
-        if (blk_begin[t] < 0) blk_begin[t] = 0;
-      }
+      blk_begin[t] = first_key(ctx + m0 / G, p.window);
     }
     const int wave_first = m0 + wave * 16;
     wave_live[t] = m0 >= 0 && wave_first < M;
@@ -167,11 +174,9 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
     wave_kv_end[t] = wave_live[t] ? ctx + wave_last / G + 1 : 0;
     wave_min_pos[t] = ctx + wave_first / G;
     wave_kv_begin[t] = wave_full_begin[t] = 0;
-    if (p.window > 0 && wave_live[t]) {
-      wave_kv_begin[t] = wave_min_pos[t] - p.window + 1;
-      if (wave_kv_begin[t] < 0) wave_kv_begin[t] = 0;
-      wave_full_begin[t] = ctx + wave_last / G - p.window + 1;
-      if (wave_full_begin[t] < 0) wave_full_begin[t] = 0;
+    if (wave_live[t]) {
+      wave_kv_begin[t] = first_key(wave_min_pos[t], p.window);
+      wave_full_begin[t] = first_key(ctx + wave_last / G, p.window);
     }
   }
   // The tiles the block walks: those of the one range, or of the union of the two; when a window
@@ -386,7 +391,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
     for (int t = 0; t < RT; ++t) {
       if (!((MASK >> t) & 1)) continue;
       // interior tile: every key visible to every row of the tile -> no per-element mask
-      const bool interior = (j0 + BN - 1 <= wave_min_pos[t]) && (p.window <= 0 || j0 >= wave_full_begin[t]);
+      const bool interior = (j0 + BN - 1 <= wave_min_pos[t]) && j0 >= wave_full_begin[t];
       float tmax = -INFINITY;
       // the maximum is taken over raw scores (the scale is positive); the scale enters in the
       // exponent's multiply-add: p = exp2(s * scale_log2 - m * scale_log2)
@@ -401,7 +406,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
             const int j = j0 + kt * 16 + lc * 4 + e;
-            const bool ok = row_ok[t] && j <= pos[t] && (p.window <= 0 || j > pos[t] - p.window);
+            const bool ok = row_ok[t] && j <= pos[t] && j >= row_first[t];
             const float v = ok ? s[t][kt][e] : -INFINITY;
             s[t][kt][e] = v;
             tmax = fmaxf(tmax, v);
@@ -563,10 +568,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     if (m0 >= 0 && m0 < M) {
       const int last_row = (M < m0 + 64 ? M : m0 + 64) - 1;
       blk_end[t] = ctx + last_row / G + 1;
-      if (p.window > 0) {
-        blk_begin[t] = ctx + m0 / G - p.window + 1;
-        if (blk_begin[t] < 0) blk_begin[t] = 0;
-      }
+      blk_begin[t] = first_key(ctx + m0 / G, p.window);
     }
   }
   // ---- this wave's tile of 32 rows and this lane's row
@@ -577,16 +579,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
   const int wave_kv_end = wave_live ? ctx + wave_last / G + 1 : 0;
   const int wave_min_pos = ctx + wave_first / G;
   int wave_kv_begin = 0, wave_full_begin = 0;
-  if (p.window > 0 && wave_live) {
-    wave_kv_begin = wave_min_pos - p.window + 1;
-    if (wave_kv_begin < 0) wave_kv_begin = 0;
-    wave_full_begin = ctx + wave_last / G - p.window + 1;
-    if (wave_full_begin < 0) wave_full_begin = 0;
+  if (wave_live) {
+    wave_kv_begin = first_key(wave_min_pos, p.window);
+    wave_full_begin = first_key(ctx + wave_last / G, p.window);
   }
   const int row = wave_first + l32;
   const bool row_ok = wave_live && row < M;
   const int qi = row_ok ? row / G : 0, hg = row_ok ? row - qi * G : 0;
-  const int pos = ctx + qi;
+  const int pos = ctx + qi, row_first = first_key(pos, p.window);
   bf16x8 qf[NQS];                          // B operand: row l32, head elements 16 ks + 8 h .. + 7
   {
     const bf16_t* qrow = p.q + (long long)(q_start + qi) * p.q_row_stride + (long long)(g * G + hg) * D + h * 8;
@@ -793,7 +793,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     read_v(0, vf[0]);                    // on its way during the softmax
     __builtin_amdgcn_sched_barrier(0);
     // interior tile: every key visible to every row of the tile -> no per-element mask
-    const bool interior = (j0 + BN - 1 <= wave_min_pos) && (p.window <= 0 || j0 >= wave_full_begin);
+    const bool interior = (j0 + BN - 1 <= wave_min_pos) && j0 >= wave_full_begin;
     float tmax = -INFINITY;
     if (interior) {
 #pragma unroll
@@ -806,7 +806,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int j = j0 + kb * 32 + acc_key(e);
-          const bool ok = row_ok && j <= pos && (p.window <= 0 || j > pos - p.window);
+          const bool ok = row_ok && j <= pos && j >= row_first;
           const float v = ok ? s[kb][e] : -INFINITY;
           s[kb][e] = v;
           tmax = fmaxf(tmax, v);
@@ -886,7 +886,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     };
     // the row's maximum over the tile, the new reference if it has grown; returns whether any row of the wave moved
     auto row_max = [&](f32x16 (&sc)[2], int j0, float& alpha) -> bool {
-      const bool interior = (j0 + BN - 1 <= wave_min_pos) && (p.window <= 0 || j0 >= wave_full_begin);
+      const bool interior = (j0 + BN - 1 <= wave_min_pos) && j0 >= wave_full_begin;
       float tmax = -INFINITY;
       if (interior) {
 #pragma unroll
@@ -899,7 +899,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
 #pragma unroll
           for (int e = 0; e < 16; ++e) {
             const int j = j0 + kb * 32 + acc_key(e);
-            const bool ok = row_ok && j <= pos && (p.window <= 0 || j > pos - p.window);
+            const bool ok = row_ok && j <= pos && j >= row_first;
             const float v = ok ? sc[kb][e] : -INFINITY;
             sc[kb][e] = v;
             tmax = fmaxf(tmax, v);
@@ -1146,8 +1146,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(Attn
   const int tok = p.cu_seqlens ? p.cu_seqlens[r] : r;
   const int pos = p.context_lens[r];      // the query's position; keys 0..pos are stored
   const int kv_len = pos + 1;
-  int kv_begin = 0;
-  if (p.window > 0 && pos - p.window + 1 > 0) kv_begin = pos - p.window + 1;
+  const int kv_begin = first_key(pos, p.window);
 
   const int hg = mt * 16 + li;
   const bool row_ok = hg < G;

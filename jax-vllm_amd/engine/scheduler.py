@@ -73,7 +73,7 @@ class Scheduler:
             raise ValueError("prompt+max_new exceeds max_model_len")
         total_pages = -(-(n + request.sampling.max_new_tokens) // cfg.page_size)
         for g in self.cache.groups:
-            if g.window is None and total_pages > g.pool.num_pages:
+            if g.keeps_all and total_pages > g.pool.num_pages:
                 raise ValueError(
                     f"request needs {total_pages} pages at full length, the pool has {g.pool.num_pages}"
                 )

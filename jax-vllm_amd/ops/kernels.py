@@ -199,7 +199,7 @@ def add_bias(y: torch.Tensor, bias: torch.Tensor) -> None:
     _check(fn(_ptr(rows), _ptr(bias), c_longlong(rows.shape[0]), c_int(rows.shape[1]), _stream()), "add_bias")
 
 
-PLAIN_ACTIVATIONS = {None: 0, "silu": 1, "gelu_tanh": 2, "gelu": 3, "tanh": 4}     # ids of act in y = act(x + bias); "gelu" is the erf form
+PLAIN_ACTIVATIONS = {None: 0, "silu": 1, "gelu_tanh": 2, "gelu": 3, "tanh": 4, "relu2": 5}     # ids of act in y = act(x + bias); "gelu" is the erf form, "relu2" max(z, 0)^2
 
 
 def bias_act(y: torch.Tensor, bias, activation) -> None:
@@ -477,10 +477,137 @@ def attn_prepare_wide(qkv, bias, q_weight, k_weight, eps: float, cos_sin, rot_di
     return q
 
 
+# --------------------------------------------------------------------------- causal filters over time
+def token_filter_max_taps() -> int:
+    return library.core().jv_token_filter_max_taps()
+
+
+def _filter_ok(weight_t, state, channels: int, what: str) -> int:
+    """Checks a filter's weights [taps, channels] and state [slots + 1, taps - 1, channels]; returns the taps."""
+    _need(weight_t.dim() == 2 and weight_t.shape[1] == channels, f"{what}: weights must be [taps, channels]")
+    taps = weight_t.shape[0]
+    _f32(weight_t, what)
+    _need(1 <= taps <= token_filter_max_taps(), f"{what}: a filter of {taps} taps, the kernels take up to {token_filter_max_taps()}")
+    if taps > 1:
+        _f32(state, what)
+        _need(state.dim() == 3 and tuple(state.shape[1:]) == (taps - 1, channels), f"{what}: the state must be [slots, taps - 1, channels]")
+    return taps
+
+
+def token_filter(x: torch.Tensor, weight_t: torch.Tensor, state, slot_ids, cu_seqlens, max_q_len: int) -> torch.Tensor:
+    """x plus its causal filter over time per channel, request by request, in x's type (float arithmetic): out[t] = x[t] +
+    sum_j weight_t[j] x[t - taps + 1 + j].  ``weight_t`` float32 [taps, channels]; ``state`` float32 [slots + 1, taps - 1,
+    channels] holds every request's last inputs before the step and after it (zeros before a sequence's start)."""
+    _dev(x, weight_t, state, slot_ids, cu_seqlens)
+    n, channels = x.shape
+    taps = _filter_ok(weight_t, state, channels, "token_filter")
+    r = slot_ids.numel()
+    _i32(slot_ids, "slot_ids")
+    _i32(cu_seqlens, "cu_seqlens", r + 1)
+    out = torch.empty_like(x)
+    fn = getattr(library.core(), f"jv_token_filter_{_suffix(x.dtype)}")
+    _check(fn(_ptr(out), _ptr(x), c_int(channels), c_int(taps), _ptr(weight_t), _ptr(state), _ptr(slot_ids), _ptr(cu_seqlens),
+              c_int(r), c_int(int(max_q_len)), _stream()), "token_filter")
+    return out
+
+
+def norm_filter_possible(hidden: int) -> bool:
+    return hidden % 4 == 0 and hidden <= 4096
+
+
+def norm_filter(h, pending: "PendingNorm | None", weight, eps: float, weight_t, state, slot_ids, dtype) -> torch.Tensor:
+    """For a step with one token per request (row i is request i): what ``postnorm_add_rmsnorm`` and then ``token_filter``
+    do, in one launch.  ``pending`` None: nothing joins the stream."""
+    y, parts = (pending.y, pending.parts) if pending is not None else (None, None)
+    post = pending.weight if pending is not None else None
+    _need(pending is None or (post is not None and pending.bias is None), "a sublayer's output under its own norm, without a bias")
+    _dev(h, y, parts, post, weight, weight_t, state, slot_ids)
+    _f32(h, "h")
+    n, hidden = h.shape
+    _need(norm_filter_possible(hidden), "rows of a multiple of 4, at most 4,096 columns")
+    _f32(weight, "weight", hidden)
+    if post is not None:
+        _f32(post, "post_weight", hidden)
+    if y is not None:
+        _need(y.shape == h.shape and y.dtype == dtype, "y must match h's shape and the output's type")
+    if parts is not None:
+        _need(parts.dtype == torch.float32 and parts.dim() == 3 and parts.shape[1:] == h.shape and parts.stride(0) % 4 == 0,
+              "parts must be float32 [P, *h.shape]")
+    taps = _filter_ok(weight_t, state, hidden, "norm_filter")
+    _i32(slot_ids, "slot_ids", n)
+    out = torch.empty((n, hidden), dtype=dtype, device=h.device)
+    fn = getattr(library.core(), f"jv_norm_filter_{_suffix(dtype)}")
+    _check(fn(_ptr(h), _ptr(y), _ptr(parts), c_int(0 if parts is None else parts.shape[0]),
+              c_longlong(0 if parts is None else parts.stride(0)), _ptr(post), _ptr(weight), _ptr(out), c_int(n), c_int(hidden),
+              c_float(pending.eps if pending is not None else 0.0), c_float(eps), _ptr(weight_t), _ptr(state), _ptr(slot_ids),
+              c_int(taps), _stream()), "norm_filter")
+    return out
+
+
+def attn_prepare_filtered(qkv, weight_t, state, slot_ids, cu_seqlens, context_lens, max_q_len: int, k_cos_sin, rot_dims: int,
+                          v_cos_sin, slot_mapping, k_pages, v_pages, page_size: int, nq: int, nkv: int, dk: int, dv: int,
+                          dp: int) -> torch.Tensor:
+    """Attention input from rows that begin with [q: nq * dk | k: nkv * dk | v: nkv * dv]: every channel through its
+    causal filter (``weight_t`` float32 [taps, channels] with ``state`` as in ``token_filter``, or None: no filter), the
+    pairs (2i, 2i + 1) of the first ``rot_dims`` elements of every q and k head turned by ``k_cos_sin``, those of all of
+    every v head by ``v_cos_sin`` (float32 [n, dv], or None).  Returns q as [n, nq * dp], heads padded with zeros to
+    ``dp``; keys go to [pages, nkv, page_size, dp], values to [pages, nkv, dp, page_size] (their pad is never written)."""
+    _dev(qkv, weight_t, state, slot_ids, cu_seqlens, context_lens, k_cos_sin, v_cos_sin, slot_mapping, k_pages, v_pages)
+    n, ld = qkv.shape
+    channels = (nq + nkv) * dk + nkv * dv
+    _need(ld >= channels, "qkv rows must begin with nq * dk + nkv * dk + nkv * dv columns")
+    _need(dk % 2 == 0 and dv % 2 == 0 and ld % 2 == 0, "head sizes and rows of an even length")
+    taps = _filter_ok(weight_t, state, channels, "attn_prepare_filtered") if weight_t is not None else 1
+    r = slot_ids.numel()
+    _i32(slot_ids, "slot_ids")
+    _i32(cu_seqlens, "cu_seqlens", r + 1)
+    _i32(context_lens, "context_lens", r)
+    _need(rot_dims % 2 == 0 and 0 <= rot_dims <= dk, "the rotated size must be even and at most the key size")
+    if rot_dims:
+        _f32(k_cos_sin, "k_cos_sin", n * rot_dims)
+    if v_cos_sin is not None:
+        _f32(v_cos_sin, "v_cos_sin", n * dv)
+    _need(dp >= max(dk, dv) and dp % 2 == 0, "the padded head size must hold keys and values")
+    _i32(slot_mapping, "slot_mapping", n)
+    _check_pages(k_pages, v_pages, qkv.dtype, nkv, page_size, dp)
+    q = torch.empty((n, nq * dp), dtype=qkv.dtype, device=qkv.device)
+    fn = getattr(library.core(), f"jv_attn_prepare_filtered_{_suffix(qkv.dtype)}")
+    _check(fn(_ptr(q), _ptr(qkv), c_longlong(ld), c_int(taps), _ptr(weight_t), _ptr(state if taps > 1 else None), _ptr(slot_ids),
+              _ptr(cu_seqlens), _ptr(context_lens), _ptr(k_cos_sin if rot_dims else None), c_int(rot_dims), _ptr(v_cos_sin),
+              _ptr(slot_mapping), _ptr(k_pages), _ptr(v_pages), c_int(page_size), c_int(r), c_int(int(max_q_len)), c_int(nq),
+              c_int(nkv), c_int(dk), c_int(dv), c_int(dp), _stream()), "attn_prepare_filtered")
+    return q
+
+
+def rotate_back_gate(o: torch.Tensor, gate, v_cos_sin, heads: int, dv: int, dp: int) -> None:
+    """In place on o [n, heads * dp]: the pairs (2m, 2m + 1) of every head's first dv elements turn back by ``v_cos_sin``
+    (float32 [n, dv] or None), then times sigmoid(gate[t, h * dv + i]) (``gate`` a [n, heads * dv] view with unit column
+    stride of o's type, or None)."""
+    _dev(o, v_cos_sin)
+    n = o.shape[0]
+    _need(o.shape == (n, heads * dp) and dp >= dv, "o must be [n, heads * dp]")
+    if v_cos_sin is not None:
+        _f32(v_cos_sin, "v_cos_sin", n * dv)
+    if gate is not None:
+        _need(gate.is_cuda and gate.dtype == o.dtype and gate.shape == (n, heads * dv) and (n == 0 or gate.stride(1) == 1),
+              "gate must be a [n, heads * dv] view with unit column stride")
+    fn = getattr(library.core(), f"jv_rotate_back_gate_{_suffix(o.dtype)}")
+    _check(fn(_ptr(o), _ptr(gate), c_longlong(0 if gate is None else gate.stride(0)), _ptr(v_cos_sin), c_longlong(n), c_int(heads),
+              c_int(dv), c_int(dp), _stream()), "rotate_back_gate")
+
+
 # --------------------------------------------------------------------------- attention
+def key_window(window: "int | None", chunk: "int | None") -> int:
+    """Which keys a query sees, in the one number the attention kernels take: 0 all up to itself, ``window`` > 0 the last
+    so many, -``chunk`` those of its own block of ``chunk`` positions, counted from position 0."""
+    _need(not (window and chunk), "a window or blocks, not both")
+    return -int(chunk) if chunk else int(window or 0)
+
+
 def paged_attention_generic(out, q, q_row_stride, k_pages, v_pages, block_tables, token_req, positions,
                             nq, nkv, head_dim, scale, window=0, sinks=None) -> None:
-    """Causal attention of every token over its request's pages (generic float-math kernel).
+    """Causal attention of every token over its request's pages (generic float-math kernel).  ``window``: 0 all earlier
+    keys, > 0 the last so many, < 0 those of the query's own block of -window positions (``key_window``).
 
     ``q`` is any tensor whose row t holds the q heads at [t * q_row_stride + h * D].  ``sinks`` (float32 [nq]):
     exp(sinks[h]) joins every row's softmax denominator (a term without key and value, not scaled)."""
@@ -883,7 +1010,7 @@ def attn_prefill_mfma(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_s
                       nq, nkv, head_dim, scale, window=0, sinks=None) -> None:
     """Causal attention of prompt portions.  ``work`` is int32 [n_work, 3]: (request index, first row
     of a group, first row of a second group of the same request or -1), see ``attn_prefill_geometry``;
-    every row of every request must be in exactly one group.  Pairing a group that sees many keys with
+    every row of every request must be in exactly one group.  ``window``: see ``key_window``.  Pairing a group that sees many keys with
     one that sees few gives all blocks the same amount of work.  ``sinks`` (float32 [nq]): exp(sinks[h]) joins every
     row's softmax denominator (a term without key and value, not scaled)."""
     _sinks_ok(sinks, nq)
@@ -1108,14 +1235,16 @@ def latent_prepare(proj, q_rank: int, rank: int, rot: int, rot_dims: int, q_weig
     """From rows ``proj`` = [q latent | kv latent | key part to rotate | ...]: returns the normed q latent
     [n, q_rank] (None for ``q_rank`` 0: queries that are projected directly; the kv latent then begins at column
     ``kv_off``, default ``q_rank``); ``interleaved``: the pairs (2i, 2i + 1) turn instead of (i, i + rot_dims / 2); stores [normed kv latent | rotated key part] of every token with a slot (>= 0) into its key
-    page [pages, 1, page_size, rank + rot] and transposed value page [pages, 1, rank + rot, page_size]."""
+    page (``rank`` 0 and no pages: the query latent alone, for a layer that reads another layer's cache) [pages, 1, page_size, rank + rot] and transposed value page [pages, 1, rank + rot, page_size]."""
     _dev(proj, q_weight, kv_weight, cos_sin, slot_mapping, k_pages, v_pages)
     n, ld = proj.shape
     kv_off = q_rank if kv_off is None else int(kv_off)
     _need(q_rank >= 0 and kv_off >= q_rank and ld >= kv_off + rank + rot, "proj rows are too short")
     if q_rank:
         _f32(q_weight, "q_weight", q_rank)
-    _f32(kv_weight, "kv_weight", rank)
+    if rank:
+        _f32(kv_weight, "kv_weight", rank)
+    _need(rank > 0 or k_pages is None, "nothing to store without a kv latent")
     _need(rot_dims % 2 == 0 and 0 <= rot_dims <= rot, "the rotated size must be even and at most the key part")
     if rot_dims:
         _f32(cos_sin, "cos_sin", n * rot_dims)
@@ -1602,18 +1731,21 @@ class MoePlan:
         self.tile_rows = tile_rows
 
 
-ROUTER_SCORES = {"sigmoid": 0, "softmax_chosen": 1, "sigmoid_normed": 2}      # the kernels' ids of how a chosen logit becomes a weight
+ROUTER_SCORES = {"sigmoid": 0, "softmax_chosen": 1, "sigmoid_normed": 2, "softmax": 3}      # the kernels' ids of how a chosen logit becomes a weight
+ROUTER_MAX_GROUPS = 64
 
 
 def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, logits_out=None,
               tile_rows: "int | None" = None, bias=None, score: str = "sigmoid", correction=None,
-              weight_scale: float = 1.0) -> MoePlan:
+              weight_scale: float = 1.0, groups: "tuple | None" = None) -> MoePlan:
     """Chooses for every token the ``top`` experts with the largest router logits (the lowest index among equal
     logits) and orders the n * top entries by expert, all on the device.  ``bias`` (float32 [experts]) is added
     to the logits before the choice; ``score``: a chosen expert's weight is "sigmoid" of its logit, or
     "softmax_chosen": the softmax over the token's chosen logits alone, or "sigmoid_normed": the experts with the
     largest sigmoid(logit) + ``correction`` (float32 [experts] or None) are chosen, and a chosen expert's weight is its
-    sigmoid(logit) (without the correction) over the sum of the chosen ones' (+ 1e-20), times ``weight_scale``.
+    sigmoid(logit) (without the correction) over the sum of the chosen ones' (+ 1e-20), times ``weight_scale``;
+    or "softmax": the softmax over ALL of the token's logits.  ``groups`` (count, keep): the experts form ``count`` equal
+    groups of neighbours, and only those of the ``keep`` groups with the largest logits can be chosen.
     Either float ``logits`` [n, experts] are given, or rows ``x`` [n, hidden] and the router matrix
     ``w_router`` [experts, hidden] of one type: then the logits are made here, in float (``logits_out``,
     float32 [n, experts], receives them if given): in the same launch as the choice (float32, odd sizes), or
@@ -1656,6 +1788,10 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     if correction is not None:
         _dev(correction)
         _f32(correction, "correction", experts)
+    count, keep = groups if groups else (1, 1)
+    _need(count == 1 or (experts % count == 0 and count <= ROUTER_MAX_GROUPS and 0 < keep <= count
+                         and keep * (experts // count) >= top and correction is None),
+          "equal groups (at most 64), enough experts in the kept ones, and no correction of the choice")
     entries = n * top
     tile_rows = tile_rows or moe_tile_rows()
     _need(tile_rows in (64, 128), "tiles have 64 or 128 rows")
@@ -1670,12 +1806,13 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     lib = library.core()
     if logits is not None:
         _check(lib.jv_moe_route(_ptr(logits), _ptr(bias), c_int(n), c_int(experts), c_int(top), c_int(ROUTER_SCORES[score]),
-                                _ptr(ids), _ptr(weights), _ptr(correction), c_float(weight_scale), _stream()), "moe_route")
+                                _ptr(ids), _ptr(weights), _ptr(correction), c_float(weight_scale), c_int(count), c_int(keep),
+                                _stream()), "moe_route")
     else:
         _check(getattr(lib, f"jv_moe_router_{_suffix(x.dtype)}")(
             _ptr(x), _ptr(w_router), _ptr(bias), c_int(n), c_int(hidden), c_int(experts), c_int(top),
             c_int(ROUTER_SCORES[score]), _ptr(ids), _ptr(weights), _ptr(logits_out), _ptr(correction),
-            c_float(weight_scale), _stream()), "moe_router")
+            c_float(weight_scale), c_int(count), c_int(keep), _stream()), "moe_router")
     _check(lib.jv_moe_group(_ptr(ids), c_int(entries), c_int(experts), c_int(tile_rows), _ptr(meta), _ptr(offsets), _ptr(tile_expert),
                             _ptr(tile_row0), _ptr(order), _ptr(rank), _stream()), "moe_group")
     return MoePlan(ids, weights, meta, offsets, tile_expert, tile_row0, order, max_tiles, top, tile_rows)
@@ -1701,14 +1838,21 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
                 weight_on_input: bool = True, matrix_cores: "bool | None" = None) -> None:
     """out[kk, t] = down[e] (act(gate[e] xs) * (up[e] xs)) for the kk-th chosen expert e of token t, float32
     [top, n, hidden]; xs = weight * x[t] with ``weight_on_input``, else x[t] and the result is multiplied
-    by the weight.  w_gate, w_up [experts, ff, hidden], w_down [experts, hidden, ff].  ``matrix_cores``:
+    by the weight.  ``w_gate`` None: experts without a gate, down[e] act(up[e] xs) with one of ``PLAIN_ACTIVATIONS``.
+    w_gate, w_up [experts, ff, hidden], w_down [experts, hidden, ff].  ``matrix_cores``:
     None takes the matrix-core kernels wherever ``moe_matrix_cores_possible``, False the float-FMA ones."""
     _dev(x, w_gate, w_up, w_down, out)
     n, hidden = x.shape
-    experts, ff, _ = w_gate.shape
-    _need(w_gate.shape == w_up.shape == (experts, ff, hidden) and w_down.shape == (experts, hidden, ff),
+    experts, ff, _ = w_up.shape
+    _need((w_gate is None or w_gate.shape == w_up.shape) and w_up.shape == (experts, ff, hidden) and w_down.shape == (experts, hidden, ff),
           "expert weights must be [experts, ff, hidden] and [experts, hidden, ff]")
-    _need(x.dtype == w_gate.dtype == w_up.dtype == w_down.dtype, "x and the weights must have one type")
+    if w_gate is not None:
+        act = _gate_act_id(activation)
+    else:
+        _need(activation in PLAIN_ACTIVATIONS and activation is not None, f"no kernel for the activation {activation!r}")
+        act = PLAIN_ACTIVATIONS[activation]
+    _need(w_gate is None or w_gate.dtype == x.dtype, "x and the weights must have one type")
+    _need(x.dtype == w_up.dtype == w_down.dtype, "x and the weights must have one type")
     _need(out.dtype == torch.float32 and tuple(out.shape) == (plan.top, n, hidden), "out must be float32 [top, n, hidden]")
     _need(plan.ids.numel() == n * plan.top, "the plan belongs to another step")
     z = torch.empty((n * plan.top, ff), dtype=x.dtype, device=x.device)
@@ -1722,7 +1866,7 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
         _check(lib.jv_moe_gate_up_mfma_bf16(
             _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),
             _ptr(p.tile_row0), _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(hidden), c_int(ff),
-            c_int(_gate_act_id(activation)), c_int(1 if weight_on_input else 0), c_int(p.tile_rows), _stream()), "moe_gate_up")
+            c_int(act), c_int(1 if weight_on_input else 0), c_int(p.tile_rows), _stream()), "moe_gate_up")
         _check(lib.jv_moe_down_mfma_bf16(
             _ptr(out), _ptr(z), _ptr(w_down), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert), _ptr(p.tile_row0),
             _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(n), c_int(hidden), c_int(ff),
@@ -1731,7 +1875,7 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
     _check(getattr(lib, f"jv_moe_gate_up_{suf}")(
         _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),
         _ptr(p.tile_row0), _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(hidden), c_int(ff),
-        c_int(_gate_act_id(activation)), c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
+        c_int(act), c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
     _check(getattr(lib, f"jv_moe_down_{suf}")(
         _ptr(out), _ptr(z), _ptr(w_down), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert), _ptr(p.tile_row0),
         _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(n), c_int(hidden), c_int(ff),

@@ -16,7 +16,7 @@ from typing import Optional
 import torch
 
 from ..ops import kernels as K
-from .spec import (LayerMemory, PagedCacheSpec, PartSpec, StepContext, TensorSpec, build_part, is_replayable,
+from .spec import (LayerMemory, PagedCacheSpec, PartSpec, StateSpec, StepContext, TensorSpec, build_part, is_replayable,
                    kv_cache_spec, register_part)
 
 
@@ -25,7 +25,9 @@ class GroupedQueryAttention:
                  qk_norm_eps: Optional[float] = None, position: Optional[PartSpec] = None,
                  window: Optional[int] = None, scale: Optional[float] = None, qkv_bias: bool = False,
                  o_bias: bool = False, v_head_dim: Optional[int] = None, qk_norm: str = "head", v_scale: float = 1.0,
-                 output_gate: bool = False, values_are_keys: bool = False, q_temperature: Optional[tuple] = None):
+                 output_gate: bool = False, values_are_keys: bool = False, q_temperature: Optional[tuple] = None,
+                 chunk: Optional[int] = None, filter_taps: Optional[int] = None, value_position: Optional[PartSpec] = None,
+                 softmax_plus_one: bool = False):
         """``v_head_dim``: a value size that differs from the key size; ``qk_norm`` "whole": the q/k norm spans all
         of q's (and all of k's) columns at once, with weights of that size, instead of every head on its own;
         ``v_scale``: a constant on the values (and so on the mixer's result before its output projection);
@@ -33,7 +35,14 @@ class GroupedQueryAttention:
         one more block of rows of the fused input projection);
         ``values_are_keys``: there is no value projection, the values are the keys as projected (before their norm and
         rotation); ``q_temperature`` (coef, every): the query at position p is multiplied by
-        1 + coef * ln(floor((p + 1) / every) + 1), after its norm.  Any of these takes the ``wide`` path: heads cached
+        1 + coef * ln(floor((p + 1) / every) + 1), after its norm;
+        ``chunk``: a token sees the keys of its own block of ``chunk`` positions only (counted from position 0);
+        ``filter_taps``: q, k and v as projected go through a causal filter over time per channel before the rotation,
+        y_t = sum_j w[:, j] u_(t - taps + 1 + j) (the last taps - 1 projected rows are the request's state ``filter``);
+        ``value_position``: a rotation of the whole value heads by their token's position, cached so, and every head's
+        result turned back by the query's position (before the gate): the weighted sum sees the values at their
+        distance from the query; ``softmax_plus_one``: one is added to the softmax denominator (a sink of score 0).
+        Any of these but ``chunk`` and ``softmax_plus_one`` takes the ``wide`` path: heads cached
         under one padded size (``K.padded_head_dim``), prepared by ``K.attn_prepare_wide``, read by the same paged
         attention kernels."""
         if num_heads % num_kv_heads:
@@ -51,7 +60,22 @@ class GroupedQueryAttention:
             raise ValueError("the period of a query temperature must be positive")
         if self.values_are_keys and (self.dv != self.dk or qkv_bias or (qk_norm == "whole" and qk_norm_eps is not None)):
             raise ValueError("values that are the keys: one head size, no input bias, a per-head q/k norm or none")
-        self.wide = (self.values_are_keys or self.q_temperature is not None or self.dv != self.dk or (qk_norm == "whole" and qk_norm_eps is not None) or self.v_scale != 1.0
+        self.chunk = int(chunk) if chunk else None
+        if self.chunk and window:
+            raise ValueError("a window or blocks, not both")
+        self.taps = int(filter_taps) if filter_taps else 0
+        self.plus_one = bool(softmax_plus_one)
+        self.value_position = build_part("position", value_position) if value_position is not None else None
+        self.filtered = bool(self.taps or self.value_position is not None)
+        if self.filtered and (self.values_are_keys or self.q_temperature is not None or qk_norm_eps is not None or qkv_bias
+                              or self.v_scale != 1.0):
+            raise ValueError("filters and turned values: without a q/k norm, biases, values taken from the keys, a constant "
+                             "on the values or a query temperature")
+        if self.value_position is not None:
+            turn = self.value_position.as_rotation()
+            if turn is None or turn != (self.dv, True):
+                raise ValueError("values turn whole, in pairs (2m, 2m + 1)")
+        self.wide = (self.filtered or self.values_are_keys or self.q_temperature is not None or self.dv != self.dk or (qk_norm == "whole" and qk_norm_eps is not None) or self.v_scale != 1.0
                      or self.output_gate)
         # what the paged attention kernels see
         self.d = K.padded_head_dim(self.dk, self.dv) if self.wide else self.dk
@@ -64,8 +88,10 @@ class GroupedQueryAttention:
         # what the position part asks of this mixer's kernels: a rotation of q and k by position
         # (rotary_dim, interleaved), or nothing (a part that acts elsewhere, or no part at all)
         self.rotation = self.position.as_rotation() if self.position is not None else None
+        if self.filtered and (self.dk % 2 or self.dv % 2 or (self.rotation is not None and not self.rotation[1])):
+            raise ValueError("the filtered attention input takes even head sizes and turns pairs (2i, 2i + 1)")
         self.qkv_bias, self.o_bias = bool(qkv_bias), bool(o_bias)
-        self.w_qkv = self.w_o = self.q_norm = self.k_norm = self.b_qkv = self.b_o = None
+        self.w_qkv = self.w_o = self.q_norm = self.k_norm = self.b_qkv = self.b_o = self.sinks = None
 
     # ---- declarations
     @property
@@ -73,7 +99,7 @@ class GroupedQueryAttention:
         """The kernels take positions, lengths and tables from the device; the host plan of a
         captured step (how many blocks share a request's keys) is made for the upper bound of
         the context lengths and is right for every shorter one."""
-        return self.position is None or is_replayable(self.position)
+        return all(part is None or is_replayable(part) for part in (self.position, self.value_position))
 
     def tensors(self) -> dict:
         t = {
@@ -96,13 +122,19 @@ class GroupedQueryAttention:
             t["o_proj.bias"] = TensorSpec((self.hidden_size,), role="vector")
         if self.output_gate:
             t["gate.weight"] = TensorSpec((self.nq * self.dv, self.hidden_size))
+        if self.taps:
+            t["q_filter.weight"] = TensorSpec((self.nq * self.dk, self.taps), role="vector")
+            t["k_filter.weight"] = TensorSpec((self.nkv * self.dk, self.taps), role="vector")
+            t["v_filter.weight"] = TensorSpec((self.nkv * self.dv, self.taps), role="vector")
         return t
 
     def cache_spec(self) -> Optional[PagedCacheSpec]:
-        return kv_cache_spec(self.nkv, self.d, self.window)
+        return kv_cache_spec(self.nkv, self.d, self.window, self.chunk)
 
     def state_spec(self):
-        return None
+        if not self.taps:
+            return None
+        return StateSpec((self.taps - 1, self.nq * self.dk + self.nkv * (self.dk + self.dv)), "float32", "filter")
 
     def bind(self, tensors: dict, dtype: torch.dtype) -> None:
         self.dtype = dtype
@@ -112,7 +144,13 @@ class GroupedQueryAttention:
             blocks.append(tensors["v_proj.weight"])
         if self.output_gate:
             blocks.append(tensors["gate.weight"])
+        rows = sum(b.shape[0] for b in blocks)
+        if self.filtered and rows % 8:      # rows of the product stay 16-byte aligned for the kernels that read heads out of them
+            blocks.append(blocks[0].new_zeros((8 - rows % 8, self.hidden_size)))
         self.w_qkv = torch.cat(blocks, dim=0).contiguous()
+        self.filters = (torch.cat([tensors[f"{s}_filter.weight"] for s in "qkv"], dim=0).t().contiguous()
+                        if self.taps else None)       # [taps, channels]
+        self.sinks = torch.zeros((self.nq,), dtype=torch.float32, device=self.w_qkv.device) if self.plus_one else None
         self.qkv_width = self.nq * self.dk + self.nkv * (self.dk + (0 if self.values_are_keys else self.dv))
         self.w_o = tensors["o_proj.weight"]
         if self.wide and self.d != self.dv:
@@ -128,6 +166,8 @@ class GroupedQueryAttention:
             self.b_o = tensors["o_proj.bias"].contiguous()
         if self.position is not None:
             self.position.bind({}, dtype, self.w_o.device)
+        if self.value_position is not None:
+            self.value_position.bind({}, dtype, self.w_o.device)
 
     def _qkv_parts_ok(self) -> bool:
         """Whether the kernel behind the qkv product (norm, rotation, page write) adds float partial
@@ -150,6 +190,8 @@ class GroupedQueryAttention:
         # at few rows the projection may come as float partial products, which the next kernel adds
         qkv = K.linear(x, self.w_qkv, partial_max_width=None,       # the rotation kernel adds parts of any width
                        partial_ok=self._qkv_parts_ok())
+        if self.filtered:
+            return self._forward_filtered(qkv, ctx, mem, cos_sin, rotary_dim)
         if self.wide:
             return self._forward_wide(qkv, ctx, mem, cos_sin, rotary_dim, interleaved)
         if self.b_qkv is not None:
@@ -173,6 +215,26 @@ class GroupedQueryAttention:
             K.add_bias(y, self.b_o)
         return y
 
+
+    def _forward_filtered(self, qkv, ctx: StepContext, mem: LayerMemory, cos_sin, rotary_dim: int):
+        if not mem.writes:
+            raise ValueError("filtered heads write the cache they declare")
+        v_turn = self.value_position.rotation_table(ctx) if self.value_position is not None else None
+        q = K.attn_prepare_filtered(
+            qkv, self.filters, mem.states.get("filter"), ctx.slot_ids, ctx.cu_seqlens, ctx.context_lens, ctx.max_q_len, cos_sin,
+            rotary_dim, v_turn, ctx.slot_mappings[mem.group], mem.pages["k"], mem.pages["v"], ctx.page_size, self.nq, self.nkv,
+            self.dk, self.dv, self.d)
+        out = torch.empty((qkv.shape[0], self.nq * self.d), dtype=qkv.dtype, device=qkv.device)
+        from . import attention_backend
+
+        attention_backend.run(self, out, q, ctx, mem)
+        gate = qkv[:, self.qkv_width:self.qkv_width + self.nq * self.dv] if self.output_gate else None
+        if v_turn is not None or gate is not None:
+            K.rotate_back_gate(out, gate, v_turn, self.nq, self.dv, self.d)
+        y = K.linear(out, self.w_o, partial_ok=True)
+        if self.b_o is not None:
+            K.add_bias(y, self.b_o)
+        return y
 
     def _forward_wide(self, qkv, ctx: StepContext, mem: LayerMemory, cos_sin, rotary_dim: int, interleaved: bool):
         if interleaved:

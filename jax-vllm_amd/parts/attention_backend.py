@@ -8,7 +8,7 @@ neighbours where the kernel gives each group waves of its own (they see the same
 while all blocks are on the chip at once, a group that sees many keys with one that sees few, so
 that all blocks carry the same load.  Everything else
 (float32, other head sizes) runs the generic float-math kernel.  The plan depends on the
-step's lengths, the heads-per-group ratio and whether the layer has a window, so it is built
+step's lengths, the heads-per-group ratio and which keys the layer's queries see, so it is built
 once per step and shared by all layers alike.
 """
 from __future__ import annotations
@@ -36,6 +36,11 @@ class MfmaPlan:
     scratch: Optional[torch.Tensor]
 
 
+def keys_seen(kv_len: int, window: int) -> int:
+    """The most keys a query sees that has ``kv_len`` keys up to itself (``K.key_window``'s number)."""
+    return min(kv_len, abs(window)) if window else kv_len
+
+
 def decode_splits(n_decode: int, blocks_per_request: int, max_kv_len: int) -> int:
     base = max(1, n_decode * blocks_per_request)
     by_fill = -(-TARGET_BLOCKS // base)
@@ -50,7 +55,7 @@ def prefill_work_items(q_lens, context_lens, g: int, window: int, group_rows: in
                        balance: bool = True):
     """Work items (request, first row of group 0, first row of group 1 or -1) of the prefill kernel
     for the requests with more than one token, heaviest first.  Rows are (query, head-in-group)
-    pairs.  With ``balance`` and no window the i-th lightest group of a request is paired with its
+    pairs.  ``window``: see ``K.key_window``.  With ``balance`` and no window the i-th lightest group of a request is paired with its
     i-th heaviest: every pair then walks about the same number of (row tile, key tile) products,
     which matters when the items are so few that the heaviest one decides the time.  Otherwise
     neighbours are paired: they share nearly all their keys, so every fragment read feeds both."""
@@ -62,7 +67,8 @@ def prefill_work_items(q_lens, context_lens, g: int, window: int, group_rows: in
         for m0 in range(0, ql * g, group_rows):
             last_row = min(ql * g, m0 + group_rows) - 1
             end = cl + last_row // g + 1
-            begin = max(0, cl + m0 // g - window + 1) if window else 0
+            first = cl + m0 // g
+            begin = max(0, first - window + 1) if window > 0 else first - first % -window if window else 0
             groups.append((-(-end // KEY_TILE) - begin // KEY_TILE, m0))
         if groups_per_item < 2:
             items.extend((t, r, m0, -1) for t, m0 in groups)
@@ -127,7 +133,7 @@ def plan_mfma(ctx, nq: int, nkv: int, head_dim: int, window: int, device) -> Mfm
         prefill = pair_up_resident_items(prefill, cus // nkv)
     decode = [r for r, ql in enumerate(ctx.q_lens_host) if ql == 1]
     max_kv_decode = max([ctx.context_lens_host[r] + 1 for r in decode], default=1)
-    splits = decode_splits(len(decode), nkv * (-(-g // 16)), max_kv_decode) if decode else 1
+    splits = decode_splits(len(decode), nkv * (-(-g // 16)), keys_seen(max_kv_decode, window)) if decode else 1
     if decode:      # a very wide block table is taken split by split
         widest = max(t.shape[1] for t in ctx.block_tables)
         splits = max(splits, K.attn_decode_min_splits(widest, ctx.page_size))
@@ -146,23 +152,24 @@ def plan_mfma(ctx, nq: int, nkv: int, head_dim: int, window: int, device) -> Mfm
 def run(att, out, qkv, ctx, mem) -> None:
     # q heads of a row sit at the front of the fused q/k/v projection, unless the mixer says where else
     q_row_stride = getattr(att, "q_row_stride", None) or (att.nq + 2 * att.nkv) * att.d
+    window = K.key_window(att.window, getattr(att, "chunk", None))
     sinks = getattr(att, "sinks", None)      # float [nq] or None: one more term exp(sink) in every softmax denominator
     if not K.mfma_attention_supported(qkv.dtype, att.d, ctx.page_size):
         K.paged_attention_generic(
             out, qkv, q_row_stride, mem.pages["k"], mem.pages["v"], ctx.block_tables[mem.group], ctx.token_req,
-            ctx.positions, att.nq, att.nkv, att.d, att.scale, att.window or 0, sinks=sinks,
+            ctx.positions, att.nq, att.nkv, att.d, att.scale, window, sinks=sinks,
         )
         return
-    key = ("mfma_attention_plan", att.nq, att.nkv, att.d, bool(att.window))
+    key = ("mfma_attention_plan", att.nq, att.nkv, att.d, window)
     plan = ctx.plans.get(key)
     if plan is None:
-        plan = ctx.plans[key] = plan_mfma(ctx, att.nq, att.nkv, att.d, att.window or 0, qkv.device)
+        plan = ctx.plans[key] = plan_mfma(ctx, att.nq, att.nkv, att.d, window, qkv.device)
     tables = ctx.block_tables[mem.group]
     if plan.n_prefill:
         K.attn_prefill_mfma(out, qkv, q_row_stride, mem.pages["k"], mem.pages["v"], tables, ctx.cu_seqlens,
                             ctx.context_lens, plan.prefill_work, plan.n_prefill, att.nq, att.nkv, att.d, att.scale,
-                            att.window or 0, sinks=sinks)
+                            window, sinks=sinks)
     if plan.n_decode:
         K.attn_decode_mfma(out, qkv, q_row_stride, mem.pages["k"], mem.pages["v"], tables, ctx.cu_seqlens,
                            ctx.context_lens, plan.decode_work, plan.n_decode, att.nq, att.nkv, att.d, att.scale,
-                           att.window or 0, plan.num_splits, plan.scratch, sinks=sinks)
+                           window, plan.num_splits, plan.scratch, sinks=sinks)

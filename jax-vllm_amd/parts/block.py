@@ -16,7 +16,7 @@ from __future__ import annotations
 import torch
 
 from ..ops import kernels as K
-from .spec import PartSpec, build_part, is_replayable, register_part
+from .spec import BLOCK_STATE, PartSpec, StateSpec, TensorSpec, build_part, is_replayable, register_part
 
 
 class PreNormBlock:
@@ -81,13 +81,23 @@ class SandwichBlock:
     (the second line only for a layer that has a feed-forward).  A sublayer's output is handed on as a
     ``K.PendingNorm`` (the output and the norm weight that belongs to it): the next norm's kernel norms it,
     adds it to the stream and norms the stream in one pass, also across the border of two layers and
-    before the head."""
+    before the head.
+
+    With ``input_taps`` what a sublayer reads is its normed input plus a causal filter of it over time per channel,
+    u + F(u), F(u)_t = sum_j w[:, j] u_(t - taps + 1 + j) (zeros before the sequence's start): the last taps - 1 inputs
+    are state of the block's own, in the request's slot.  A step of one token a request filters in the norm's kernel."""
 
     def __init__(self, norm: PartSpec, has_feed_forward: bool = True,
-                 names=("norm1", "norm1b", "norm2", "norm2b")):
+                 names=("norm1", "norm1b", "norm2", "norm2b"), input_taps: int | None = None, hidden_size: int | None = None,
+                 filter_names=("canon1", "canon2")):
         self.has_feed_forward = bool(has_feed_forward)
         self.names = tuple(names) if self.has_feed_forward else tuple(names[:2])
         self.norms = [build_part("norm", norm) for _ in self.names]
+        self.taps = int(input_taps) if input_taps else 0
+        self.hidden_size = int(hidden_size) if hidden_size else None
+        if self.taps and not self.hidden_size:
+            raise ValueError("a filter on the sublayers' inputs needs the width")
+        self.filter_names = tuple(filter_names[:2 if self.has_feed_forward else 1]) if self.taps else ()
 
     @property
     def replayable(self) -> bool:
@@ -98,21 +108,37 @@ class SandwichBlock:
         for name, part in zip(self.names, self.norms):
             for k, v in part.tensors().items():
                 out[f"{name}.{k}"] = v
+        for name in self.filter_names:
+            out[f"{name}.weight"] = TensorSpec((self.hidden_size, self.taps), role="vector", init="small")
         return out
+
+    def state_spec(self):
+        return tuple(StateSpec((self.taps - 1, self.hidden_size), "float32", name) for name in self.filter_names) or None
 
     def bind(self, tensors: dict, dtype: torch.dtype) -> None:
         for name, part in zip(self.names, self.norms):
             part.bind({k[len(name) + 1:]: v for k, v in tensors.items() if k.startswith(name + ".")}, dtype)
+        self.dtype = dtype
+        self.filters = [tensors[f"{name}.weight"].t().contiguous() for name in self.filter_names]     # [taps, width]
+
+    def _input(self, i: int, h, delta, ctx, mem):
+        """What sublayer i reads; ``h`` takes what ``delta`` still owes the stream."""
+        norm = self.norms[2 * i]
+        if not self.taps:
+            return norm.add_norm(h, delta)
+        state = mem.states[BLOCK_STATE + self.filter_names[i]]
+        if (ctx.decode_only and K.norm_filter_possible(self.hidden_size)
+                and (delta is None or isinstance(delta, K.PendingNorm) and delta.weight is not None and delta.bias is None)):
+            return K.norm_filter(h, delta, norm.weight, norm.eps, self.filters[i], state, ctx.slot_ids, self.dtype)
+        return K.token_filter(norm.add_norm(h, delta), self.filters[i], state, ctx.slot_ids, ctx.cu_seqlens, ctx.max_q_len)
 
     def forward(self, h, delta, mixer, feed_forward, ctx, mem):
-        from ..ops import kernels as K
-
-        x = self.norms[0].add_norm(h, delta)
+        x = self._input(0, h, delta, ctx, mem)
         a = mixer.forward(x, ctx, mem)
         pending = K.pending_norm(a, self.norms[1].weight, self.norms[1].eps)
         if not self.has_feed_forward:
             return pending
-        y = self.norms[2].add_norm(h, pending)
+        y = self._input(1, h, pending, ctx, mem)
         f = feed_forward.forward(y, ctx)
         return K.pending_norm(f, self.norms[3].weight, self.norms[3].eps)
 

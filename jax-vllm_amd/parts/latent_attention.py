@@ -21,7 +21,8 @@ the rotation may pair (i, i + dims/2) or (2i, 2i + 1), as its position part says
 per head whose exponential joins the softmax denominator (no key, no value, not scaled); ``output_gate``
 "head": one gate per head, sigmoid(W_g h)_h with W_g [heads, hidden], instead of one per output element;
 ``own_cache`` False: the layer has no W_dkv and reads the cached vectors e of an earlier layer (the schedule's
-``cache_of``), with its own W_uk, W_uv, queries and everything else.
+``cache_of``), with its own W_uk, W_uv, queries, window and everything else (the cache keeps what the layer that looks
+back furthest needs).
 """
 from __future__ import annotations
 
@@ -132,7 +133,7 @@ class LatentAttention:
                                   cos_sin, ctx.slot_mappings[mem.group], mem.pages["k"], mem.pages["v"], ctx.page_size,
                                   kv_off=self.kv_at, interleaved=self.interleaved)
         elif self.q_rank:
-            cq = K.rmsnorm(proj[:, :self.q_rank].contiguous(), self.q_norm, self.eps)
+            cq = K.latent_prepare(proj, self.q_rank, 0, 0, 0, self.q_norm, None, self.eps, None, None, None, None, ctx.page_size)
         q = K.linear(cq, self.w_q_up) if self.q_rank else proj       # proj's rows begin with the queries
         qe = torch.empty((n, H * E), dtype=x.dtype, device=x.device)
         K.head_linear(qe, E, q, self.dim + self.rot, self.w_k_up_t)             # W_uk[h]^T q_plain

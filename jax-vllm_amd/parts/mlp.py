@@ -47,7 +47,8 @@ class GatedMLP:
 
 class DenseMLP:
     """A feed-forward without a gate: ``down( act(up(x) + b_up) ) + b_down``; the activation is one of
-    ``ops.kernels.PLAIN_ACTIVATIONS`` ("gelu" is the erf form), computed in float; the biases are optional."""
+    ``ops.kernels.PLAIN_ACTIVATIONS`` ("gelu" is the erf form, "relu2" the square of relu), computed in float; the biases
+    are optional."""
 
     replayable = True
 
@@ -57,6 +58,7 @@ class DenseMLP:
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.activation, self.bias = activation, bool(bias)
         self.w_up = self.w_down = self.b_up = self.b_down = None
+        self.partial_out = True     # whether the result may be a float stack of partial products (the next norm adds them)
 
     def tensors(self) -> dict:
         h, i = self.hidden_size, self.intermediate_size
@@ -74,7 +76,7 @@ class DenseMLP:
     def forward(self, x, ctx=None) -> torch.Tensor:
         z = K.linear(x, self.w_up)
         K.bias_act(z, self.b_up, self.activation)
-        y = K.linear(z, self.w_down, partial_ok=True)       # the next norm adds the partial products
+        y = K.linear(z, self.w_down, partial_ok=self.partial_out)       # the next norm adds the partial products
         # the second bias is left to whoever takes the output: a block that norms it adds the bias in that kernel
         return K.BiasedOutput(y, self.b_down) if self.b_down is not None else y
 

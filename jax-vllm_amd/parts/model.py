@@ -12,8 +12,8 @@ from typing import Optional
 
 import torch
 
-from .spec import (PagedCacheSpec, LayerMemory, LayerSpec, ModelSpec, StateSpec, StepContext, TensorSpec, build_part,
-                   is_replayable)
+from .spec import (BLOCK_STATE, PagedCacheSpec, LayerMemory, LayerSpec, ModelSpec, StateSpec, StepContext, TensorSpec,
+                   build_part, is_replayable, state_specs_of)
 
 
 class Layer:
@@ -58,7 +58,7 @@ class RunMemoryPlan:
     run: int
     layer: int
     cache: Optional[PagedCacheSpec]
-    state: Optional[StateSpec]
+    state: object                      # StateSpec, a tuple of them (mixer's and block's), or None
     cache_of: Optional[int]
 
 
@@ -111,8 +111,12 @@ class DecoderModel:
     def memory_plan(self) -> list:
         plan = []
         for i, run in enumerate(self.spec.schedule):
-            mixer = self.layers[run.layer].mixer
-            plan.append(RunMemoryPlan(i, run.layer, mixer.cache_spec(), mixer.state_spec(), run.cache_of))
+            mixer, block = self.layers[run.layer].mixer, self.layers[run.layer].block
+            states = mixer.state_spec()
+            of_block = state_specs_of(block.state_spec()) if hasattr(block, "state_spec") else ()
+            if of_block:
+                states = state_specs_of(states) + tuple(StateSpec(st.shape, st.dtype, BLOCK_STATE + st.name) for st in of_block)
+            plan.append(RunMemoryPlan(i, run.layer, mixer.cache_spec(), states, run.cache_of))
         return plan
 
     def replayable(self) -> bool:

@@ -1,12 +1,14 @@
-"""Routed experts: a feed-forward of many small gated feed-forwards, of which each token uses a few
+"""Routed experts: a feed-forward of many small feed-forwards, gated or not, of which each token uses a few
 (no reference counterpart).
 
     z = W_router x (+ b)  (float);   the ``top`` experts with the largest z are chosen;
     s = sigmoid(z), or (``score`` "softmax_chosen") the softmax over the chosen z alone, or (``score``
     "sigmoid_normed") the experts with the largest sigmoid(z) + correction are chosen and
-    s = sigmoid(z) / (sum of the chosen sigmoids + 1e-20) * ``weight_scale``
+    s = sigmoid(z) / (sum of the chosen sigmoids + 1e-20) * ``weight_scale``, or (``score`` "softmax") the
+    softmax over ALL z, as it is; with ``groups`` (count, keep) the experts form equal groups of neighbours
+    and only those of the ``keep`` groups with the largest z can be chosen
     out = sum over the chosen e of  expert_e(s_e * x)   [+ shared(x)  or  + sigmoid(w_sg . x) shared(x)]
-    expert(u) = W_down ( act(W_gate u) * (W_up u) )
+    expert(u) = W_down ( act(W_gate u) * (W_up u) ),  or (``gated`` False) W_down act(W_up u)
 
 The score multiplies the expert's INPUT (``weight_on_input``; with False it multiplies the output).  Since
 the products are linear, s (W u) is computed instead of W (s u): in float, after the product.  Routing,
@@ -29,9 +31,13 @@ class RoutedExperts:
     def __init__(self, hidden_size: int, num_experts: int, top: int, expert_size: int, activation: str = "silu",
                  weight_on_input: bool = True, shared: Optional[PartSpec] = None,
                  expert_names=("gate", "up", "down"), router_bias: bool = False, score: str = "sigmoid",
-                 choice_correction: bool = False, weight_scale: float = 1.0, shared_gate: bool = False):
-        if activation not in K.GATE_ACTIVATIONS:
-            raise ValueError(f"the expert kernels have {sorted(K.GATE_ACTIVATIONS)}, not {activation!r}")
+                 choice_correction: bool = False, weight_scale: float = 1.0, shared_gate: bool = False,
+                 gated: bool = True, groups: Optional[tuple] = None):
+        known = K.GATE_ACTIVATIONS if gated else {a: i for a, i in K.PLAIN_ACTIVATIONS.items() if a}
+        if activation not in known:
+            raise ValueError(f"the expert kernels have {sorted(known)}, not {activation!r}")
+        self.gated = bool(gated)
+        self.groups = (int(groups[0]), int(groups[1])) if groups else None
         self.hidden_size, self.experts, self.top, self.ff = int(hidden_size), int(num_experts), int(top), int(expert_size)
         if not 0 < self.top <= self.experts:
             raise ValueError(f"top = {self.top} of {self.experts} experts")
@@ -42,6 +48,13 @@ class RoutedExperts:
         self.choice_correction, self.weight_scale = bool(choice_correction), float(weight_scale)
         if (self.choice_correction or self.weight_scale != 1.0) and score != "sigmoid_normed":
             raise ValueError("a correction of the choice and a constant on the weights belong to the score 'sigmoid_normed'")
+        if self.groups is not None:
+            count, keep = self.groups
+            if not (0 < keep <= count <= K.ROUTER_MAX_GROUPS) or self.experts % count or keep * (self.experts // count) < self.top:
+                raise ValueError(f"{self.top} of {self.experts} experts in the best {keep} of {count} groups: equal groups, at "
+                                 f"most {K.ROUTER_MAX_GROUPS}, with enough experts in the kept ones")
+            if self.choice_correction:
+                raise ValueError("groups are ranked by their logits: no correction of the choice beside them")
         self.shared_gate = bool(shared_gate)
         if self.shared_gate and shared is None:
             raise ValueError("a gate on the shared expert without a shared expert")
@@ -61,7 +74,8 @@ class RoutedExperts:
         if self.router_bias:
             t["router.bias"] = TensorSpec((self.experts,), role="vector")
         for e in range(self.experts):
-            t[f"experts.{e}.{g}.weight"] = TensorSpec((self.ff, self.hidden_size))
+            if self.gated:
+                t[f"experts.{e}.{g}.weight"] = TensorSpec((self.ff, self.hidden_size))
             t[f"experts.{e}.{u}.weight"] = TensorSpec((self.ff, self.hidden_size))
             t[f"experts.{e}.{d}.weight"] = TensorSpec((self.hidden_size, self.ff))
         if self.choice_correction:
@@ -78,7 +92,7 @@ class RoutedExperts:
         self.w_router = tensors["router.weight"]
         if self.router_bias:
             self.b_router = tensors["router.bias"].contiguous()
-        self.w_gate = torch.stack([tensors[f"experts.{e}.{g}.weight"] for e in range(self.experts)]).contiguous()
+        self.w_gate = torch.stack([tensors[f"experts.{e}.{g}.weight"] for e in range(self.experts)]).contiguous() if self.gated else None
         self.w_up = torch.stack([tensors[f"experts.{e}.{u}.weight"] for e in range(self.experts)]).contiguous()
         self.w_down = torch.stack([tensors[f"experts.{e}.{d}.weight"] for e in range(self.experts)]).contiguous()
         if self.choice_correction:
@@ -93,7 +107,7 @@ class RoutedExperts:
         n = x.shape[0]
         plan = K.moe_route(None, self.top, x=x, w_router=self.w_router, bias=self.b_router, score=self.score,
                            tile_rows=K.moe_tile_rows_for(x.dtype, self.hidden_size, self.ff, n * self.top, self.experts),
-                           correction=self.correction, weight_scale=self.weight_scale)
+                           correction=self.correction, weight_scale=self.weight_scale, groups=self.groups)
         shares = self.top + (1 if self.shared_gate else 0)
         out = torch.empty((shares, n, self.hidden_size), dtype=torch.float32, device=x.device)
         K.moe_experts(x, plan, self.w_gate, self.w_up, self.w_down, self.activation, out[:self.top], self.weight_on_input)

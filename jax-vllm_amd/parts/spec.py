@@ -76,40 +76,60 @@ class PagedTensorSpec:
 class PagedCacheSpec:
     """What a mixer keeps per token in pages: the tensors it declares (a page of each for every
     page id) and which earlier tokens it reads.  ``window`` None: every earlier token is read
-    ("full"); otherwise only the last ``window`` are, and older pages are given back.  Mixers with
+    ("full"); otherwise only the last ``window`` are, and older pages are given back.  ``chunk``: a token
+    reads those of its own block of ``chunk`` positions (counted from position 0), and the pages of a
+    finished block are given back.  Mixers with
     the same need share a page pool and a block table (a *group*), whatever tensors they keep."""
 
     tensors: tuple
     window: Optional[int] = None
+    chunk: Optional[int] = None
 
     def __post_init__(self):
         names = [t.name for t in self.tensors]
         if len(set(names)) != len(names) or not names:
             raise ValueError(f"a paged cache needs tensors with distinct names, got {names}")
+        if self.window and self.chunk:
+            raise ValueError("a mixer reads the last tokens or those of its own block, not both")
 
     @property
     def group_key(self) -> tuple:
-        return ("window", self.window) if self.window else ("full",)
+        return ("window", self.window) if self.window else ("chunk", self.chunk) if self.chunk else ("full",)
 
 
-def kv_cache_spec(num_kv_heads: int, head_dim: int, window: Optional[int] = None) -> PagedCacheSpec:
+def widest_need(keys) -> tuple:
+    """The group key that keeps what every one of these needs reads: a cache that several runs read lives as long as the
+    one that looks back furthest."""
+    keys = set(keys)
+    if len(keys) == 1:
+        return keys.pop()
+    if all(k[0] == "window" for k in keys):
+        return ("window", max(k[1] for k in keys))
+    return ("full",)
+
+
+def kv_cache_spec(num_kv_heads: int, head_dim: int, window: Optional[int] = None, chunk: Optional[int] = None) -> PagedCacheSpec:
     """Keys and values of grouped-query attention in the layout its kernels read: a key page is
     ``[kv_heads, page_size, head_dim]`` (one head's keys of a page are contiguous), a value page
     is transposed, ``[kv_heads, head_dim, page_size]`` (8 consecutive keys of one head element are
     16 aligned bytes)."""
     shape = (int(num_kv_heads), int(head_dim))
-    return PagedCacheSpec((PagedTensorSpec("k", shape, slot_axis=1), PagedTensorSpec("v", shape, slot_axis=2)), window)
+    return PagedCacheSpec((PagedTensorSpec("k", shape, slot_axis=1), PagedTensorSpec("v", shape, slot_axis=2)), window, chunk)
 
 
 @dataclass(frozen=True)
 class StateSpec:
     """State of fixed size per request (one row per slot), zeroed when a request starts.  A mixer that
     keeps several such tensors (a recurrence's matrix and the last inputs of a short convolution, say)
-    returns a tuple of them from ``state_spec()``, each with a ``name`` of its own."""
+    returns a tuple of them from ``state_spec()``, each with a ``name`` of its own.  A block arrangement that
+    keeps state of its own declares it the same way; its names then stand under ``BLOCK_STATE``."""
 
     shape: tuple
     dtype: str = "float32"
     name: str = "state"
+
+
+BLOCK_STATE = "block."     # in front of the state names a block arrangement declared, in ``LayerMemory.states``
 
 
 def state_specs_of(spec) -> tuple:

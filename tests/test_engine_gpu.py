@@ -691,8 +691,14 @@ def test_schedule_repeats_a_layer_shares_a_cache_and_windows(folders, dtype):
     model = custom_model(folders["B"], dtype, schedule, windows)
     plan = model.memory_plan()
     assert [p.cache_of for p in plan] == [None, None, None, 0, None]
-    with pytest.raises(ValueError, match="already given back"):      # all keys wanted of a cache that keeps a window
-        make_core(None, dtype, 16, pages=4, model=custom_model(folders["B"], dtype, [(0, None), (1, None), (2, 1)], windows))
+    # all keys wanted of a cache whose own layer sees a window: the pages stay
+    wider = [(0, None), (1, None), (2, 1)]
+    core = make_core(None, dtype, 16, pages=8, model=custom_model(folders["B"], dtype, wider, windows))
+    assert core.group_keys == [("full",)]
+    toks = np.random.default_rng(4).integers(0, cfg["vocab_size"], size=100).tolist()
+    core.start_request("a")
+    got = [core.run([entry("a", toks[at:at + 20])]).cpu().numpy() for at in range(0, 100, 20)]
+    check_logits(dtype, np.concatenate(got), P.forward_scheduled(w, cfg, toks, wider, windows).numpy(), what="all keys of a windowed layer's cache")
     core = make_core(None, dtype, 16, pages=24, model=model)
     assert core.group_keys == [("full",), ("window", 24)]
     toks = np.random.default_rng(5).integers(0, cfg["vocab_size"], size=150).tolist()
