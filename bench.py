@@ -110,6 +110,26 @@ def zeripel_shape(width, layers, heads, ff, experts, top, expert_ff, shared_ff, 
             "embedding": {"scale": 1.0, "bigram": {"buckets": 100003, "mul_prev": 1000003, "mul_cur": 7919}}, "layers": out}
 
 
+def fezuzen_shape(width, layers, heads, experts, top, expert_ff, shared_ff, groups, vocab=32000, size=1024):
+    """Layers in turns: latent attention (a cached vector of 224 + 32 elements, a window of ``size``; every second one
+    reads the cache of the one two layers before) and grouped-query attention with heads of 128 in blocks of ``size``
+    positions; filters of 4 taps everywhere; routed experts without a gate in every layer, chosen from the best half of
+    ``groups`` groups."""
+    latent = {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": 224, "q_rank": width // 4 + 256,
+              "scale": 96 ** -0.5, "mask": {"size": size},
+              "rot": {"base": 500000.0, "dims": 32, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    att = {"type": "attention", "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "conv": 4,
+                                          "scale": 128 ** -0.5, "mask": {"size": size}, "rot": {"base": 500000.0, "dims": 128}}}
+    mlp = {"kind": "moe", "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": groups // 2}},
+           "expert": {"ff": expert_ff}, "shared": {"ff": shared_ff}}
+    out = []
+    for i in range(layers):
+        mixer = dict(latent, **({"kv_from": i - 2} if i % 4 == 2 else {}))
+        out.append(dict(att, mlp=mlp) if i % 2 else {"type": "latent_attention", "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Fezuzen", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "canon": {"taps": 4},
+            "logit_scale": 0.5, "layers": out}
+
+
 # --only design: Lomozen beside the dense model of the same width, depth, vocabulary and feed-forward
 # parameters per token (top * expert + shared = intermediate)
 DESIGN_SHAPES = {
@@ -137,6 +157,13 @@ BOZISUN_SHAPES = {
 ZERIPEL_SHAPES = {
     "2k": (zeripel_shape(2048, 8, 16, 3072, 32, 4, 512, 1024),) + DESIGN_SHAPES["2k"],
     "4k": (zeripel_shape(4096, 8, 32, 8192, 64, 6, 1024, 2048),) + DESIGN_SHAPES["4k"],
+}
+# --only design --design fezuzen: Fezuzen beside Lomozen (the closest kin: latent attention inside a window, norms on both sides
+# of every sublayer, routed experts with a shared one) and the dense model, all of one width, depth, vocabulary and
+# feed-forward parameters per token (2 * (top * expert + shared) = 3 * intermediate)
+FEZUZEN_SHAPES = {
+    "2k": (fezuzen_shape(2048, 8, 16, 32, 4, 768, 1536, 8),) + DESIGN_SHAPES["2k"],
+    "4k": (fezuzen_shape(4096, 8, 32, 64, 6, 1536, 3072, 8),) + DESIGN_SHAPES["4k"],
 }
 PROMPT_LEN = 1024
 MAX_CONTEXT = 8192
@@ -265,6 +292,7 @@ def measure_design(args, rng):
     models = (zip(("dumazen", "lomozen", "dense"), DUMAZEN_SHAPES[args.design_shape]) if args.design == "dumazen"
               else zip(("bozisun", "lomozen", "dense"), BOZISUN_SHAPES[args.design_shape]) if args.design == "bozisun"
               else zip(("zeripel", "lomozen", "dense"), ZERIPEL_SHAPES[args.design_shape]) if args.design == "zeripel"
+              else zip(("fezuzen", "lomozen", "dense"), FEZUZEN_SHAPES[args.design_shape]) if args.design == "fezuzen"
               else zip(("lomozen", "dense"), DESIGN_SHAPES[args.design_shape]))
     out["design"] = args.design
     for name, cfg in models:
@@ -434,7 +462,7 @@ def main():
     ap.add_argument("--no-kernel-share", action="store_true", help="leave out the per-kernel time shares")
     ap.add_argument("--design-shape", choices=sorted(DESIGN_SHAPES), default="2k",
                     help="with --only design: the width of both models (2,048 or 4,096), 8 layers each")
-    ap.add_argument("--design", choices=["lomozen", "dumazen", "bozisun", "zeripel"], default="lomozen",
+    ap.add_argument("--design", choices=["lomozen", "dumazen", "bozisun", "zeripel", "fezuzen"], default="lomozen",
                     help="with --only design: the architecture that is measured beside its kin of equal size")
     ap.add_argument("--design-models", default="", help="with --only design: only these of the models, with commas between them")
     ap.add_argument("--only", choices=["prefill", "decode", "mixed", "long-prompt", "ttft", "calibrate", "design"], default=None,
