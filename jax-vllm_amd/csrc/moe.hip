@@ -28,6 +28,7 @@
 #define MOE_SCORE_SIGMOID_NORMED 2   // chosen by sigmoid(logit) + correction; weight = sigmoid(logit) / (sum over the chosen + 1e-20) * scale
 #define MOE_SCORE_SOFTMAX 3          // weight = exp(logit) / sum of exp over all of the token's logits
 #define MOE_MAX_GROUPS 64
+#define MOE_RANK_EXPERTS 128         // up to so many experts are ranked by counting
 __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int lane, int* ids, float* weights,
                                          int score, const float* __restrict__ correction, float weight_scale,
                                          int groups, int keep) {
@@ -48,13 +49,62 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
       for (int i = 0; i < size; ++i) best = fmaxf(best, zt[lane * size + i]);
     int ahead = 0;
     for (int g = 0; g < groups; ++g) {
-      const float other = __shfl(best, g, JV_WAVE);
+      const float other = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(best), g));
       if (other > best || (other == best && g < lane)) ++ahead;
     }
     const unsigned long long kept = __ballot(lane < groups && ahead < keep);
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // the groups are read before their entries change
     for (int e = lane; e < experts; e += JV_WAVE)
       if (!((kept >> (e / size)) & 1)) zt[e] = -INFINITY;
+  }
+  if (experts <= MOE_RANK_EXPERTS) {
+    // an expert's place is the number of experts ahead of it (a larger value, or an equal one of a lower number): every
+    // lane counts for its own experts over the values in LDS, instead of `top` searches across the wave one after the other
+    constexpr int PER = MOE_RANK_EXPERTS / JV_WAVE;
+    float z[PER], c[PER];
+    int ahead[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int e = lane + i * JV_WAVE;
+      z[i] = e < experts ? zt[e] : -INFINITY;
+      c[i] = z[i];
+      if (normed && z[i] != -INFINITY) c[i] = 1.f / (1.f + expf(-z[i])) + (correction && e < experts ? correction[e] : 0.f);
+      if (c[i] != c[i]) c[i] = -INFINITY;         // a NaN takes the last places, its weight shows it
+      ahead[i] = 0;
+    }
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (lane + i * JV_WAVE < experts) zt[lane + i * JV_WAVE] = c[i];
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // the values are read by the wave's other lanes
+    for (int e = 0; e < experts; ++e) {
+      const float o = zt[e];
+#pragma unroll
+      for (int i = 0; i < PER; ++i) ahead[i] += (o > c[i] || (o == c[i] && e < lane + i * JV_WAVE)) ? 1 : 0;
+    }
+    float s[PER], share = 0.f, most = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const bool chosen = lane + i * JV_WAVE < experts && ahead[i] < top;
+      if (!chosen) ahead[i] = top;
+      else most = fmaxf(most, z[i]);
+    }
+    if (score == MOE_SCORE_SOFTMAX_CHOSEN) most = wave_max(most);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      s[i] = score == MOE_SCORE_SOFTMAX_CHOSEN ? expf(z[i] - most) : score == MOE_SCORE_SOFTMAX ? expf(z[i] - zmax) * inv_sum
+                                                                                             : 1.f / (1.f + expf(-z[i]));
+      if (ahead[i] < top) share += s[i];
+    }
+    float f = 1.f;
+    if (score == MOE_SCORE_SOFTMAX_CHOSEN) f = 1.f / wave_sum(share);
+    if (normed) f = weight_scale / (wave_sum(share) + 1e-20f);
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (ahead[i] < top) {
+        ids[ahead[i]] = lane + i * JV_WAVE;
+        weights[ahead[i]] = s[i] * f;
+      }
+    return;
   }
   for (int kk = 0; kk < top; ++kk) {
     float bv = -INFINITY;
@@ -177,6 +227,37 @@ moe_router_kernel(const T* __restrict__ x, const T* __restrict__ W, const float*
              weight_scale, groups, keep);
 }
 
+// Exclusive sums over the experts of their entries and of their tiles, by one wave: start, tile0 [experts + 1].
+__device__ __forceinline__ void moe_scan_counts(const int* count, int* start, int* tile0, int experts, int tile_rows, int lane) {
+  int at = 0, tiles = 0;
+  for (int e0 = 0; e0 < experts; e0 += JV_WAVE) {
+    const int e = e0 + lane;
+    const int c = e < experts ? count[e] : 0, t = (c + tile_rows - 1) / tile_rows;
+    int ci = c, ti = t;
+#pragma unroll
+    for (int o = 1; o < JV_WAVE; o <<= 1) {
+      const int cu = __shfl_up(ci, o, JV_WAVE), tu = __shfl_up(ti, o, JV_WAVE);
+      if (lane >= o) { ci += cu; ti += tu; }
+    }
+    if (e < experts) { start[e] = at + ci - c; tile0[e] = tiles + ti - t; }
+    at += __shfl(ci, JV_WAVE - 1, JV_WAVE);
+    tiles += __shfl(ti, JV_WAVE - 1, JV_WAVE);
+  }
+  if (lane == 0) { start[experts] = at; tile0[experts] = tiles; }
+}
+
+// What a grouping hands on, from the sums: meta [0] number of tiles, offsets [experts + 1], tile_expert / tile_row0.
+__device__ __forceinline__ void moe_write_tiles(const int* start, const int* tile0, int experts, int tile_rows, int* meta,
+                                                int* offsets, int* tile_expert, int* tile_row0) {
+  if (threadIdx.x == 0) meta[0] = tile0[experts];
+  for (int e = threadIdx.x; e <= experts; e += blockDim.x) offsets[e] = start[e];
+  for (int e = threadIdx.x; e < experts; e += blockDim.x)
+    for (int i = tile0[e]; i < tile0[e + 1]; ++i) {
+      tile_expert[i] = e;
+      tile_row0[i] = start[e] + (i - tile0[e]) * tile_rows;
+    }
+}
+
 // One block.  meta: [0] number of tiles; offsets [experts + 1]; tile_expert / tile_row0 [max_tiles];
 // order [entries]: entry index at each position; rank [entries] scratch.  A tile has tile_rows rows.
 __global__ void __launch_bounds__(1024)
@@ -191,26 +272,53 @@ moe_group_kernel(const int* __restrict__ ids, int entries, int experts, int tile
   __syncthreads();
   for (int s = threadIdx.x; s < entries; s += blockDim.x) rank[s] = atomicAdd(&count[ids[s]], 1);
   __syncthreads();
-  if (threadIdx.x == 0) {
-    int at = 0, tiles = 0;
-    for (int e = 0; e < experts; ++e) {
-      start[e] = at;
-      tile0[e] = tiles;
-      at += count[e];
-      tiles += (count[e] + tile_rows - 1) / tile_rows;
+  if (threadIdx.x < JV_WAVE) moe_scan_counts(count, start, tile0, experts, tile_rows, threadIdx.x);
+  __syncthreads();
+  moe_write_tiles(start, tile0, experts, tile_rows, meta, offsets, tile_expert, tile_row0);
+  for (int s = threadIdx.x; s < entries; s += blockDim.x) order[start[ids[s]] + rank[s]] = s;
+}
+
+// Choice and grouping of few tokens in one launch of one block: a wave a token picks, then the block groups.  Every
+// token has `top` chosen entries and `always` further ones, for the experts behind the routed ones (number experts,
+// experts + 1, ...), whose weight is 1: a shared expert cut into pieces of the routed ones' size.  Entry s = token *
+// (top + always) + kk.  LDS: logits [16][experts] | ids [entries] | rank [entries] | count, start, first tile of experts + always.
+__global__ void __launch_bounds__(1024)
+moe_route_group_kernel(const float* __restrict__ logits, const float* __restrict__ bias, int n, int experts, int top,
+                       int always, int score, int* __restrict__ ids, float* __restrict__ weights,
+                       const float* __restrict__ correction, float weight_scale, int groups, int keep, int tile_rows,
+                       int* __restrict__ meta, int* __restrict__ offsets, int* __restrict__ tile_expert,
+                       int* __restrict__ tile_row0, int* __restrict__ order) {
+  extern __shared__ float zs[];
+  const int all = experts + always, per = top + always, entries = n * per;
+  int* lid = (int*)(zs + 16 * experts);
+  int* rank = lid + entries;
+  int* count = rank + entries;
+  int* start = count + all;
+  int* tile0 = start + all + 1;
+  const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE;
+  for (int e = threadIdx.x; e < all; e += blockDim.x) count[e] = 0;
+  float* zt = zs + wid * experts;
+  for (int t = wid; t < n; t += 16) {
+    for (int e = lane; e < experts; e += JV_WAVE) zt[e] = logits[(long long)t * experts + e] + (bias ? bias[e] : 0.f);
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");        // a group's lane reads what other lanes wrote
+    moe_pick(zt, experts, top, lane, lid + t * per, weights + (long long)t * per, score, correction, weight_scale, groups, keep);
+    if (lane < always) {
+      lid[t * per + top + lane] = experts + lane;
+      weights[(long long)t * per + top + lane] = 1.f;
     }
-    start[experts] = at;
-    tile0[experts] = tiles;
-    meta[0] = tiles;
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");        // before the wave's next token takes its place
   }
   __syncthreads();
-  for (int e = threadIdx.x; e <= experts; e += blockDim.x) offsets[e] = start[e];
-  for (int e = threadIdx.x; e < experts; e += blockDim.x)
-    for (int i = tile0[e]; i < tile0[e + 1]; ++i) {
-      tile_expert[i] = e;
-      tile_row0[i] = start[e] + (i - tile0[e]) * tile_rows;
-    }
-  for (int s = threadIdx.x; s < entries; s += blockDim.x) order[start[ids[s]] + rank[s]] = s;
+  for (int s = threadIdx.x; s < entries; s += blockDim.x) {
+    const int e = lid[s];
+    ids[s] = e;
+    rank[s] = atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  if (wid == 0) moe_scan_counts(count, start, tile0, all, tile_rows, lane);
+  __syncthreads();
+  moe_write_tiles(start, tile0, all, tile_rows, meta, offsets, tile_expert, tile_row0);
+  for (int s = threadIdx.x; s < entries; s += blockDim.x) order[start[lid[s]] + rank[s]] = s;
 }
 
 // grid (max tiles, column tiles of the expert width).  x [tokens, hidden]; Wg, Wu [experts, ff, hidden];
@@ -386,6 +494,27 @@ extern "C" int jv_moe_route(const float* logits, const float* bias, int n, int e
   if (experts > 3840) return (int)hipErrorInvalidValue;
   hipLaunchKernelGGL(moe_route_kernel, dim3((n + 3) / 4), dim3(256), 4 * experts * sizeof(float), (hipStream_t)stream,
                      logits, bias, n, experts, top, score, ids, weights, correction, weight_scale, groups, keep);
+  return JV_LAUNCH_CHECK();
+}
+
+// 1 if the one-block form takes these sizes, else 0
+extern "C" int jv_moe_route_group_fits(int n, int experts, int top, int always) {
+  if (n <= 0 || experts <= 0 || top <= 0 || always < 0 || always > JV_WAVE) return 0;
+  return n <= 64 && (16LL * experts + 2LL * n * (top + always) + 3LL * (experts + always) + 2) * 4 <= 60 * 1024;
+}
+
+extern "C" int jv_moe_route_group(const float* logits, const float* bias, int n, int experts, int top, int always, int score,
+                                  int* ids, float* weights, const float* correction, float weight_scale, int groups,
+                                  int keep, int tile_rows, int* meta, int* offsets, int* tile_expert, int* tile_row0,
+                                  int* order, void* stream) {
+  if (n <= 0) return 0;
+  if (!jv_moe_route_group_fits(n, experts, top, always) || top > experts || score < 0 || score > MOE_SCORE_SOFTMAX ||
+      !moe_groups_ok(experts, top, groups, keep) || tile_rows <= 0)
+    return (int)hipErrorInvalidValue;
+  const size_t shmem = (16 * (size_t)experts + 2 * (size_t)n * (top + always) + 3 * (size_t)(experts + always) + 2) * 4;
+  hipLaunchKernelGGL(moe_route_group_kernel, dim3(1), dim3(1024), shmem, (hipStream_t)stream, logits, bias, n, experts, top,
+                     always, score, ids, weights, correction, weight_scale, groups, keep, tile_rows, meta, offsets,
+                     tile_expert, tile_row0, order);
   return JV_LAUNCH_CHECK();
 }
 

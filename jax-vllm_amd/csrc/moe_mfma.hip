@@ -30,15 +30,21 @@ moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const
                 const float* __restrict__ weights, int top, int n_tokens, int K, int N, int act, int use_weight) {
   constexpr int TM = 16 * MT;
   constexpr bool GATED = MODE == MM_GATED, BY_TOKEN = MODE != MM_DOWN;
-  if (tile_expert && (int)blockIdx.x >= meta[0]) return;
+  // Blocks b, b + 8, b + 16, ... run on one XCD (with an L2 of its own): each of the 8 takes one run of the (tile, rows of W)
+  // pairs, rows of W fastest, so the rows of x of a tile and the weights of an expert are read into one L2 and used there.
+  const int per_tile = (N + MM_T - 1) / MM_T;
+  const int live = (tile_expert ? meta[0] : (n_tokens + TM - 1) / TM) * per_tile, chunk = (live + 7) / 8;
+  const int pair = ((int)blockIdx.x & 7) * chunk + ((int)blockIdx.x >> 3);
+  if (((int)blockIdx.x >> 3) >= chunk || pair >= live) return;
+  const int tile = pair / per_tile;
   __shared__ __attribute__((aligned(16))) bf16_t xs[TM * MM_S];
   __shared__ __attribute__((aligned(16))) bf16_t w0s[MM_T * MM_S];
   __shared__ __attribute__((aligned(16))) bf16_t w1s[GATED ? MM_T * MM_S : 8];
   __shared__ int ent[TM];
-  const int e = tile_expert ? tile_expert[blockIdx.x] : 0, row0 = tile_expert ? tile_row0[blockIdx.x] : blockIdx.x * TM;
+  const int e = tile_expert ? tile_expert[tile] : 0, row0 = tile_expert ? tile_row0[tile] : tile * TM;
   const int rows = min(TM, (tile_expert ? offsets[e + 1] : n_tokens) - row0);
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, li = lane & 15, lc = lane >> 4;
-  const int n0 = blockIdx.y * MM_T;
+  const int n0 = (pair - tile * per_tile) * MM_T;
   if (tid < TM) ent[tid] = tile_expert ? order[row0 + min(tid, rows - 1)] : row0 + min(tid, rows - 1);   // rows beyond the tile repeat its last row
   __syncthreads();
   // staging: thread t brings pieces t and t + 256 of each operand: piece p = row p / 8, columns (p % 8) * 8 .. + 7
@@ -134,10 +140,13 @@ moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const
 }
 
 template <int MODE>
-static int launch_moe_mfma(int tile_rows, dim3 grid, hipStream_t stream, void* out, const bf16_t* a, const bf16_t* W0,
+static int launch_moe_mfma(int tile_rows, int max_tiles, hipStream_t stream, void* out, const bf16_t* a, const bf16_t* W0,
                            const bf16_t* W1, const int* meta, const int* offsets, const int* tile_expert,
                            const int* tile_row0, const int* order, const float* weights, int top, int n_tokens, int K,
                            int N, int act, int use_weight) {
+  const long long pairs = (long long)max_tiles * ((N + MM_T - 1) / MM_T);
+  if (pairs > 0x7ffffff0ll) return (int)hipErrorInvalidValue;
+  const dim3 grid((unsigned)(pairs + 7));
   if (tile_rows == 128)
     hipLaunchKernelGGL((moe_mfma_kernel<MODE, 8>), grid, dim3(256), 0, stream, out, a, W0, W1, meta, offsets, tile_expert,
                        tile_row0, order, weights, top, n_tokens, K, N, act, use_weight);
@@ -158,10 +167,10 @@ extern "C" int jv_moe_gate_up_mfma_bf16(void* z, const void* x, const void* Wg, 
   if (max_tiles <= 0 || ff <= 0) return 0;
   if (!(Wg ? jv_act_known(act) : jv_plain_act_known(act)) || hidden < 8 || hidden % 8 || (ff + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
   if (!Wg)
-    return launch_moe_mfma<MM_PLAIN>(tile_rows, dim3(max_tiles, (ff + MM_T - 1) / MM_T), (hipStream_t)stream, z,
+    return launch_moe_mfma<MM_PLAIN>(tile_rows, max_tiles, (hipStream_t)stream, z,
                                      (const bf16_t*)x, (const bf16_t*)Wu, nullptr, meta, offsets, tile_expert, tile_row0,
                                      order, weights, top, 0, hidden, ff, act, scale_input);
-  return launch_moe_mfma<MM_GATED>(tile_rows, dim3(max_tiles, (ff + MM_T - 1) / MM_T), (hipStream_t)stream, z, (const bf16_t*)x,
+  return launch_moe_mfma<MM_GATED>(tile_rows, max_tiles, (hipStream_t)stream, z, (const bf16_t*)x,
                                (const bf16_t*)Wg, (const bf16_t*)Wu, meta, offsets, tile_expert, tile_row0, order,
                                weights, top, 0, hidden, ff, act, scale_input);
 }
@@ -173,7 +182,7 @@ extern "C" int jv_moe_down_mfma_bf16(float* y, const void* z, const void* Wd, co
                                      int scale_output, int tile_rows, void* stream) {
   if (max_tiles <= 0 || hidden <= 0) return 0;
   if (ff < 8 || ff % 8 || (hidden + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
-  return launch_moe_mfma<MM_DOWN>(tile_rows, dim3(max_tiles, (hidden + MM_T - 1) / MM_T), (hipStream_t)stream, y,
+  return launch_moe_mfma<MM_DOWN>(tile_rows, max_tiles, (hipStream_t)stream, y,
                                 (const bf16_t*)z, (const bf16_t*)Wd, nullptr, meta, offsets, tile_expert, tile_row0, order,
                                 weights, top, n_tokens, ff, hidden, 0, scale_output);
 }
@@ -183,6 +192,6 @@ extern "C" int jv_moe_down_mfma_bf16(float* y, const void* z, const void* Wd, co
 extern "C" int jv_gemm_rows_f32out_bf16(float* y, const void* x, const void* W, int M, int N, int K, void* stream) {
   if (M <= 0 || N <= 0) return 0;
   if (K < 8 || K % 8 || (N + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
-  return launch_moe_mfma<MM_DOWN>(128, dim3((M + 127) / 128, (N + MM_T - 1) / MM_T), (hipStream_t)stream, y, (const bf16_t*)x,
+  return launch_moe_mfma<MM_DOWN>(128, (M + 127) / 128, (hipStream_t)stream, y, (const bf16_t*)x,
                                 (const bf16_t*)W, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 1, M, K, N, 0, 0);
 }

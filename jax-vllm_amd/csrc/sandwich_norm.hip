@@ -98,9 +98,14 @@ struct SnFilter {
   int lags;
 };
 
-#define SN_V 4      // 16-byte pieces a thread: rows of up to 4 * SN_V * 256 = 4,096 floats
-template <typename T, bool FILTER>
-__global__ void __launch_bounds__(256)
+#define SN_V 4          // 16-byte pieces a thread of a block of 256: rows of up to 4 * SN_V * 256 = 4,096 floats
+#define SN_FEW_ROWS 64  // up to so many rows a row gets a thread for each of its 16-byte pieces
+#define SN_PARTS 4      // partial results a thread with one piece asks for at once
+
+// V pieces a thread, blocks of `blockDim.x` threads; L > 0: with a filter of up to L lags (L = 0: none).  Everything a
+// row needs is asked for before its first sum (the filter's inputs and weights too): a row's time is its chain of loads.
+template <typename T, int V, int L>
+__global__ void __launch_bounds__(V == 1 ? 1024 : 256)
 postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, const float* __restrict__ parts,
                                 int n_parts, long long part_stride, const float* __restrict__ bias,
                                 const float* __restrict__ wb,
@@ -109,41 +114,65 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
   __shared__ float red[32];
   const long long i = blockIdx.x;
   const long long r = rows ? (long long)rows[i] : i;
-  float4 v[SN_V], x[SN_V], b[SN_V];
+  const int step = blockDim.x * 4;
+  const float4 zero4 = float4{0.f, 0.f, 0.f, 0.f};
+  float4 v[V], x[V], b[V], g[V];
+  float4 past[L ? L * V : 1], tap[L ? (L + 1) * V : 1];
+  float* st = nullptr;
+  if constexpr (L > 0) st = f.state + (long long)f.slot_ids[r] * f.lags * hidden;
   float ss = 0.f;
 #pragma unroll
-  for (int q = 0; q < SN_V; ++q) {
-    const int c = (threadIdx.x + q * 256) * 4;
+  for (int q = 0; q < V; ++q) {
+    const int c = threadIdx.x * 4 + q * step;
     const int cc = c < hidden ? c : 0;           // a piece beyond the row reads the row's first piece, its share is left out
-    v[q] = y ? sn_load4<T>(y + r * hidden + cc) : float4{0.f, 0.f, 0.f, 0.f};
+    v[q] = y ? sn_load4<T>(y + r * hidden + cc) : zero4;
     x[q] = *(const float4*)(h + r * hidden + cc);
     b[q] = wb ? *(const float4*)(wb + cc) : float4{1.f, 1.f, 1.f, 1.f};
-  }
-  for (int p = 0; p < n_parts; ++p) {
+    g[q] = w ? *(const float4*)(w + cc) : zero4;
+    if constexpr (L > 0) {
 #pragma unroll
-    for (int q = 0; q < SN_V; ++q) {
-      const int c = (threadIdx.x + q * 256) * 4;
-      const float4 t = *(const float4*)(parts + p * part_stride + r * hidden + (c < hidden ? c : 0));
-      v[q].x += t.x; v[q].y += t.y; v[q].z += t.z; v[q].w += t.w;
+      for (int j = 0; j < L; ++j)
+        past[q * L + j] = j < f.lags ? *(const float4*)(st + (long long)j * hidden + cc) : zero4;
+#pragma unroll
+      for (int j = 0; j <= L; ++j)
+        tap[q * (L + 1) + j] = j <= f.lags ? *(const float4*)(f.wt + (long long)j * hidden + cc) : zero4;
     }
+  }
+  constexpr int PB = V == 1 ? SN_PARTS : 1;
+  for (int p0 = 0; p0 < n_parts; p0 += PB) {
+    float4 t[PB][V];
+#pragma unroll
+    for (int p = 0; p < PB; ++p)
+#pragma unroll
+      for (int q = 0; q < V; ++q) {
+        const int c = threadIdx.x * 4 + q * step;
+        t[p][q] = p0 + p < n_parts ? *(const float4*)(parts + (p0 + p) * part_stride + r * hidden + (c < hidden ? c : 0)) : zero4;
+      }
+#pragma unroll
+    for (int p = 0; p < PB; ++p)
+#pragma unroll
+      for (int q = 0; q < V; ++q) { v[q].x += t[p][q].x; v[q].y += t[p][q].y; v[q].z += t[p][q].z; v[q].w += t[p][q].w; }
   }
   if (bias) {
 #pragma unroll
-    for (int q = 0; q < SN_V; ++q) {
-      const int c = (threadIdx.x + q * 256) * 4;
+    for (int q = 0; q < V; ++q) {
+      const int c = threadIdx.x * 4 + q * step;
       const float4 t = *(const float4*)(bias + (c < hidden ? c : 0));
       v[q].x += t.x; v[q].y += t.y; v[q].z += t.z; v[q].w += t.w;
     }
   }
 #pragma unroll
-  for (int q = 0; q < SN_V; ++q)
-    if ((threadIdx.x + q * 256) * 4 < hidden) ss += v[q].x * v[q].x + v[q].y * v[q].y + v[q].z * v[q].z + v[q].w * v[q].w;
-  ss = block_sum(ss, red);
-  const float inv_b = wb ? rsqrtf(ss / (float)hidden + eps) : plain_scale;
+  for (int q = 0; q < V; ++q)
+    if (threadIdx.x * 4 + q * step < hidden) ss += v[q].x * v[q].x + v[q].y * v[q].y + v[q].z * v[q].z + v[q].w * v[q].w;
+  float inv_b = plain_scale;
+  if (wb) {
+    ss = block_sum(ss, red);
+    inv_b = rsqrtf(ss / (float)hidden + eps);
+  }
   float ss2 = 0.f;
 #pragma unroll
-  for (int q = 0; q < SN_V; ++q) {
-    const int c = (threadIdx.x + q * 256) * 4;
+  for (int q = 0; q < V; ++q) {
+    const int c = threadIdx.x * 4 + q * step;
     x[q].x += v[q].x * inv_b * b[q].x; x[q].y += v[q].y * inv_b * b[q].y;
     x[q].z += v[q].z * inv_b * b[q].z; x[q].w += v[q].w * inv_b * b[q].w;
     if (c < hidden) {
@@ -154,8 +183,8 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
   if (!out) return;
   if (!w) {          // the reader takes the stream itself: no norm, the row in the activation type
 #pragma unroll
-    for (int q = 0; q < SN_V; ++q) {
-      const int c = (threadIdx.x + q * 256) * 4;
+    for (int q = 0; q < V; ++q) {
+      const int c = threadIdx.x * 4 + q * step;
       if (c < hidden) sn_store4<T>(out + i * hidden + c, x[q]);
     }
     return;
@@ -163,26 +192,25 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
   ss2 = block_sum(ss2, red);
   const float inv = rsqrtf(ss2 / (float)hidden + eps_out);
 #pragma unroll
-  for (int q = 0; q < SN_V; ++q) {
-    const int c = (threadIdx.x + q * 256) * 4;
-    if (c < hidden) {
-      const float4 g = *(const float4*)(w + c);
-      const float4 o = float4{x[q].x * inv * g.x, x[q].y * inv * g.y, x[q].z * inv * g.z, x[q].w * inv * g.w};
-      if constexpr (FILTER) {
-        // the input in the activation type, as a later step reads it
-        const float4 u = float4{to_f32(from_f32<T>(o.x)), to_f32(from_f32<T>(o.y)), to_f32(from_f32<T>(o.z)), to_f32(from_f32<T>(o.w))};
-        float* st = f.state + (long long)f.slot_ids[r] * f.lags * hidden + c;
-        float4 acc = float4{0.f, 0.f, 0.f, 0.f};
-        for (int j = 0; j <= f.lags; ++j) {
-          const float4 in = j < f.lags ? *(const float4*)(st + (long long)j * hidden) : u;
-          const float4 k = *(const float4*)(f.wt + (long long)j * hidden + c);
-          acc = float4{fmaf(k.x, in.x, acc.x), fmaf(k.y, in.y, acc.y), fmaf(k.z, in.z, acc.z), fmaf(k.w, in.w, acc.w)};
-          if (j > 0) *(float4*)(st + (long long)(j - 1) * hidden) = in;
-        }
-        sn_store4<T>(out + i * hidden + c, float4{acc.x + u.x, acc.y + u.y, acc.z + u.z, acc.w + u.w});
-      } else {
-        sn_store4<T>(out + i * hidden + c, o);
+  for (int q = 0; q < V; ++q) {
+    const int c = threadIdx.x * 4 + q * step;
+    if (c >= hidden) continue;
+    const float4 o = float4{x[q].x * inv * g[q].x, x[q].y * inv * g[q].y, x[q].z * inv * g[q].z, x[q].w * inv * g[q].w};
+    if constexpr (L > 0) {
+      // the input in the activation type, as a later step reads it
+      const float4 u = float4{to_f32(from_f32<T>(o.x)), to_f32(from_f32<T>(o.y)), to_f32(from_f32<T>(o.z)), to_f32(from_f32<T>(o.w))};
+      float4 acc = zero4;
+#pragma unroll
+      for (int j = 0; j <= L; ++j) {
+        if (j > f.lags) break;
+        const float4 in = j < f.lags ? past[q * L + (j < L ? j : 0)] : u;
+        const float4 k = tap[q * (L + 1) + j];
+        acc = float4{fmaf(k.x, in.x, acc.x), fmaf(k.y, in.y, acc.y), fmaf(k.z, in.z, acc.z), fmaf(k.w, in.w, acc.w)};
+        if (j > 0) *(float4*)(st + (long long)(j - 1) * hidden + c) = in;
       }
+      sn_store4<T>(out + i * hidden + c, float4{acc.x + u.x, acc.y + u.y, acc.z + u.z, acc.w + u.w});
+    } else {
+      sn_store4<T>(out + i * hidden + c, o);
     }
   }
 }
@@ -197,7 +225,10 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
     if (n_out <= 0 || hidden <= 0) return 0;                                                             \
     if ((!y && n_parts <= 0) || hidden > 16384) return (int)hipErrorInvalidValue;                        \
     if (hidden % 4 == 0 && hidden <= 4 * SN_V * 256) {                                                   \
-      hipLaunchKernelGGL((postnorm_add_rmsnorm_vec_kernel<T, false>), dim3(n_out), dim3(256), 0,         \
+      const bool few = n_out <= SN_FEW_ROWS;                                                             \
+      auto kernel = few || hidden <= 1024 ? postnorm_add_rmsnorm_vec_kernel<T, 1, 0>                     \
+                    : hidden <= 2048 ? postnorm_add_rmsnorm_vec_kernel<T, 2, 0> : postnorm_add_rmsnorm_vec_kernel<T, SN_V, 0>; \
+      hipLaunchKernelGGL(kernel, dim3(n_out), dim3(few ? (hidden / 4 + 63) / 64 * 64 : 256), 0,          \
                          (hipStream_t)stream, h, (const T*)y, parts, n_parts, part_stride, bias, wb, w,  \
                          (T*)out, rows, hidden, eps, eps_out, plain_scale, SnFilter{});                  \
       return JV_LAUNCH_CHECK();                                                                          \
@@ -213,10 +244,11 @@ postnorm_add_rmsnorm_vec_kernel(float* __restrict__ h, const T* __restrict__ y, 
                                       int n, int hidden, float eps, float eps_out, const float* wt,        \
                                       float* state, const int* slot_ids, int taps, void* stream) {         \
     if (n <= 0 || hidden <= 0) return 0;                                                                 \
-    if (hidden % 4 || hidden > 4 * SN_V * 256 || !w || !out || !wt || taps < 1 ||                        \
+    if (hidden % 4 || hidden > 4 * SN_V * 256 || !w || !out || !wt || taps < 1 || taps > 8 ||            \
         (taps > 1 && (!state || !slot_ids)))                                                             \
       return (int)hipErrorInvalidValue;                                                                  \
-    hipLaunchKernelGGL((postnorm_add_rmsnorm_vec_kernel<T, true>), dim3(n), dim3(256), 0,                \
+    auto kernel = taps <= 4 ? postnorm_add_rmsnorm_vec_kernel<T, 1, 3> : postnorm_add_rmsnorm_vec_kernel<T, 1, 7>; \
+    hipLaunchKernelGGL(kernel, dim3(n), dim3((hidden / 4 + 63) / 64 * 64), 0,                            \
                        (hipStream_t)stream, h, (const T*)y, parts, n_parts, part_stride,                 \
                        (const float*)nullptr, wb, w, (T*)out, (const int*)nullptr, hidden, eps, eps_out,  \
                        1.f, SnFilter{wt, state, slot_ids, taps - 1});                                    \

@@ -12,9 +12,10 @@
 #include "common.h"
 
 #define TF_MAX_LAGS 7
-#define TF_SEG 16
+#define TF_RUN 8          // rows a thread asks for at once; a segment of token_filter
 
 template <typename T, int E> struct TfVec { typedef T type __attribute__((ext_vector_type(E))); };
+template <typename T> struct TfVec<T, 1> { struct type { T v; __device__ T operator[](int) const { return v; } }; };
 
 template <typename T, int E> __device__ __forceinline__ void tf_load(const T* p, float (&v)[E]) {
   if constexpr (E == 1) {
@@ -24,6 +25,10 @@ template <typename T, int E> __device__ __forceinline__ void tf_load(const T* p,
 #pragma unroll
     for (int e = 0; e < E; ++e) v[e] = to_f32<T>(x[e]);
   }
+}
+template <typename T, int E> __device__ __forceinline__ void tf_widen(const typename TfVec<T, E>::type& x, float (&v)[E]) {
+#pragma unroll
+  for (int e = 0; e < E; ++e) v[e] = to_f32<T>(x[e]);
 }
 template <typename T, int E> __device__ __forceinline__ void tf_store(T* p, const float (&v)[E]) {
   if constexpr (E == 1) {
@@ -88,7 +93,7 @@ __device__ __forceinline__ void tf_leave_state(const T* in, long long ld, int n,
   }
 }
 
-// grid (requests, blocks of 256 pieces of E channels, segments of TF_SEG tokens)
+// grid (requests, blocks of 256 pieces of E channels, segments of TF_RUN tokens)
 template <typename T, int E, int L>
 __global__ void __launch_bounds__(256)
 token_filter_kernel(T* __restrict__ out, const T* __restrict__ x, int channels, int lags, const float* __restrict__ wt,
@@ -96,21 +101,25 @@ token_filter_kernel(T* __restrict__ out, const T* __restrict__ x, int channels, 
   const int r = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * E;
   if (c >= channels) return;
   const int t0 = cu_seqlens[r], n = cu_seqlens[r + 1] - t0;
-  const int s0 = blockIdx.z * TF_SEG;
+  const int s0 = blockIdx.z * TF_RUN;
   if (s0 >= n) return;
   float* st = state + (long long)slot_ids[r] * lags * channels + c;
   const T* in = x + (long long)t0 * channels + c;
   T* o = out + (long long)t0 * channels + c;
+  typename TfVec<T, E>::type raw[TF_RUN];
+#pragma unroll
+  for (int u = 0; u < TF_RUN; ++u) raw[u] = *(const typename TfVec<T, E>::type*)(in + (long long)min(s0 + u, n - 1) * channels);
   TfWindow<E, L> f;
   f.open(in, channels, s0, st, lags, channels, wt + c);
-  const int s1 = min(n, s0 + TF_SEG);
-  for (int i = s0; i < s1; ++i) {
+#pragma unroll
+  for (int u = 0; u < TF_RUN; ++u) {
+    if (s0 + u >= n) break;
     float a[E], y[E];
-    tf_load<T, E>(in + (long long)i * channels, a);
+    tf_widen<T, E>(raw[u], a);
     f.step(a, y);
 #pragma unroll
     for (int e = 0; e < E; ++e) y[e] += a[e];
-    tf_store<T, E>(o + (long long)i * channels, y);
+    tf_store<T, E>(o + (long long)(s0 + u) * channels, y);
   }
   if (blockIdx.z == 0) tf_leave_state<T, E>(in, channels, n, st, lags, channels);
 }
@@ -120,9 +129,10 @@ token_filter_kernel(T* __restrict__ out, const T* __restrict__ x, int channels, 
 //   q, k: the pairs (2i, 2i + 1) of a head's first rot_dims elements turn by the token's angles k_cs [n][rot_dims]
 //   v:    all pairs (2m, 2m + 1) turn by v_cs [n][dv]          (null: values as filtered)
 // q goes to rows [n][nq][dp] (zeros behind dk), k to pages [page][nkv][slot][dp], v to transposed pages
-// [page][nkv][dp][slot]; the pad of the pages is never written.  grid (requests, blocks of 256 pieces, segments of
-// TF_SEG positions): segments are cut at positions that are multiples of 8, so that 8 tokens of a value element that
-// lie side by side in a page are written as one piece.
+// [page][nkv][dp][slot]; the pad of the pages is never written.  grid (requests, blocks of 256 pieces, segments):
+// segments are cut at positions that are multiples of 8, so that 8 tokens of a value element that lie side by side in
+// a page are written as one piece.  The first one has 16 positions (its first multiple of 8 may lie up to 7 before the
+// step: 9 rows at least), the others 8.  ONE: a step of one token a request.
 template <typename T> struct alignas(sizeof(T) * 8) TfPack8 { T v[8]; };
 
 template <int E>
@@ -138,7 +148,7 @@ __device__ __forceinline__ void tf_turn(float (&y)[E], const float* cs, int half
   }
 }
 
-template <typename T, int E, int L>
+template <typename T, int E, int L, bool ONE>
 __global__ void __launch_bounds__(256)
 attn_prepare_filtered_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, long long ld, int lags,
                              const float* __restrict__ wt, float* __restrict__ state, const int* __restrict__ slot_ids,
@@ -146,90 +156,90 @@ attn_prepare_filtered_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, l
                              const float* __restrict__ k_cs, int rot_dims, const float* __restrict__ v_cs,
                              const int* __restrict__ slot_mapping, T* __restrict__ k_pages, T* __restrict__ v_pages,
                              int page_size, int nq, int nkv, int dk, int dv, int dp) {
+  constexpr int RUN = ONE ? 1 : TF_RUN;
   const int channels = (nq + nkv) * dk + nkv * dv;
   const int r = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * E;
   if (c >= channels) return;
   const int t0 = cu_seqlens[r], n = cu_seqlens[r + 1] - t0;
-  const int lead = context_lens[r] & 7;            // the step's first position, relative to the multiple of 8 before it
-  const int base = (int)blockIdx.z * TF_SEG - lead;
-  const int i0 = max(0, base), i1 = min(n, base + TF_SEG);
+  int base = 0, seg = 1;
+  if (!ONE) {
+    const int lead = context_lens[r] & 7;          // the step's first position, relative to the multiple of 8 before it
+    base = (blockIdx.z == 0 ? 0 : 8 + 8 * (int)blockIdx.z) - lead;
+    seg = blockIdx.z == 0 ? 16 : 8;
+  }
+  const int i0 = max(0, base), i1 = min(n, base + seg);
   if (i0 >= i1) return;
   const int v_at = (nq + nkv) * dk;
   const bool is_v = c >= v_at, is_q = c < nq * dk;
   const int head = is_v ? (c - v_at) / dv : c / dk;                // k heads follow the q heads
   const int d0 = is_v ? (c - v_at) - head * dv : c - head * dk;
   const int kvh = is_v ? head : head - nq;
-  float* st = state + (long long)(slot_ids ? slot_ids[r] : 0) * lags * channels + c;
+  float* st = state + (long long)slot_ids[r] * lags * channels + c;
   const T* in = qkv + (long long)t0 * ld + c;
   TfWindow<E, L> f;
   f.open(in, ld, i0, st, lags, channels, wt ? wt + c : nullptr);
-  if (!is_v) {
-    for (int i = i0; i < i1; ++i) {
+  for (int b0 = base; b0 < i1; b0 += RUN) {
+    typename TfVec<T, E>::type raw[RUN];
+    int sm[RUN];
+#pragma unroll
+    for (int u = 0; u < RUN; ++u) {
+      const int i = min(max(b0 + u, i0), i1 - 1);
+      raw[u] = *(const typename TfVec<T, E>::type*)(in + (long long)i * ld);
+      sm[u] = is_q ? -1 : slot_mapping[t0 + i];
+    }
+    TfPack8<T> pk[ONE ? 1 : E];
+#pragma unroll
+    for (int u = 0; u < RUN; ++u) {
+      const int i = b0 + u;
+      if (i < i0 || i >= i1) { sm[u] = -1; continue; }
       const long long t = t0 + i;
       float a[E], y[E];
-      tf_load<T, E>(in + (long long)i * ld, a);
+      tf_widen<T, E>(raw[u], a);
       f.step(a, y);
+      if (is_v) {
+        if (v_cs) tf_turn<E>(y, v_cs + t * dv, dv >> 1, d0, dv);
+        if constexpr (ONE) {
+          if (sm[u] >= 0) {
+            const long long page = sm[u] / page_size;
+            T* dst = v_pages + ((page * nkv + kvh) * dp + d0) * (long long)page_size + (sm[u] - (int)page * page_size);
+#pragma unroll
+            for (int e = 0; e < E; ++e) dst[(long long)e * page_size] = from_f32<T>(y[e]);
+          }
+        } else {
+#pragma unroll
+          for (int e = 0; e < E; ++e) pk[e].v[u] = from_f32<T>(y[e]);
+        }
+        continue;
+      }
       if (rot_dims) tf_turn<E>(y, k_cs + t * rot_dims, rot_dims >> 1, d0, rot_dims);
       if (is_q) {
         T* dst = q_out + (t * nq + head) * dp;
         tf_store<T, E>(dst + d0, y);
         if (d0 + E == dk)
           for (int p = dk; p < dp; ++p) dst[p] = from_f32<T>(0.f);
-      } else {
-        const int sm = slot_mapping[t];
-        if (sm >= 0) {
-          const long long page = sm / page_size;
-          tf_store<T, E>(k_pages + ((page * nkv + kvh) * page_size + (sm - (int)page * page_size)) * (long long)dp + d0, y);
-        }
+      } else if (sm[u] >= 0) {
+        const long long page = sm[u] / page_size;
+        tf_store<T, E>(k_pages + ((page * nkv + kvh) * page_size + (sm[u] - (int)page * page_size)) * (long long)dp + d0, y);
       }
     }
-  } else {
-    for (int run = 0; run < TF_SEG; run += 8) {
-      const int b0 = base + run;
-      if (b0 >= i1) break;
-      if (b0 >= i0 && b0 + 8 <= i1) {              // 8 tokens at once
-        TfPack8<T> pk[E];
+    if constexpr (!ONE) {
+      if (!is_v) continue;
+      bool side_by_side = sm[0] >= 0 && (sm[0] & 7) == 0 && (page_size & 7) == 0;      // 8 tokens at once
 #pragma unroll
-        for (int u = 0; u < 8; ++u) {
-          float a[E], y[E];
-          tf_load<T, E>(in + (long long)(b0 + u) * ld, a);
-          f.step(a, y);
-          if (v_cs) tf_turn<E>(y, v_cs + (long long)(t0 + b0 + u) * dv, dv >> 1, d0, dv);
+      for (int u = 1; u < RUN; ++u) side_by_side = side_by_side && sm[u] == sm[0] + u;
+      if (side_by_side) {
+        const long long page = sm[0] / page_size;
+        T* dst = v_pages + ((page * nkv + kvh) * dp + d0) * (long long)page_size + (sm[0] - (int)page * page_size);
 #pragma unroll
-          for (int e = 0; e < E; ++e) pk[e].v[u] = from_f32<T>(y[e]);
-        }
-        const int* sm8 = slot_mapping + t0 + b0;
-        bool side_by_side = sm8[0] >= 0 && (sm8[0] & 7) == 0 && (page_size & 7) == 0;
-#pragma unroll
-        for (int u = 1; u < 8; ++u) side_by_side = side_by_side && sm8[u] == sm8[0] + u;
-        if (side_by_side) {
-          const long long page = sm8[0] / page_size;
-          T* dst = v_pages + ((page * nkv + kvh) * dp + d0) * (long long)page_size + (sm8[0] - (int)page * page_size);
-#pragma unroll
-          for (int e = 0; e < E; ++e) *(TfPack8<T>*)(dst + (long long)e * page_size) = pk[e];
-        } else {
-#pragma unroll
-          for (int u = 0; u < 8; ++u) {
-            const int sm = sm8[u];
-            if (sm < 0) continue;
-            const long long page = sm / page_size;
-            T* dst = v_pages + ((page * nkv + kvh) * dp + d0) * (long long)page_size + (sm - (int)page * page_size);
-#pragma unroll
-            for (int e = 0; e < E; ++e) dst[(long long)e * page_size] = pk[e].v[u];
-          }
-        }
+        for (int e = 0; e < E; ++e) *(TfPack8<T>*)(dst + (long long)e * page_size) = pk[e];
       } else {
-        for (int i = max(b0, i0); i < min(b0 + 8, i1); ++i) {
-          float a[E], y[E];
-          tf_load<T, E>(in + (long long)i * ld, a);
-          f.step(a, y);
-          if (v_cs) tf_turn<E>(y, v_cs + (long long)(t0 + i) * dv, dv >> 1, d0, dv);
-          const int sm = slot_mapping[t0 + i];
-          if (sm < 0) continue;
-          const long long page = sm / page_size;
-          T* dst = v_pages + ((page * nkv + kvh) * dp + d0) * (long long)page_size + (sm - (int)page * page_size);
 #pragma unroll
-          for (int e = 0; e < E; ++e) dst[(long long)e * page_size] = from_f32<T>(y[e]);
+        for (int u = 0; u < RUN; ++u) {
+          if (sm[u] < 0) continue;
+          const long long page = sm[u] / page_size;
+          T* dst = v_pages + ((page * nkv + kvh) * dp + d0) * (long long)page_size + (sm[u] - (int)page * page_size);
+#pragma unroll
+          for (int e = 0; e < E; ++e) dst[(long long)e * page_size] = pk[e].v[u];
         }
       }
     }
@@ -299,8 +309,9 @@ struct TfAttn {
 };
 
 template <typename T, int E, int L>
-static void launch_attn_prepare_filtered(dim3 grid, hipStream_t stream, T* q_out, const T* qkv, T* k_pages, T* v_pages, const TfAttn& a) {
-  hipLaunchKernelGGL((attn_prepare_filtered_kernel<T, E, L>), grid, dim3(256), 0, stream, q_out, qkv, a.ld, a.lags, a.wt, a.state,
+static void launch_attn_prepare_filtered(dim3 grid, bool one, hipStream_t stream, T* q_out, const T* qkv, T* k_pages, T* v_pages, const TfAttn& a) {
+  auto kernel = one ? attn_prepare_filtered_kernel<T, E, L, true> : attn_prepare_filtered_kernel<T, E, L, false>;
+  hipLaunchKernelGGL(kernel, grid, dim3(256), 0, stream, q_out, qkv, a.ld, a.lags, a.wt, a.state,
                      a.slot_ids, a.cu_seqlens, a.context_lens, a.k_cs, a.rot_dims, a.v_cs, a.slot_mapping, k_pages, v_pages,
                      a.page_size, a.nq, a.nkv, a.dk, a.dv, a.dp);
 }
@@ -315,7 +326,7 @@ static void launch_attn_prepare_filtered(dim3 grid, hipStream_t stream, T* q_out
     const bool vec = channels % EP == 0 && tf_aligned(out, 16) && tf_aligned(x, 16) && tf_aligned(wt, 32) &&       \
                      tf_aligned(state, 32);                                                                        \
     const int pieces = vec ? channels / EP : channels;                                                             \
-    const int segs = (max_q_len + TF_SEG - 1) / TF_SEG;                                                            \
+    const int segs = (max_q_len + TF_RUN - 1) / TF_RUN;                                                            \
     if ((pieces + 255) / 256 > 65535 || segs > 65535) return (int)hipErrorInvalidValue;                            \
     const dim3 grid(n_requests, (pieces + 255) / 256, segs);                                                       \
     if (vec)                                                                                                       \
@@ -331,7 +342,7 @@ static void launch_attn_prepare_filtered(dim3 grid, hipStream_t stream, T* q_out
       int nkv, int dk, int dv, int dp, void* stream) {                                                             \
     if (n_requests <= 0 || max_q_len <= 0) return 0;                                                               \
     if (taps < 1 || taps > TF_MAX_LAGS + 1 || (taps > 1 && (!wt || !state || !slot_ids)) || nq <= 0 || nkv <= 0 || \
-        dk <= 0 || dv <= 0 || dk % 2 || dv % 2 || dp < dk || dp < dv || rot_dims < 0 || rot_dims > dk ||           \
+        !slot_ids || dk <= 0 || dv <= 0 || dk % 2 || dv % 2 || dp < dk || dp < dv || rot_dims < 0 || rot_dims > dk ||           \
         rot_dims % 2 || (rot_dims && !k_cs) || !slot_mapping || !k_pages || !v_pages || page_size <= 0)            \
       return (int)hipErrorInvalidValue;                                                                            \
     constexpr int EP = 16 / (int)sizeof(T);                                                                        \
@@ -340,7 +351,7 @@ static void launch_attn_prepare_filtered(dim3 grid, hipStream_t stream, T* q_out
     if (!vec && (dp % 2 || ld % 2)) return (int)hipErrorInvalidValue;                                              \
     if (page_size % 8 == 0 && !tf_aligned(v_pages, 8 * sizeof(T))) return (int)hipErrorInvalidValue;               \
     const int channels = (nq + nkv) * dk + nkv * dv, pieces = channels / (vec ? EP : 2);                           \
-    const int segs = max_q_len == 1 ? 1 : (max_q_len + 7 + TF_SEG - 1) / TF_SEG;                                   \
+    const int segs = max_q_len <= 9 ? 1 : (max_q_len + 7 - 16 + 7) / 8 + 1;                                        \
     if ((pieces + 255) / 256 > 65535 || segs > 65535) return (int)hipErrorInvalidValue;                            \
     const TfAttn a{ld, taps - 1, wt, state, slot_ids, cu_seqlens, context_lens, k_cs, rot_dims, v_cs, slot_mapping, \
                    page_size, nq, nkv, dk, dv, dp};                                                                \
@@ -349,7 +360,7 @@ static void launch_attn_prepare_filtered(dim3 grid, hipStream_t stream, T* q_out
                                    : launch_attn_prepare_filtered<T, EP, TF_MAX_LAGS>)                             \
                       : (taps <= 4 ? launch_attn_prepare_filtered<T, 2, 3>                                         \
                                    : launch_attn_prepare_filtered<T, 2, TF_MAX_LAGS>);                             \
-    launch(grid, (hipStream_t)stream, (T*)q_out, (const T*)qkv, (T*)k_pages, (T*)v_pages, a);                      \
+    launch(grid, max_q_len == 1, (hipStream_t)stream, (T*)q_out, (const T*)qkv, (T*)k_pages, (T*)v_pages, a);                      \
     return JV_LAUNCH_CHECK();                                                                                      \
   }                                                                                                                \
   extern "C" int jv_rotate_back_gate_##SUF(void* o, const void* g, long long ldg, const float* v_cs, long long n,  \

@@ -124,6 +124,7 @@ class EngineCore:
         # the recorded step's plan for other requests)
         self._replayable = model.replayable()
         self._spare_slot = config.max_num_seqs     # the state row of rows that pad a captured step
+        self._spare_rows = self._state_rows([self._spare_slot])
         self.graph_replays = 0
         self.steps_followed = 0              # decode steps started before the tokens of the step before were on the host
 
@@ -272,9 +273,8 @@ class EngineCore:
         if r < rb:
             # rows that pad the step write the spare state row: it starts from zero in every step, so
             # that a mixer which keeps adding to its state never runs it up to infinity there
-            for m in self.memories:
-                for st in m.states.values():
-                    st[self._spare_slot].zero_()
+            if self._spare_rows:
+                torch._foreach_zero_(self._spare_rows)
         g.dev.copy_(g.host_tensor, non_blocking=True)
         if g.copied is None:
             g.copied = torch.cuda.Event()
@@ -299,13 +299,14 @@ class EngineCore:
             self.graph_replays += 1
         return g.logits[:r]
 
+    def _state_rows(self, slots) -> list:
+        """These slots' rows of every state tensor."""
+        return [st[s] for m in self.memories for st in m.states.values() if st[0].numel() for s in slots]
+
     def _zero_new_state(self) -> None:
-        slots = self.cache.take_new_slots()
-        if slots and any(m.states for m in self.memories):
-            idx = torch.tensor(slots, dtype=torch.long, device=self.device)
-            for m in self.memories:
-                for st in m.states.values():
-                    st.index_fill_(0, idx, 0)
+        rows = self._state_rows(self.cache.take_new_slots())
+        if rows:
+            torch._foreach_zero_(rows)      # few launches for all of a model's state tensors
 
     def _build(self, entries):
         """All per-token and per-request integers of the step, packed on the host into one

@@ -1697,12 +1697,40 @@ def moe_tile_rows() -> int:
     return library.core().jv_moe_tile_rows()
 
 
+MOE_SKINNY_ROWS = 16            # rows of a tile of the weight-streaming expert kernels
+MOE_SKINNY_MAX_MEAN = 6         # up to so many rows an expert (on average over all experts) they are preferred
+
+
 def moe_tile_rows_for(dtype, hidden: int, ff: int, entries: int, experts: int) -> int:
-    """Rows of a tile for a step: 128 where the matrix-core kernels run and an expert gets about a
-    hundred rows or more (a row of W then feeds twice the products), else 64."""
-    if moe_matrix_cores_possible(dtype, hidden, ff) and entries >= 96 * experts:
-        return 128
+    """Rows of a tile for a step: 16 (the kernels that stream the experts' weights) where an expert gets a few rows at
+    most, 128 where the matrix-core kernels run and an expert gets about a hundred rows or more (a row of W then feeds
+    twice the products), else 64."""
+    if moe_matrix_cores_possible(dtype, hidden, ff):
+        if entries <= MOE_SKINNY_MAX_MEAN * experts:
+            return MOE_SKINNY_ROWS
+        if entries >= 96 * experts:
+            return 128
     return moe_tile_rows()
+
+
+def moe_always_possible(x, w_router, top: int, always: int) -> bool:
+    """Whether ``moe_route(None, top, x=x, w_router=w_router, always=always)`` runs: bfloat16 rows whose logits come from a
+    product of their own, few enough for the one-block form."""
+    n = x.shape[0]
+    return (_router_logits_plan(x, w_router) is not None
+            and bool(library.core().jv_moe_route_group_fits(c_int(n), c_int(w_router.shape[0]), c_int(top), c_int(always))))
+
+
+def _router_logits_plan(x, w_router):
+    """How the router logits of bfloat16 rows are made by a product with float output: a ``streaming_plan`` for few rows,
+    "rows" for the tiled product, None where the fused kernel (or the float one) makes them."""
+    if x.dtype != torch.bfloat16 or x.shape[1] % 8 or x.shape[1] < 8 or w_router.shape[0] > 3840:
+        return None
+    rows = x.shape[0]
+    if rows <= SKINNY_AUTO_ROWS:
+        plan = streaming_plan(rows, w_router.shape[0], w_router.shape[1], device=x.device)
+        return plan if plan is not None and plan[1] == 1 else None
+    return "rows" if rows > ROUTER_FUSED_MAX_ROWS else None
 
 
 ROUTER_FUSED_MAX_ROWS = 64      # 17..64 rows: logits and choice in one launch
@@ -1737,7 +1765,7 @@ ROUTER_MAX_GROUPS = 64
 
 def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, logits_out=None,
               tile_rows: "int | None" = None, bias=None, score: str = "sigmoid", correction=None,
-              weight_scale: float = 1.0, groups: "tuple | None" = None) -> MoePlan:
+              weight_scale: float = 1.0, groups: "tuple | None" = None, always: int = 0) -> MoePlan:
     """Chooses for every token the ``top`` experts with the largest router logits (the lowest index among equal
     logits) and orders the n * top entries by expert, all on the device.  ``bias`` (float32 [experts]) is added
     to the logits before the choice; ``score``: a chosen expert's weight is "sigmoid" of its logit, or
@@ -1746,22 +1774,22 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     sigmoid(logit) (without the correction) over the sum of the chosen ones' (+ 1e-20), times ``weight_scale``;
     or "softmax": the softmax over ALL of the token's logits.  ``groups`` (count, keep): the experts form ``count`` equal
     groups of neighbours, and only those of the ``keep`` groups with the largest logits can be chosen.
+    ``always`` (few tokens: ``moe_always_possible``): every token also gets the ``always`` experts behind the routed ones
+    (number experts, experts + 1, ...) with weight 1, behind its chosen ones; the plan's ``top`` then counts them in.
     Either float ``logits`` [n, experts] are given, or rows ``x`` [n, hidden] and the router matrix
     ``w_router`` [experts, hidden] of one type: then the logits are made here, in float (``logits_out``,
     float32 [n, experts], receives them if given): in the same launch as the choice (float32, odd sizes), or
     for bfloat16 by a matrix-core product with float output before it.  ``tile_rows``: rows of a tile of the grouping
     (``moe_tile_rows_for``; default: the float-FMA kernels' 64)."""
-    if (logits is None and x.dtype == torch.bfloat16 and x.shape[1] % 8 == 0 and x.shape[1] >= 8
-            and w_router.shape[0] <= 3840):
+    if logits is None:
         # bfloat16: the logits come from a matrix-core product with float output (never rounded to bfloat16): the
         # weight-streaming one for the few rows of a decode step, the tiled one for prompt portions; between
         # them (measured at 32 rows: one block of the tiled product walks the whole router alone) the fused kernel
-        rows = x.shape[0]
-        plan = streaming_plan(rows, w_router.shape[0], w_router.shape[1], device=x.device) if rows <= SKINNY_AUTO_ROWS else None
-        if plan is not None and plan[1] == 1:
-            logits = gemm_skinny(x, w_router, torch.float32, block_shape=plan[0])
-        elif rows > ROUTER_FUSED_MAX_ROWS:
+        how = _router_logits_plan(x, w_router)
+        if how == "rows":
             logits = gemm_rows_f32out(x, w_router)
+        elif how is not None:
+            logits = gemm_skinny(x, w_router, torch.float32, block_shape=how[0])
         if logits is not None and logits_out is not None:
             logits_out.copy_(logits if bias is None else logits + bias)
     _need(score in ROUTER_SCORES, f"no router score {score!r}: there are {sorted(ROUTER_SCORES)}")
@@ -1792,18 +1820,27 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     _need(count == 1 or (experts % count == 0 and count <= ROUTER_MAX_GROUPS and 0 < keep <= count
                          and keep * (experts // count) >= top and correction is None),
           "equal groups (at most 64), enough experts in the kept ones, and no correction of the choice")
-    entries = n * top
+    lib = library.core()
+    one_launch = logits is not None and bool(lib.jv_moe_route_group_fits(c_int(n), c_int(experts), c_int(top), c_int(always)))
+    _need(always == 0 or one_launch, "experts for every token take logits and few tokens")
+    all_experts, per = experts + always, top + always
+    entries = n * per
     tile_rows = tile_rows or moe_tile_rows()
-    _need(tile_rows in (64, 128), "tiles have 64 or 128 rows")
-    max_tiles = -(-entries // tile_rows) + experts
-    ints = torch.empty(entries * 3 + 1 + experts + 1 + 2 * max_tiles, dtype=torch.int32, device=dev)
+    _need(tile_rows in (16, 64, 128), "tiles have 16, 64 or 128 rows")
+    max_tiles = min(entries, -(-entries // tile_rows) + all_experts)
+    ints = torch.empty(entries * 3 + 1 + all_experts + 1 + 2 * max_tiles, dtype=torch.int32, device=dev)
     ids, rank, order = ints[:entries], ints[entries:2 * entries], ints[2 * entries:3 * entries]
     at = 3 * entries
-    meta, offsets = ints[at:at + 1], ints[at + 1:at + 2 + experts]
-    at += 2 + experts
+    meta, offsets = ints[at:at + 1], ints[at + 1:at + 2 + all_experts]
+    at += 2 + all_experts
     tile_expert, tile_row0 = ints[at:at + max_tiles], ints[at + max_tiles:at + 2 * max_tiles]
     weights = torch.empty(entries, dtype=torch.float32, device=dev)
-    lib = library.core()
+    if one_launch:
+        _check(lib.jv_moe_route_group(_ptr(logits), _ptr(bias), c_int(n), c_int(experts), c_int(top), c_int(always),
+                                      c_int(ROUTER_SCORES[score]), _ptr(ids), _ptr(weights), _ptr(correction),
+                                      c_float(weight_scale), c_int(count), c_int(keep), c_int(tile_rows), _ptr(meta),
+                                      _ptr(offsets), _ptr(tile_expert), _ptr(tile_row0), _ptr(order), _stream()), "moe_route_group")
+        return MoePlan(ids, weights, meta, offsets, tile_expert, tile_row0, order, max_tiles, per, tile_rows)
     if logits is not None:
         _check(lib.jv_moe_route(_ptr(logits), _ptr(bias), c_int(n), c_int(experts), c_int(top), c_int(ROUTER_SCORES[score]),
                                 _ptr(ids), _ptr(weights), _ptr(correction), c_float(weight_scale), c_int(count), c_int(keep),
@@ -1862,6 +1899,18 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
     mfma = possible and matrix_cores is not False
     _need(mfma or plan.tile_rows == moe_tile_rows(), "the float-FMA kernels take tiles of 64 rows")
     p = plan
+    _need(mfma or p.tile_rows != MOE_SKINNY_ROWS, "tiles of 16 rows belong to the weight-streaming kernels")
+    if mfma and p.tile_rows == MOE_SKINNY_ROWS:
+        _need(lib.jv_moe_skinny_rows() == MOE_SKINNY_ROWS, "the library's tiles have another size")
+        _check(lib.jv_moe_gate_up_skinny_bf16(
+            _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),
+            _ptr(p.tile_row0), _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(hidden), c_int(ff),
+            c_int(act), c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
+        _check(lib.jv_moe_down_skinny_bf16(
+            _ptr(out), _ptr(z), _ptr(w_down), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert), _ptr(p.tile_row0),
+            _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(n), c_int(hidden), c_int(ff),
+            c_int(0 if weight_on_input else 1), _stream()), "moe_down")
+        return
     if mfma:
         _check(lib.jv_moe_gate_up_mfma_bf16(
             _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),

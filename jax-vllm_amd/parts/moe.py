@@ -13,6 +13,9 @@
 The score multiplies the expert's INPUT (``weight_on_input``; with False it multiplies the output).  Since
 the products are linear, s (W u) is computed instead of W (s u): in float, after the product.  Routing,
 the grouping of rows by expert and the two grouped products all run on the device (``ops.kernels.moe_*``).
+For the few tokens of a decode step a shared expert without a gate whose size is a multiple of the experts' rides in
+the grouped products as further experts that every token has with weight 1 (W_down act(W_up u) is a sum over the inner
+size, so it may be cut there): its own launches are saved.
 The result is handed on as (rows of the shared expert or None, float stack [top, tokens, hidden] of the
 chosen experts' outputs); the next norm adds them in that order.  A shared expert under a gate of the token's own
 (``shared_gate``) joins the float stack as one more share.
@@ -24,7 +27,10 @@ from typing import Optional
 import torch
 
 from ..ops import kernels as K
+from .mlp import DenseMLP
 from .spec import PartSpec, TensorSpec, build_part, is_replayable, register_part
+
+SHARED_ALONG_MAX_TOKENS = 16      # tokens of a step that takes the shared expert along (its rows then fill one tile)
 
 
 class RoutedExperts:
@@ -99,18 +105,45 @@ class RoutedExperts:
             self.correction = tensors["router.correction"].contiguous()
         if self.shared is not None:
             self.shared.bind({k[len("shared."):]: v for k, v in tensors.items() if k.startswith("shared.")}, dtype)
+        self.pieces = self._shared_pieces(dtype)
+        if self.pieces:
+            E, n, ff, hid = self.experts, self.pieces, self.ff, self.hidden_size
+            up, down = self.shared.w_up, self.shared.w_down
+            self.w_up = torch.cat([self.w_up, up.view(n, ff, hid)]).contiguous()
+            self.w_down = torch.cat([self.w_down, down.view(hid, n, ff).transpose(0, 1)]).contiguous()
+            self.shared.w_up = self.w_up[E:].view(n * ff, hid)          # the same buffer
+            if n == 1:
+                self.shared.w_down = self.w_down[E]
         if self.shared_gate:
             w = tensors["shared_gate.weight"]
             self.w_shared_gate = torch.cat([w, w.new_zeros((7, w.shape[1]))]).contiguous()   # rows of 16 bytes and more
 
+    def _shared_pieces(self, dtype) -> int:
+        """The number of experts' sizes the shared expert is cut into for the steps that take it along, 0: it never is."""
+        s = self.shared
+        if (self.gated or self.shared_gate or not isinstance(s, DenseMLP) or s.bias or s.activation != self.activation
+                or s.intermediate_size % self.ff or not K.moe_matrix_cores_possible(dtype, self.hidden_size, self.ff)):
+            return 0
+        return s.intermediate_size // self.ff
+
     def forward(self, x, ctx=None):
         n = x.shape[0]
+        if (self.pieces and n <= SHARED_ALONG_MAX_TOKENS
+                and K.moe_always_possible(x, self.w_router, self.top, self.pieces)):
+            per = self.top + self.pieces
+            plan = K.moe_route(None, self.top, x=x, w_router=self.w_router, bias=self.b_router, score=self.score,
+                               tile_rows=K.MOE_SKINNY_ROWS, correction=self.correction, weight_scale=self.weight_scale,
+                               groups=self.groups, always=self.pieces)
+            out = torch.empty((per, n, self.hidden_size), dtype=torch.float32, device=x.device)
+            K.moe_experts(x, plan, None, self.w_up, self.w_down, self.activation, out, self.weight_on_input)
+            return None, out
         plan = K.moe_route(None, self.top, x=x, w_router=self.w_router, bias=self.b_router, score=self.score,
                            tile_rows=K.moe_tile_rows_for(x.dtype, self.hidden_size, self.ff, n * self.top, self.experts),
                            correction=self.correction, weight_scale=self.weight_scale, groups=self.groups)
         shares = self.top + (1 if self.shared_gate else 0)
         out = torch.empty((shares, n, self.hidden_size), dtype=torch.float32, device=x.device)
-        K.moe_experts(x, plan, self.w_gate, self.w_up, self.w_down, self.activation, out[:self.top], self.weight_on_input)
+        K.moe_experts(x, plan, self.w_gate, self.w_up[:self.experts], self.w_down[:self.experts],
+                      self.activation, out[:self.top], self.weight_on_input)
         rows = self.shared.forward(x, ctx) if self.shared is not None else None
         if self.shared_gate:
             K.row_gate(out[self.top], rows, K.linear(x, self.w_shared_gate)[:, :1])

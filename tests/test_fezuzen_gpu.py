@@ -826,6 +826,65 @@ def test_kernel_experts_without_a_gate(dtype, n, hidden, ff):
     assert float((out.double().cpu() - want).abs().max()) <= tol * float(want.abs().max())
 
 
+@pytest.mark.parametrize("gated", [False, True], ids=["plain", "gated"])
+@pytest.mark.parametrize("n", [1, 3, 16, 40])
+@pytest.mark.parametrize("hidden,ff,experts,top", [(64, 32, 5, 2), (40, 24, 8, 3), (2048, 328, 6, 2), (520, 1544, 4, 1)])
+def test_kernel_experts_streamed_for_few_tokens(gated, n, hidden, ff, experts, top):
+    """Tiles of 16 rows (one expert gets more than a tile): the weights streamed, the inner size shared out to the waves."""
+    from jax_vllm_amd.ops import kernels as K
+
+    g = torch.Generator().manual_seed(17)
+    bf = torch.bfloat16
+    x = torch.randn(n, hidden, generator=g).to(bf)
+    gate, up = ((torch.randn(experts, ff, hidden, generator=g) * hidden ** -0.5).to(bf) for _ in range(2))
+    down = (torch.randn(experts, hidden, ff, generator=g) * ff ** -0.5).to(bf)
+    logits = torch.randn(n, experts, generator=g)
+    logits[:, 1] += 3.0
+    for on_input in (False, True):
+        plan = K.moe_route(_dev(logits), top, score="softmax", tile_rows=16)
+        out = torch.empty(top, n, hidden, device="cuda")
+        K.moe_experts(_dev(x), plan, _dev(gate) if gated else None, _dev(up), _dev(down), "silu" if gated else "relu2", out, on_input)
+        ids, wts = plan.ids.view(n, top).cpu().long(), plan.weights.view(n, top).cpu().double()
+        want = torch.empty(top, n, hidden, dtype=torch.float64)
+        for t in range(n):
+            for k in range(top):
+                e, w = ids[t, k], wts[t, k]
+                u = up[e].double() @ x[t].double() * (w if on_input else 1.0)
+                q = gate[e].double() @ x[t].double() * (w if on_input else 1.0)
+                z = torch.nn.functional.silu(q) * u if gated else torch.relu(u) ** 2
+                want[k, t] = (1.0 if on_input else w) * (down[e].double() @ z)
+        assert float((out.double().cpu() - want).abs().max()) <= 2e-2 * float(want.abs().max())
+
+
+@pytest.mark.parametrize("n,experts,top,always,groups", [(1, 4, 1, 1, None), (8, 70, 3, 2, (7, 3)), (16, 9, 4, 3, None), (64, 130, 2, 0, (2, 1))])
+def test_kernel_router_and_grouping_in_one_launch(n, experts, top, always, groups):
+    """Every token has its chosen experts and the ones behind the routed experts; the grouping by experts and tiles."""
+    from jax_vllm_amd.ops import kernels as K
+
+    g = torch.Generator().manual_seed(18)
+    logits = torch.randn(n, experts, generator=g)
+    plan = K.moe_route(_dev(logits), top, score="softmax", groups=groups, always=always, tile_rows=16)
+    per = top + always
+    assert plan.top == per
+    ids, wts = plan.ids.view(n, per).cpu().long(), plan.weights.view(n, per).cpu().double()
+    f = {"router": {"experts": experts, "top": top}}
+    if groups:
+        f["router"]["groups"] = {"count": groups[0], "keep": groups[1]}
+    choice, weight = P.router({"router": torch.eye(experts, dtype=torch.float64)}, "", f, logits.double())
+    assert torch.equal(ids[:, :top], choice) and torch.allclose(wts[:, :top], weight, atol=1e-6)
+    assert torch.equal(ids[:, top:], torch.arange(experts, experts + always).expand(n, always)) and (wts[:, top:] == 1).all()
+    order, offsets, flat = plan.order.cpu().long(), plan.offsets.cpu().long(), ids.reshape(-1)
+    assert sorted(order.tolist()) == list(range(n * per)) and int(offsets[-1]) == n * per
+    tiles = []
+    for e in range(experts + always):
+        lo, hi = int(offsets[e]), int(offsets[e + 1])
+        assert (flat[order[lo:hi]] == e).all()
+        tiles += [(e, r) for r in range(lo, hi, 16)]
+    m = int(plan.meta.cpu()[0])
+    assert m == len(tiles) <= plan.max_tiles
+    assert list(zip(plan.tile_expert.cpu()[:m].tolist(), plan.tile_row0.cpu()[:m].tolist())) == tiles
+
+
 @BOTH
 def test_kernel_query_latent_alone(dtype):
     """A layer that reads another layer's cache norms its query latent and stores nothing."""
