@@ -29,6 +29,21 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// The maximum over a wave by moves between the lanes' registers (no LDS traffic): shifts inside the rows of 16 lanes, then
+// the rows' last lanes broadcast into the next rows; lane 63 ends up with the whole wave's, NaNs are not seen.
+template <int CTRL> __device__ __forceinline__ float lane_move(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(v), __float_as_int(v), CTRL, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float wave_max_lanes(float v) {
+  v = fmaxf(v, lane_move<0x111>(v));      // row_shr:1, 2, 4, 8
+  v = fmaxf(v, lane_move<0x112>(v));
+  v = fmaxf(v, lane_move<0x114>(v));
+  v = fmaxf(v, lane_move<0x118>(v));
+  v = fmaxf(v, lane_move<0x142>(v));      // row_bcast:15
+  v = fmaxf(v, lane_move<0x143>(v));      // row_bcast:31
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
+}
+
 // Sum over a whole block of up to 1024 threads; `red` is shared scratch of >= 17 floats.
 __device__ __forceinline__ float block_sum(float v, float* red) {
   const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE;

@@ -28,7 +28,7 @@
 #define MOE_SCORE_SIGMOID_NORMED 2   // chosen by sigmoid(logit) + correction; weight = sigmoid(logit) / (sum over the chosen + 1e-20) * scale
 #define MOE_SCORE_SOFTMAX 3          // weight = exp(logit) / sum of exp over all of the token's logits
 #define MOE_MAX_GROUPS 64
-#define MOE_RANK_EXPERTS 128         // up to so many experts are ranked by counting
+#define MOE_LANE_EXPERTS 256         // up to so many experts a lane keeps its own in registers
 __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int lane, int* ids, float* weights,
                                          int score, const float* __restrict__ correction, float weight_scale,
                                          int groups, int keep) {
@@ -57,53 +57,55 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
     for (int e = lane; e < experts; e += JV_WAVE)
       if (!((kept >> (e / size)) & 1)) zt[e] = -INFINITY;
   }
-  if (experts <= MOE_RANK_EXPERTS) {
-    // an expert's place is the number of experts ahead of it (a larger value, or an equal one of a lower number): every
-    // lane counts for its own experts over the values in LDS, instead of `top` searches across the wave one after the other
-    constexpr int PER = MOE_RANK_EXPERTS / JV_WAVE;
+  if (experts <= MOE_LANE_EXPERTS && top <= JV_WAVE) {
+    // the values stay in registers; per choice one maximum across the wave by lane moves within the registers' rows, and
+    // the lowest lane that holds it (the experts of the first 64 first); a taken expert becomes a NaN, which no maximum sees
+    constexpr int PER = MOE_LANE_EXPERTS / JV_WAVE;
     float z[PER], c[PER];
-    int ahead[PER];
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
       const int e = lane + i * JV_WAVE;
-      z[i] = e < experts ? zt[e] : -INFINITY;
+      z[i] = e < experts ? zt[e] : 0.f;
       c[i] = z[i];
-      if (normed && z[i] != -INFINITY) c[i] = 1.f / (1.f + expf(-z[i])) + (correction && e < experts ? correction[e] : 0.f);
+      if (normed && z[i] != -INFINITY && e < experts) c[i] = 1.f / (1.f + expf(-z[i])) + (correction ? correction[e] : 0.f);
       if (c[i] != c[i]) c[i] = -INFINITY;         // a NaN takes the last places, its weight shows it
-      ahead[i] = 0;
+      if (e >= experts) c[i] = __builtin_nanf("");
     }
+    float zk = 0.f;                               // of the lane's choice: lane kk keeps the kk-th
+    int ek = 0;
+    for (int kk = 0; kk < top; ++kk) {
+      float m = c[0];
 #pragma unroll
-    for (int i = 0; i < PER; ++i)
-      if (lane + i * JV_WAVE < experts) zt[lane + i * JV_WAVE] = c[i];
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // the values are read by the wave's other lanes
-    for (int e = 0; e < experts; ++e) {
-      const float o = zt[e];
+      for (int i = 1; i < PER; ++i) m = fmaxf(m, c[i]);
+      m = wave_max_lanes(m);
+      bool found = false;
 #pragma unroll
-      for (int i = 0; i < PER; ++i) ahead[i] += (o > c[i] || (o == c[i] && e < lane + i * JV_WAVE)) ? 1 : 0;
-    }
-    float s[PER], share = 0.f, most = -INFINITY;
-#pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const bool chosen = lane + i * JV_WAVE < experts && ahead[i] < top;
-      if (!chosen) ahead[i] = top;
-      else most = fmaxf(most, z[i]);
-    }
-    if (score == MOE_SCORE_SOFTMAX_CHOSEN) most = wave_max(most);
-#pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      s[i] = score == MOE_SCORE_SOFTMAX_CHOSEN ? expf(z[i] - most) : score == MOE_SCORE_SOFTMAX ? expf(z[i] - zmax) * inv_sum
-                                                                                             : 1.f / (1.f + expf(-z[i]));
-      if (ahead[i] < top) share += s[i];
-    }
-    float f = 1.f;
-    if (score == MOE_SCORE_SOFTMAX_CHOSEN) f = 1.f / wave_sum(share);
-    if (normed) f = weight_scale / (wave_sum(share) + 1e-20f);
-#pragma unroll
-    for (int i = 0; i < PER; ++i)
-      if (ahead[i] < top) {
-        ids[ahead[i]] = lane + i * JV_WAVE;
-        weights[ahead[i]] = s[i] * f;
+      for (int i = 0; i < PER; ++i) {
+        const unsigned long long at = __ballot(c[i] == m);
+        if (found || !at) continue;
+        found = true;
+        const int l = __ffsll(at) - 1;
+        const float zv = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(z[i]), l));
+        if (lane == kk) { zk = zv; ek = l + i * JV_WAVE; }
+        if (lane == l) c[i] = __builtin_nanf("");
       }
+    }
+    const bool mine = lane < top;
+    float w;
+    if (score == MOE_SCORE_SOFTMAX) {
+      w = expf(zk - zmax) * inv_sum;
+    } else if (score == MOE_SCORE_SOFTMAX_CHOSEN) {
+      const float first = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(zk), 0));      // the largest
+      w = mine ? expf(zk - first) : 0.f;
+      w *= 1.f / wave_sum(w);
+    } else {
+      w = mine ? 1.f / (1.f + expf(-zk)) : 0.f;
+      if (normed) w *= weight_scale / (wave_sum(w) + 1e-20f);
+    }
+    if (mine) {
+      ids[lane] = ek;
+      weights[lane] = w;
+    }
     return;
   }
   for (int kk = 0; kk < top; ++kk) {
@@ -295,10 +297,10 @@ moe_route_group_kernel(const float* __restrict__ logits, const float* __restrict
   int* count = rank + entries;
   int* start = count + all;
   int* tile0 = start + all + 1;
-  const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE;
+  const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE, waves = blockDim.x / JV_WAVE;
   for (int e = threadIdx.x; e < all; e += blockDim.x) count[e] = 0;
   float* zt = zs + wid * experts;
-  for (int t = wid; t < n; t += 16) {
+  for (int t = wid; t < n; t += waves) {
     for (int e = lane; e < experts; e += JV_WAVE) zt[e] = logits[(long long)t * experts + e] + (bias ? bias[e] : 0.f);
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");        // a group's lane reads what other lanes wrote
     moe_pick(zt, experts, top, lane, lid + t * per, weights + (long long)t * per, score, correction, weight_scale, groups, keep);
@@ -512,7 +514,8 @@ extern "C" int jv_moe_route_group(const float* logits, const float* bias, int n,
       !moe_groups_ok(experts, top, groups, keep) || tile_rows <= 0)
     return (int)hipErrorInvalidValue;
   const size_t shmem = (16 * (size_t)experts + 2 * (size_t)n * (top + always) + 3 * (size_t)(experts + always) + 2) * 4;
-  hipLaunchKernelGGL(moe_route_group_kernel, dim3(1), dim3(1024), shmem, (hipStream_t)stream, logits, bias, n, experts, top,
+  const int waves = n < 4 ? 4 : n > 16 ? 16 : n;
+  hipLaunchKernelGGL(moe_route_group_kernel, dim3(1), dim3(64 * waves), shmem, (hipStream_t)stream, logits, bias, n, experts, top,
                      always, score, ids, weights, correction, weight_scale, groups, keep, tile_rows, meta, offsets,
                      tile_expert, tile_row0, order);
   return JV_LAUNCH_CHECK();

@@ -12,6 +12,7 @@
 #include "common.h"
 
 #define TF_MAX_LAGS 7
+#define TF_BYTES 8        // of neighbouring channels a thread takes (2,048 tokens, 16 + 2 * 4 heads of 128: 15.6 us, with 16 bytes 20.3)
 #define TF_RUN 8          // rows a thread asks for at once; a segment of token_filter
 
 template <typename T, int E> struct TfVec { typedef T type __attribute__((ext_vector_type(E))); };
@@ -322,7 +323,7 @@ static void launch_attn_prepare_filtered(dim3 grid, bool one, hipStream_t stream
                                        int max_q_len, void* stream) {                                              \
     if (n_requests <= 0 || channels <= 0 || max_q_len <= 0) return 0;                                              \
     if (taps < 1 || taps > TF_MAX_LAGS + 1 || !wt || (taps > 1 && !state)) return (int)hipErrorInvalidValue;                     \
-    constexpr int EP = 16 / (int)sizeof(T);                                                                        \
+    constexpr int EP = TF_BYTES / (int)sizeof(T);                                                                        \
     const bool vec = channels % EP == 0 && tf_aligned(out, 16) && tf_aligned(x, 16) && tf_aligned(wt, 32) &&       \
                      tf_aligned(state, 32);                                                                        \
     const int pieces = vec ? channels / EP : channels;                                                             \
@@ -345,7 +346,7 @@ static void launch_attn_prepare_filtered(dim3 grid, bool one, hipStream_t stream
         !slot_ids || dk <= 0 || dv <= 0 || dk % 2 || dv % 2 || dp < dk || dp < dv || rot_dims < 0 || rot_dims > dk ||           \
         rot_dims % 2 || (rot_dims && !k_cs) || !slot_mapping || !k_pages || !v_pages || page_size <= 0)            \
       return (int)hipErrorInvalidValue;                                                                            \
-    constexpr int EP = 16 / (int)sizeof(T);                                                                        \
+    constexpr int EP = TF_BYTES / (int)sizeof(T);                                                                        \
     const bool vec = dk % EP == 0 && dv % EP == 0 && dp % EP == 0 && ld % EP == 0 && tf_aligned(qkv, 16) &&        \
                      tf_aligned(q_out, 16) && tf_aligned(k_pages, 16) && tf_aligned(wt, 32) && tf_aligned(state, 32); \
     if (!vec && (dp % 2 || ld % 2)) return (int)hipErrorInvalidValue;                                              \
@@ -367,7 +368,7 @@ static void launch_attn_prepare_filtered(dim3 grid, bool one, hipStream_t stream
                                            int heads, int dv, int dp, void* stream) {                              \
     if (n <= 0 || heads <= 0) return 0;                                                                            \
     if (dv <= 0 || dp < dv || (v_cs && dv % 2)) return (int)hipErrorInvalidValue;                                  \
-    constexpr int EP = 16 / (int)sizeof(T);                                                                        \
+    constexpr int EP = TF_BYTES / (int)sizeof(T);                                                                        \
     const bool vec = dv % EP == 0 && dp % EP == 0 && tf_aligned(o, 16) && (!g || (ldg % EP == 0 && tf_aligned(g, 16))); \
     const bool two = dv % 2 == 0 && dp % 2 == 0 && (!g || (ldg % 2 == 0 && tf_aligned(g, 2 * sizeof(T))));         \
     if (!vec && !two && v_cs) return (int)hipErrorInvalidValue;                                                    \
