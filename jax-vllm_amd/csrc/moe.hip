@@ -283,10 +283,10 @@ moe_group_kernel(const int* __restrict__ ids, int entries, int experts, int tile
 // Choice and grouping of few tokens in one launch of one block: a wave a token picks, then the block groups.  Every
 // token has `top` chosen entries and `always` further ones, for the experts behind the routed ones (number experts,
 // experts + 1, ...), whose weight is 1: a shared expert cut into pieces of the routed ones' size.  Entry s = token *
-// (top + always) + kk.  LDS: logits [16][experts] | ids [entries] | rank [entries] | count, start, first tile of experts + always.
+// (top + always) + kk.  The logits may come as `parts` partial products, added here in their order.  LDS: logits [16][experts] | ids [entries] | rank [entries] | count, start, first tile of experts + always.
 __global__ void __launch_bounds__(1024)
-moe_route_group_kernel(const float* __restrict__ logits, const float* __restrict__ bias, int n, int experts, int top,
-                       int always, int score, int* __restrict__ ids, float* __restrict__ weights,
+moe_route_group_kernel(const float* __restrict__ logits, int parts, long long part_stride,
+                       const float* __restrict__ bias, int n, int experts, int top, int always, int score, int* __restrict__ ids, float* __restrict__ weights,
                        const float* __restrict__ correction, float weight_scale, int groups, int keep, int tile_rows,
                        int* __restrict__ meta, int* __restrict__ offsets, int* __restrict__ tile_expert,
                        int* __restrict__ tile_row0, int* __restrict__ order) {
@@ -301,7 +301,18 @@ moe_route_group_kernel(const float* __restrict__ logits, const float* __restrict
   for (int e = threadIdx.x; e < all; e += blockDim.x) count[e] = 0;
   float* zt = zs + wid * experts;
   for (int t = wid; t < n; t += waves) {
-    for (int e = lane; e < experts; e += JV_WAVE) zt[e] = logits[(long long)t * experts + e] + (bias ? bias[e] : 0.f);
+    for (int e = lane; e < experts; e += JV_WAVE) {
+      const float* at = logits + (long long)t * experts + e;
+      float z = 0.f;
+      for (int p0 = 0; p0 < parts; p0 += 8) {                     // eight asked for before they are added
+        float v[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) v[u] = at[min(p0 + u, parts - 1) * part_stride];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) z += p0 + u < parts ? v[u] : 0.f;
+      }
+      zt[e] = z + (bias ? bias[e] : 0.f);
+    }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");        // a group's lane reads what other lanes wrote
     moe_pick(zt, experts, top, lane, lid + t * per, weights + (long long)t * per, score, correction, weight_scale, groups, keep);
     if (lane < always) {
@@ -505,18 +516,18 @@ extern "C" int jv_moe_route_group_fits(int n, int experts, int top, int always) 
   return n <= 64 && (16LL * experts + 2LL * n * (top + always) + 3LL * (experts + always) + 2) * 4 <= 60 * 1024;
 }
 
-extern "C" int jv_moe_route_group(const float* logits, const float* bias, int n, int experts, int top, int always, int score,
+extern "C" int jv_moe_route_group(const float* logits, int parts, long long part_stride, const float* bias, int n, int experts, int top, int always, int score,
                                   int* ids, float* weights, const float* correction, float weight_scale, int groups,
                                   int keep, int tile_rows, int* meta, int* offsets, int* tile_expert, int* tile_row0,
                                   int* order, void* stream) {
   if (n <= 0) return 0;
   if (!jv_moe_route_group_fits(n, experts, top, always) || top > experts || score < 0 || score > MOE_SCORE_SOFTMAX ||
-      !moe_groups_ok(experts, top, groups, keep) || tile_rows <= 0)
+      !moe_groups_ok(experts, top, groups, keep) || tile_rows <= 0 || parts < 1)
     return (int)hipErrorInvalidValue;
   const size_t shmem = (16 * (size_t)experts + 2 * (size_t)n * (top + always) + 3 * (size_t)(experts + always) + 2) * 4;
   const int waves = n < 4 ? 4 : n > 16 ? 16 : n;
-  hipLaunchKernelGGL(moe_route_group_kernel, dim3(1), dim3(64 * waves), shmem, (hipStream_t)stream, logits, bias, n, experts, top,
-                     always, score, ids, weights, correction, weight_scale, groups, keep, tile_rows, meta, offsets,
+  hipLaunchKernelGGL(moe_route_group_kernel, dim3(1), dim3(64 * waves), shmem, (hipStream_t)stream, logits, parts,
+                     part_stride, bias, n, experts, top, always, score, ids, weights, correction, weight_scale, groups, keep, tile_rows, meta, offsets,
                      tile_expert, tile_row0, order);
   return JV_LAUNCH_CHECK();
 }

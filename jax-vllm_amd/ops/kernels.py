@@ -1713,23 +1713,28 @@ def moe_tile_rows_for(dtype, hidden: int, ff: int, entries: int, experts: int) -
     return moe_tile_rows()
 
 
+def moe_one_launch(n: int, experts: int, top: int, always: int = 0) -> bool:
+    """Whether choice and grouping of n tokens run as one block."""
+    return bool(library.core().jv_moe_route_group_fits(c_int(n), c_int(experts), c_int(top), c_int(always)))
+
+
 def moe_always_possible(x, w_router, top: int, always: int) -> bool:
     """Whether ``moe_route(None, top, x=x, w_router=w_router, always=always)`` runs: bfloat16 rows whose logits come from a
     product of their own, few enough for the one-block form."""
-    n = x.shape[0]
-    return (_router_logits_plan(x, w_router) is not None
-            and bool(library.core().jv_moe_route_group_fits(c_int(n), c_int(w_router.shape[0]), c_int(top), c_int(always))))
+    n, experts = x.shape[0], w_router.shape[0]
+    return moe_one_launch(n, experts, top, always) and _router_logits_plan(x, w_router, True) is not None
 
 
-def _router_logits_plan(x, w_router):
-    """How the router logits of bfloat16 rows are made by a product with float output: a ``streaming_plan`` for few rows,
-    "rows" for the tiled product, None where the fused kernel (or the float one) makes them."""
+def _router_logits_plan(x, w_router, one_launch: bool):
+    """How the router logits of bfloat16 rows are made by a product with float output: the number of partial products of
+    the few-rows product where the one-block form takes them, "rows" for the tiled product, None where the fused kernel
+    (or the float one) makes them."""
     if x.dtype != torch.bfloat16 or x.shape[1] % 8 or x.shape[1] < 8 or w_router.shape[0] > 3840:
         return None
     rows = x.shape[0]
-    if rows <= SKINNY_AUTO_ROWS:
-        plan = streaming_plan(rows, w_router.shape[0], w_router.shape[1], device=x.device)
-        return plan if plan is not None and plan[1] == 1 else None
+    if rows <= SKINNY_MAX_ROWS:
+        # 256 columns a block: a router is so narrow that only the inner size can be shared out to many blocks
+        return -(-x.shape[1] // 256) if one_launch else None
     return "rows" if rows > ROUTER_FUSED_MAX_ROWS else None
 
 
@@ -1776,27 +1781,28 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     groups of neighbours, and only those of the ``keep`` groups with the largest logits can be chosen.
     ``always`` (few tokens: ``moe_always_possible``): every token also gets the ``always`` experts behind the routed ones
     (number experts, experts + 1, ...) with weight 1, behind its chosen ones; the plan's ``top`` then counts them in.
-    Either float ``logits`` [n, experts] are given, or rows ``x`` [n, hidden] and the router matrix
+    Either float ``logits`` [n, experts] are given (few tokens: or a stack [parts, n, experts] of partial sums), or rows ``x`` [n, hidden] and the router matrix
     ``w_router`` [experts, hidden] of one type: then the logits are made here, in float (``logits_out``,
     float32 [n, experts], receives them if given): in the same launch as the choice (float32, odd sizes), or
     for bfloat16 by a matrix-core product with float output before it.  ``tile_rows``: rows of a tile of the grouping
     (``moe_tile_rows_for``; default: the float-FMA kernels' 64)."""
     if logits is None:
-        # bfloat16: the logits come from a matrix-core product with float output (never rounded to bfloat16): the
-        # weight-streaming one for the few rows of a decode step, the tiled one for prompt portions; between
-        # them (measured at 32 rows: one block of the tiled product walks the whole router alone) the fused kernel
-        how = _router_logits_plan(x, w_router)
+        # bfloat16: the logits come from a matrix-core product with float output (never rounded to bfloat16): for the
+        # few rows of a decode step with the inner size shared out to blocks (the one-block form adds the parts), the
+        # tiled one for prompt portions
+        how = _router_logits_plan(x, w_router, moe_one_launch(x.shape[0], w_router.shape[0], top, always))
         if how == "rows":
             logits = gemm_rows_f32out(x, w_router)
         elif how is not None:
-            logits = gemm_skinny(x, w_router, torch.float32, block_shape=how[0])
+            logits = gemm_tile64(x, w_router, torch.float32, ksplit=how)
         if logits is not None and logits_out is not None:
-            logits_out.copy_(logits if bias is None else logits + bias)
+            whole = logits.sum(0) if logits.dim() == 3 else logits
+            logits_out.copy_(whole if bias is None else whole + bias)
     _need(score in ROUTER_SCORES, f"no router score {score!r}: there are {sorted(ROUTER_SCORES)}")
     if logits is not None:
         _dev(logits)
         _f32(logits, "logits")
-        n, experts = logits.shape
+        n, experts = logits.shape[-2:]
         dev = logits.device
     else:
         _dev(x, w_router, logits_out)
@@ -1821,7 +1827,9 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
                          and keep * (experts // count) >= top and correction is None),
           "equal groups (at most 64), enough experts in the kept ones, and no correction of the choice")
     lib = library.core()
-    one_launch = logits is not None and bool(lib.jv_moe_route_group_fits(c_int(n), c_int(experts), c_int(top), c_int(always)))
+    one_launch = logits is not None and moe_one_launch(n, experts, top, always)
+    parts = logits.shape[0] if logits is not None and logits.dim() == 3 else 1
+    _need(parts == 1 or one_launch, "partial logits are added by the one-block form only")
     _need(always == 0 or one_launch, "experts for every token take logits and few tokens")
     all_experts, per = experts + always, top + always
     entries = n * per
@@ -1836,7 +1844,7 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     tile_expert, tile_row0 = ints[at:at + max_tiles], ints[at + max_tiles:at + 2 * max_tiles]
     weights = torch.empty(entries, dtype=torch.float32, device=dev)
     if one_launch:
-        _check(lib.jv_moe_route_group(_ptr(logits), _ptr(bias), c_int(n), c_int(experts), c_int(top), c_int(always),
+        _check(lib.jv_moe_route_group(_ptr(logits), c_int(parts), c_longlong(n * experts), _ptr(bias), c_int(n), c_int(experts), c_int(top), c_int(always),
                                       c_int(ROUTER_SCORES[score]), _ptr(ids), _ptr(weights), _ptr(correction),
                                       c_float(weight_scale), c_int(count), c_int(keep), c_int(tile_rows), _ptr(meta),
                                       _ptr(offsets), _ptr(tile_expert), _ptr(tile_row0), _ptr(order), _stream()), "moe_route_group")

@@ -30,7 +30,7 @@ from ..ops import kernels as K
 from .mlp import DenseMLP
 from .spec import PartSpec, TensorSpec, build_part, is_replayable, register_part
 
-SHARED_ALONG_MAX_TOKENS = 16      # tokens of a step that takes the shared expert along (its rows then fill one tile)
+SHARED_ALONG_MAX_TOKENS = 32      # tokens of a step that takes the shared expert along (its rows then fill two tiles)
 
 
 class RoutedExperts:

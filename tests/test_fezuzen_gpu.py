@@ -858,12 +858,16 @@ def test_kernel_experts_streamed_for_few_tokens(gated, n, hidden, ff, experts, t
 
 @pytest.mark.parametrize("n,experts,top,always,groups", [(1, 4, 1, 1, None), (8, 70, 3, 2, (7, 3)), (16, 9, 4, 3, None), (64, 130, 2, 0, (2, 1))])
 def test_kernel_router_and_grouping_in_one_launch(n, experts, top, always, groups):
-    """Every token has its chosen experts and the ones behind the routed experts; the grouping by experts and tiles."""
+    """Every token has its chosen experts and the ones behind the routed experts; the grouping by experts and tiles; the logits as
+    partial sums."""
     from jax_vllm_amd.ops import kernels as K
 
     g = torch.Generator().manual_seed(18)
-    logits = torch.randn(n, experts, generator=g)
-    plan = K.moe_route(_dev(logits), top, score="softmax", groups=groups, always=always, tile_rows=16)
+    stack = torch.randn(11, n, experts, generator=g)
+    logits = stack[0]
+    for part in stack[1:]:
+        logits = logits + part
+    plan = K.moe_route(_dev(stack), top, score="softmax", groups=groups, always=always, tile_rows=16)
     per = top + always
     assert plan.top == per
     ids, wts = plan.ids.view(n, per).cpu().long(), plan.weights.view(n, per).cpu().double()
