@@ -5,7 +5,8 @@ shared, and given back.
 Layers whose mixers have the same need (all earlier keys; a window of a given length; or the keys of
 the query's own block of a given number of positions) form a *group*: one page pool and one block table per request serve all layers of the
 group, each layer having page storage of its own.  Pages of a window group are given back
-as soon as the window has passed them, those of a block group when the next token begins another block; all pages and the slot are given back when the
+as soon as the window has passed them, those of a block group when the next token begins another block (the pages of
+first tokens that stay in sight are kept in either case); all pages and the slot are given back when the
 request ends.  Full pages of the all-keys group are hashed by content (chained over the
 prefix) so that a later request with the same prefix takes them instead of recomputing.
 
@@ -26,7 +27,7 @@ from .state_slots import StateSlotPool
 
 @dataclass
 class CacheGroup:
-    key: tuple                 # ("full",), ("window", W) or ("chunk", C)
+    key: tuple                 # ("full",), ("window", W) or ("chunk", C); the latter two with a third entry: first tokens kept
     runs: list                 # schedule entries whose own cache lives in this group
     pool: PagePool
 
@@ -35,8 +36,14 @@ class CacheGroup:
         """Whether a request's pages stay until it ends."""
         return self.key[0] == "full"
 
+    @property
+    def kept_tokens(self) -> int:
+        """First tokens of a sequence that every later one reads, whatever its window or block."""
+        return self.key[2] if len(self.key) > 2 else 0
+
     def first_needed(self, position: int) -> int:
-        """The earliest position whose key the query at ``position``, or any later one, still reads."""
+        """The earliest position whose key the query at ``position``, or any later one, still reads (besides the kept
+        first tokens)."""
         if self.key[0] == "window":
             return max(0, position - self.key[1] + 1)
         if self.key[0] == "chunk":
@@ -206,7 +213,7 @@ class CacheManager:
             dead_pages = g.first_needed(ctx) // ps
             if not dead_pages:
                 continue
-            gone = [i for i in range(min(dead_pages, len(table))) if table[i] != NULL_PAGE]
+            gone = [i for i in range(self._pages_for(g.kept_tokens), min(dead_pages, len(table))) if table[i] != NULL_PAGE]
             g.pool.release([table[i] for i in gone])
             for i in gone:
                 table[i] = NULL_PAGE

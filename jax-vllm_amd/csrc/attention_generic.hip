@@ -6,10 +6,10 @@
 //
 //   query token t of request r = token_req[t] sits at absolute position p = positions[t]
 //   and sees keys j with  max(0, p - window + 1) <= j <= p   (window 0: all j <= p; window < 0: those of
-//   its own block of -window positions, counted from position 0);
+//   its own block of -window positions, counted from position 0), and with `keep` > 0 the first `keep` keys j <= p too;
 //   key j lives in page block_tables[r, j / page_size] at slot j % page_size;
 //   q head h reads kv head h / (nq / nkv).
-// With `sinks` (one float per q head) every row's softmax denominator also holds exp(sinks[h]).
+// With `cap` > 0 a score is cap * tanh(score / cap), after its scale.  With `sinks` (one float per q head) every row's softmax denominator also holds exp(sinks[h]).
 // Cache layout: K pages[page][kv_head][slot][D], V pages[page][kv_head][D][slot].
 #include "common.h"
 
@@ -22,7 +22,7 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
                                const int* __restrict__ block_tables, int table_stride,
                                const int* __restrict__ token_req, const int* __restrict__ positions,
                                int page_size, int nq, int nkv, int D, float scale, int window,
-                               const float* __restrict__ sinks) {
+                               const float* __restrict__ sinks, float cap, int keep) {
   extern __shared__ float lds[];      // q[D] | p[64] | V offsets of the tile's keys as long long [64]
   float* qs = lds;
   float* ps = lds + D;
@@ -44,9 +44,15 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
 #pragma unroll
   for (int e = 0; e < GEN_MAX_E; ++e) acc[e] = 0.f;
 
-  for (int j0 = lo; j0 <= pos; j0 += 64) {
+  // the kept first keys in front of the window, then the window: two runs of consecutive keys
+  const int kept = keep < lo ? keep : lo;
+  const int kept_tiles = (kept + 63) / 64;
+  const int tiles = kept_tiles + (pos - lo) / 64 + 1;
+  for (int it = 0; it < tiles; ++it) {
+    const int j0 = it < kept_tiles ? it * 64 : lo + (it - kept_tiles) * 64;
+    const int end = it < kept_tiles ? kept : pos + 1;         // keys of this run
     const int j = j0 + lane;
-    const bool valid = j <= pos;
+    const bool valid = j < end;
     float s = -INFINITY;
     long long off = 0;
     if (valid) {
@@ -56,6 +62,7 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
       float dot = 0.f;
       for (int d = 0; d < D; ++d) dot += qs[d] * to_f32(kr[d]);
       s = dot * scale;
+      if (cap > 0.f) s = cap * tanhf(s / cap);
     }
     const float m_new = fmaxf(m, wave_max(s));  // finite: key j0 is always valid
     const float p = valid ? expf(s - m_new) : 0.f;
@@ -66,7 +73,7 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
     ps[lane] = p;
     offs[lane] = off;
     __syncthreads();
-    const int n = (pos - j0 + 1 < 64) ? pos - j0 + 1 : 64;
+    const int n = end - j0 < 64 ? end - j0 : 64;
 #pragma unroll
     for (int e = 0; e < GEN_MAX_E; ++e) {
       const int d = lane + 64 * e;
@@ -92,15 +99,16 @@ paged_attention_generic_kernel(T* __restrict__ out, const T* __restrict__ q, lon
       void* out, const void* q, long long q_row_stride, const void* k_pages, const void* v_pages,  \
       const int* block_tables, int table_stride, const int* token_req, const int* positions,       \
       int page_size, int n_tokens, int nq, int nkv, int D, float scale, int window,                \
-      const float* sinks, void* stream) {                                                          \
+      const float* sinks, float cap, int keep, void* stream) {                                     \
     if (n_tokens <= 0) return 0;                                                                   \
-    if (D > 64 * GEN_MAX_E || nkv <= 0 || nq % nkv != 0 || page_size <= 0)                         \
+    if (D > 64 * GEN_MAX_E || nkv <= 0 || nq % nkv != 0 || page_size <= 0 || keep < 0)             \
       return (int)hipErrorInvalidValue;                                                            \
     const size_t shmem = (D + 64 + 2) * sizeof(float) + 64 * sizeof(long long);                    \
     hipLaunchKernelGGL(paged_attention_generic_kernel<T>, dim3(n_tokens, nq), dim3(64), shmem,     \
                        (hipStream_t)stream, (T*)out, (const T*)q, q_row_stride,                    \
                        (const T*)k_pages, (const T*)v_pages, block_tables, table_stride,           \
-                       token_req, positions, page_size, nq, nkv, D, scale, window, sinks);         \
+                       token_req, positions, page_size, nq, nkv, D, scale, window, sinks, cap,     \
+                       keep);                                                                      \
     return JV_LAUNCH_CHECK();                                                                      \
   }
 

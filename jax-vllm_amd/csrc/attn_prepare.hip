@@ -6,6 +6,7 @@
 //            (a wave a (token, head))
 //   q, k  <- the first rot_dims elements of every head turned by the token's angles
 //   q     <- q * (1 + coef * ln(floor((position + 1) / every) + 1))    (optional: a query temperature that grows with position)
+//   v     <- (1 - mix) v + mix v_first    (optional: the same token's values of another layer)
 //   v     <- v * v_scale;  the v heads begin at column v_off of the row (behind k, or AT k: values that are the keys as projected)
 // and stored in the layout the paged attention kernels read, every head padded with zeros to one size
 // Dp >= max(dk, dv): q rows [n][nq][Dp], key pages [pages][nkv][page_size][Dp], value pages transposed
@@ -95,7 +96,8 @@ attn_prepare_heads_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, long
                           int rot_dims, const int* __restrict__ slot_mapping, T* __restrict__ k_pages,
                           T* __restrict__ v_pages, int page_size, int nq, int nkv, int dk, int dv, int dp,
                           float v_scale, int v_elsewhere, long long v_off, const int* __restrict__ positions,
-                          float qt_coef, int qt_every) {
+                          float qt_coef, int qt_every, const T* __restrict__ v_first, long long first_stride,
+                          float mix) {
   extern __shared__ float heads_lds[];     // [4 waves][dk]
   const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE;
   float* buf = heads_lds + wid * dk;
@@ -113,8 +115,11 @@ attn_prepare_heads_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, long
     const int kvh = head - nq - nkv;
     const long long c0 = v_off + (long long)kvh * dv;
     T* dst = v_pages + (page * nkv + kvh) * (long long)dp * page_size + slot;
-    for (int i = lane; i < dv; i += JV_WAVE)
-      dst[(long long)i * page_size] = from_f32<T>((to_f32(x[c0 + i]) + (bias ? bias[c0 + i] : 0.f)) * v_scale);
+    for (int i = lane; i < dv; i += JV_WAVE) {
+      float v = to_f32(x[c0 + i]) + (bias ? bias[c0 + i] : 0.f);
+      if (v_first) v = (1.f - mix) * v + mix * to_f32(v_first[t * first_stride + (long long)kvh * dv + i]);
+      dst[(long long)i * page_size] = from_f32<T>(v * v_scale);
+    }
   }
   const bool work = is_q || (is_k && store);      // a k head that nobody will read is skipped
   const int c0 = (live && !is_v ? head : 0) * dk;
@@ -161,7 +166,8 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
                               const float* __restrict__ q_w, const float* __restrict__ k_w, float eps,
                               const float* __restrict__ cos_sin, int rot_dims, const int* __restrict__ slot_mapping,
                               T* __restrict__ k_pages, int page_size, long long n_items, int nq, int nkv, int dk,
-                              int dp, int lph, const int* __restrict__ positions, float qt_coef, int qt_every) {
+                              int dp, int lph, const int* __restrict__ positions, float qt_coef, int qt_every,
+                              const float* __restrict__ bias) {
   constexpr int EP = 16 / (int)sizeof(T);
   typedef T tv __attribute__((ext_vector_type(EP)));
   const int lane = threadIdx.x & (JV_WAVE - 1), wid = threadIdx.x / JV_WAVE;
@@ -179,7 +185,10 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
   const float* w = is_q ? q_w : k_w;
   float a[EP], ss = 0.f;
 #pragma unroll
-  for (int e = 0; e < EP; ++e) { a[e] = to_f32<T>(xv[e]); ss = fmaf(a[e], a[e], ss); }
+  for (int e = 0; e < EP; ++e) {
+    a[e] = to_f32<T>(xv[e]) + (bias ? bias[head * dk + e0 + e] : 0.f);
+    ss = fmaf(a[e], a[e], ss);
+  }
   if (w) {
     for (int o = lph / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, JV_WAVE);
     const float inv = rsqrtf(ss / (float)dk + eps);
@@ -226,8 +235,10 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
                                             void* k_pages, void* v_pages, int page_size, int n, int nq,         \
                                             int nkv, int dk, int dv, int dp, float v_scale, int per_head,       \
                                             long long v_off, const int* positions, float qt_coef, int qt_every, \
+                                            const void* v_first, long long first_stride, float mix,             \
                                             void* stream) {                                                     \
     if (n <= 0) return 0;                                                                                       \
+    if (v_first && q_w && !per_head) return (int)hipErrorInvalidValue;                                          \
     if (v_off < 0 || (positions && (qt_every <= 0 || (q_w && !per_head)))) return (int)hipErrorInvalidValue;    \
     if (q_w && !per_head && v_off != (long long)(nq + nkv) * dk) return (int)hipErrorInvalidValue;              \
     if (nq <= 0 || nkv <= 0 || dk <= 0 || dv <= 0 || dp < dk || dp < dv || rot_dims < 0 || rot_dims > dk ||     \
@@ -236,11 +247,12 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
     if (!q_w || per_head) {                                                                                     \
       /* a wave a (token, head); the v heads of many tokens through the tile writer where its pieces align */  \
       constexpr int EP = 16 / (int)sizeof(T);                                                                   \
-      const bool v_tile = slot_mapping && !bias && v_written_by_tile<T>(k_pages, n, page_size, dv) &&           \
+      const bool v_tile = slot_mapping && v_written_by_tile<T>(k_pages, n, page_size, dv) &&                    \
                           ld % EP == 0 && v_off % EP == 0 && ((uintptr_t)qkv % 16) == 0;                        \
       if (v_tile) {                                                                                             \
         const int e = launch_v_pages_write<T>(qkv, ld, v_off, slot_mapping, v_pages, page_size, n, nkv, dv,     \
-                                              dp, v_scale, stream);                                             \
+                                              dp, v_scale, stream, bias ? bias + v_off : nullptr, v_first,      \
+                                              first_stride, mix);                                               \
         if (e) return e;                                                                                        \
       }                                                                                                         \
       const int lph = dk / EP;                                                                                  \
@@ -252,7 +264,7 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
         hipLaunchKernelGGL(attn_prepare_heads_vec_kernel<T>, dim3((unsigned)blocks), dim3(256), 0,              \
                            (hipStream_t)stream, (T*)q_out, (const T*)qkv, ld, q_w, k_w, eps, cos_sin, rot_dims, \
                            slot_mapping, (T*)k_pages, page_size, items, nq, nkv, dk, dp, lph, positions,        \
-                           qt_coef, qt_every);                                                                  \
+                           qt_coef, qt_every, bias);                                                            \
         return JV_LAUNCH_CHECK();                                                                               \
       }                                                                                                         \
       const int walk = (v_tile || !slot_mapping) ? nq + nkv : nq + 2 * nkv;                                     \
@@ -261,7 +273,7 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
                          (size_t)4 * dk * sizeof(float), (hipStream_t)stream, (T*)q_out, (const T*)qkv, ld,     \
                          bias, q_w, k_w, eps, cos_sin, rot_dims, slot_mapping, (T*)k_pages, (T*)v_pages,        \
                          page_size, nq, nkv, dk, dv, dp, v_scale, v_tile ? 1 : 0, v_off, positions, qt_coef,   \
-                         qt_every);                                                                             \
+                         qt_every, (const T*)v_first, first_stride, mix);                                       \
       return JV_LAUNCH_CHECK();                                                                                 \
     }                                                                                                           \
     const size_t shmem = (size_t)(nq + nkv) * dk * sizeof(float);                                               \

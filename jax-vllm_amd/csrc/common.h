@@ -61,11 +61,21 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 // exported interface (the Python side names them).
 #define JV_ACT_SILU 1        // gate / (1 + exp(-gate))
 #define JV_ACT_GELU_TANH 2   // 0.5 gate (1 + tanh(sqrt(2/pi) (gate + 0.044715 gate^3)))
-__host__ __device__ __forceinline__ bool jv_act_known(int act) { return act == JV_ACT_SILU || act == JV_ACT_GELU_TANH; }
-__device__ __forceinline__ float jv_gated(int act, float gate, float up) {
-  if (act == JV_ACT_GELU_TANH) {
+#define JV_ACT_CLAMPED 6     // g / (1 + exp(-slope g)) (u + 1) with g = min(gate, limit), u = up clamped to [-limit, limit]
+// An activation with its constants (those of JV_ACT_CLAMPED; the others have none).
+struct JvAct { int id; float limit, slope; };
+__host__ __device__ __forceinline__ bool jv_act_known(int act) {
+  return act == JV_ACT_SILU || act == JV_ACT_GELU_TANH || act == JV_ACT_CLAMPED;
+}
+__device__ __forceinline__ float jv_gated(JvAct act, float gate, float up) {
+  if (act.id == JV_ACT_GELU_TANH) {
     const float inner = 0.7978845608028654f * (gate + 0.044715f * gate * gate * gate);
     return 0.5f * gate * (1.f + tanhf(inner)) * up;
+  }
+  if (act.id == JV_ACT_CLAMPED) {      // comparisons that a NaN passes through
+    const float g = gate > act.limit ? act.limit : gate;
+    const float u = up > act.limit ? act.limit : up < -act.limit ? -act.limit : up;
+    return g / (1.f + expf(-act.slope * g)) * (u + 1.f);
   }
   return gate / (1.f + expf(-gate)) * up;
 }

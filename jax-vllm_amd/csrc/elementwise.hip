@@ -313,7 +313,8 @@ __global__ void rmsnorm_kernel(T* __restrict__ out, const T* __restrict__ x,
 // Interleaved layout (gate and up alternate along the row): out[t, j] = act(gu[t, 2j]) * gu[t, 2j+1];
 // each thread takes four outputs (8 inputs, 16 bytes of bfloat16) when inter % 4 == 0.
 template <typename T, int ACT>
-__global__ void gated_mul_pairs_kernel(T* __restrict__ out, const T* __restrict__ gu, int inter) {
+__global__ void gated_mul_pairs_kernel(T* __restrict__ out, const T* __restrict__ gu, int inter, JvAct act) {
+  act.id = ACT;
   const long long t = blockIdx.y;
   const int j = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
   if (j >= inter) return;
@@ -322,17 +323,18 @@ __global__ void gated_mul_pairs_kernel(T* __restrict__ out, const T* __restrict_
   if ((inter & 3) == 0) {
     float v[8];
     load8<T>(gp, v);
-    store4<T>(op, float4{jv_gated(ACT, v[0], v[1]), jv_gated(ACT, v[2], v[3]), jv_gated(ACT, v[4], v[5]),
-                         jv_gated(ACT, v[6], v[7])});
+    store4<T>(op, float4{jv_gated(act, v[0], v[1]), jv_gated(act, v[2], v[3]), jv_gated(act, v[4], v[5]),
+                         jv_gated(act, v[6], v[7])});
   } else {
     for (int e = 0; e < 4 && j + e < inter; ++e)
-      op[e] = from_f32<T>(jv_gated(ACT, to_f32(gp[2 * e]), to_f32(gp[2 * e + 1])));
+      op[e] = from_f32<T>(jv_gated(act, to_f32(gp[2 * e]), to_f32(gp[2 * e + 1])));
   }
 }
 
 // grid (column blocks, tokens); each thread takes 4 neighbouring columns when inter % 4 == 0.
 template <typename T, int VEC, int ACT>
-__global__ void gated_mul_kernel(T* __restrict__ out, const T* __restrict__ gu, int inter) {
+__global__ void gated_mul_kernel(T* __restrict__ out, const T* __restrict__ gu, int inter, JvAct act) {
+  act.id = ACT;
   const long long t = blockIdx.y;
   const int j = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
   if (j >= inter) return;
@@ -340,24 +342,24 @@ __global__ void gated_mul_kernel(T* __restrict__ out, const T* __restrict__ gu, 
   T* op = out + t * inter + j;
   if (VEC == 4) {
     const float4 g = load4<T>(gp), u = load4<T>(gp + inter);
-    store4<T>(op, float4{jv_gated(ACT, g.x, u.x), jv_gated(ACT, g.y, u.y), jv_gated(ACT, g.z, u.z),
-                         jv_gated(ACT, g.w, u.w)});
+    store4<T>(op, float4{jv_gated(act, g.x, u.x), jv_gated(act, g.y, u.y), jv_gated(act, g.z, u.z),
+                         jv_gated(act, g.w, u.w)});
   } else {
-    op[0] = from_f32<T>(jv_gated(ACT, to_f32(gp[0]), to_f32(gp[inter])));
+    op[0] = from_f32<T>(jv_gated(act, to_f32(gp[0]), to_f32(gp[inter])));
   }
 }
 
 template <typename T, int ACT>
-static void launch_gated_mul(T* o, const T* g, unsigned ny, int inter, int interleaved, hipStream_t stream) {
+static void launch_gated_mul(T* o, const T* g, unsigned ny, int inter, int interleaved, JvAct act, hipStream_t stream) {
   if (interleaved)
     hipLaunchKernelGGL((gated_mul_pairs_kernel<T, ACT>), dim3(((inter + 3) / 4 + 255) / 256, ny), dim3(256), 0, stream,
-                       o, g, inter);
+                       o, g, inter, act);
   else if (inter % 4 == 0)
     hipLaunchKernelGGL((gated_mul_kernel<T, 4, ACT>), dim3((inter / 4 + 255) / 256, ny), dim3(256), 0, stream, o, g,
-                       inter);
+                       inter, act);
   else
     hipLaunchKernelGGL((gated_mul_kernel<T, 1, ACT>), dim3((inter + 255) / 256, ny), dim3(256), 0, stream, o, g,
-                       inter);
+                       inter, act);
 }
 
 // ---------------------------------------------------------------- float -> T copy of selected rows
@@ -487,17 +489,18 @@ __global__ void scaled_sum_kernel(float* __restrict__ out, const T* __restrict__
     return JV_LAUNCH_CHECK();                                                                       \
   }                                                                                                 \
   extern "C" int jv_gated_mul_##SUF(void* out, const void* gu, long long n_tokens, int inter,       \
-                                    int interleaved, int act, void* stream) {                      \
+                                    int interleaved, int act, float act_limit, float act_slope, void* stream) { \
     if (n_tokens <= 0 || inter <= 0) return 0;                                                      \
     if (!jv_act_known(act)) return (int)hipErrorInvalidValue;                                       \
     for (long long t0 = 0; t0 < n_tokens; t0 += 65535) { /* grid.y limit */                         \
       const unsigned ny = (unsigned)(n_tokens - t0 < 65535 ? n_tokens - t0 : 65535);                \
       T* o = (T*)out + t0 * inter;                                                                  \
       const T* g = (const T*)gu + t0 * 2 * inter;                                                   \
-      if (act == JV_ACT_GELU_TANH)                                                                  \
-        launch_gated_mul<T, JV_ACT_GELU_TANH>(o, g, ny, inter, interleaved, (hipStream_t)stream);   \
-      else                                                                                          \
-        launch_gated_mul<T, JV_ACT_SILU>(o, g, ny, inter, interleaved, (hipStream_t)stream);        \
+      const JvAct a{act, act_limit, act_slope};                                                     \
+      auto launch = act == JV_ACT_GELU_TANH ? launch_gated_mul<T, JV_ACT_GELU_TANH>                 \
+                    : act == JV_ACT_CLAMPED ? launch_gated_mul<T, JV_ACT_CLAMPED>                   \
+                                            : launch_gated_mul<T, JV_ACT_SILU>;                     \
+      launch(o, g, ny, inter, interleaved, a, (hipStream_t)stream);                                 \
     }                                                                                               \
     return JV_LAUNCH_CHECK();                                                                       \
   }                                                                                                 \

@@ -26,7 +26,7 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 template <int MT, typename OutT, bool PAIRS>
 __global__ void __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2)))   // one block a compute unit, 256 registers a lane
 gemm_tile64_kernel(OutT* __restrict__ y, const bf16_t* __restrict__ x, const bf16_t* __restrict__ W,
-                   int M, int N, int K, long long ldx, long long ldy, int k_per, int act) {
+                   int M, int N, int K, long long ldx, long long ldy, int k_per, JvAct act) {
   constexpr int ROWS = MT * 16;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t (*xs)[ROWS * T64_XS] = (bf16_t (*)[ROWS * T64_XS])smem;   // [2][ROWS][T64_XS]
@@ -144,7 +144,7 @@ gemm_tile64_kernel(OutT* __restrict__ y, const bf16_t* __restrict__ x, const bf1
 
 template <int MT, typename OutT, bool PAIRS>
 static int launch_tile64(void* y, const void* x, const void* W, int M, int N, int K, long long ldx, long long ldy,
-                         int ksplit, int act, hipStream_t stream) {
+                         int ksplit, JvAct act, hipStream_t stream) {
   // columns per group: a whole number of chunks, every group with at least one column
   const int chunks = (K + T64_KC - 1) / T64_KC;
   const int k_per = ((chunks + ksplit - 1) / ksplit) * T64_KC;
@@ -166,7 +166,7 @@ static int launch_tile64(void* y, const void* x, const void* W, int M, int N, in
 
 template <typename OutT, bool PAIRS>
 static int dispatch_tile64(void* y, const void* x, const void* W, int M, int N, int K, long long ldx,
-                           long long ldy, int ksplit, int act, hipStream_t s) {
+                           long long ldy, int ksplit, JvAct act, hipStream_t s) {
   switch ((M + 15) / 16) {
     case 1: return launch_tile64<1, OutT, PAIRS>(y, x, W, M, N, K, ldx, ldy, ksplit, act, s);
     case 2: return launch_tile64<2, OutT, PAIRS>(y, x, W, M, N, K, ldx, ldy, ksplit, act, s);
@@ -183,13 +183,14 @@ static int dispatch_tile64(void* y, const void* x, const void* W, int M, int N, 
 // and y is [ksplit][M][ldy], partial products that the reader adds in that order; refused when
 // a group would be left without columns.
 extern "C" int jv_gemm_tile64_bf16(void* y, const void* x, const void* W, int M, int N, int K, long long ldx,
-                                   long long ldy, int out_f32, int gate_act, int ksplit, void* stream) {
+                                   long long ldy, int out_f32, int gate_act, float act_limit, float act_slope,
+                                   int ksplit, void* stream) {
   if (M <= 0 || N <= 0) return 0;
   if (M > 64 || K <= 0 || K % 8 != 0 || ldx % 8 != 0) return (int)hipErrorInvalidValue;
   if (gate_act && (!jv_act_known(gate_act) || out_f32 || N % 2 != 0 || ksplit != 1)) return (int)hipErrorInvalidValue;
   if (ksplit < 1 || ksplit > 65535 || (ksplit > 1 && !out_f32)) return (int)hipErrorInvalidValue;
   hipStream_t s = (hipStream_t)stream;
-  if (gate_act) return dispatch_tile64<bf16_t, true>(y, x, W, M, N, K, ldx, ldy, ksplit, gate_act, s);
-  return out_f32 ? dispatch_tile64<float, false>(y, x, W, M, N, K, ldx, ldy, ksplit, 0, s)
-                 : dispatch_tile64<bf16_t, false>(y, x, W, M, N, K, ldx, ldy, ksplit, 0, s);
+  if (gate_act) return dispatch_tile64<bf16_t, true>(y, x, W, M, N, K, ldx, ldy, ksplit, JvAct{gate_act, act_limit, act_slope}, s);
+  return out_f32 ? dispatch_tile64<float, false>(y, x, W, M, N, K, ldx, ldy, ksplit, JvAct{}, s)
+                 : dispatch_tile64<bf16_t, false>(y, x, W, M, N, K, ldx, ldy, ksplit, JvAct{}, s);
 }

@@ -5,7 +5,8 @@
 //   route:   z = router logits (float, plus an optional bias per expert) -> the `top` largest per token
 //            (lowest index among equals), weight = sigmoid(z), or the softmax over the chosen logits alone, or
 //            ("sigmoid_normed") the largest sigmoid(z) + correction chosen, weight = sigmoid(z) over the sum of the
-//            chosen sigmoids (+ 1e-20) times a constant, or ("softmax") the softmax over ALL logits, as it is.
+//            chosen sigmoids (+ 1e-20) times a constant, or ("sigmoid_corrected") chosen alike, weight = sigmoid(z) times a
+//            constant, or ("softmax") the softmax over ALL logits, as it is.
 //            Experts may form equal groups of neighbours: only those of the `keep` groups with the largest logits
 //            (lowest group among equals) can then be chosen
 //   group:   entry s = token * top + kk  ->  position in a list ordered by expert; tiles of MOE_TM rows
@@ -27,12 +28,15 @@
 #define MOE_SCORE_SOFTMAX_CHOSEN 1   // weight = exp(logit) / sum of exp over the token's chosen logits
 #define MOE_SCORE_SIGMOID_NORMED 2   // chosen by sigmoid(logit) + correction; weight = sigmoid(logit) / (sum over the chosen + 1e-20) * scale
 #define MOE_SCORE_SOFTMAX 3          // weight = exp(logit) / sum of exp over all of the token's logits
+#define MOE_SCORE_SIGMOID_CORRECTED 4  // chosen by sigmoid(logit) + correction; weight = sigmoid(logit) * scale
+#define MOE_SCORE_LAST 4
 #define MOE_MAX_GROUPS 64
 #define MOE_LANE_EXPERTS 256         // up to so many experts a lane keeps its own in registers
 __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int lane, int* ids, float* weights,
                                          int score, const float* __restrict__ correction, float weight_scale,
                                          int groups, int keep) {
   const bool normed = score == MOE_SCORE_SIGMOID_NORMED;
+  const bool corrected = normed || score == MOE_SCORE_SIGMOID_CORRECTED;      // the choice looks at sigmoid + correction
   float zmax = 0.f, inv_sum = 0.f;
   if (score == MOE_SCORE_SOFTMAX) {      // over all experts, before any is left out
     float m = -INFINITY, sum = 0.f;
@@ -67,7 +71,7 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
       const int e = lane + i * JV_WAVE;
       z[i] = e < experts ? zt[e] : 0.f;
       c[i] = z[i];
-      if (normed && z[i] != -INFINITY && e < experts) c[i] = 1.f / (1.f + expf(-z[i])) + (correction ? correction[e] : 0.f);
+      if (corrected && z[i] != -INFINITY && e < experts) c[i] = 1.f / (1.f + expf(-z[i])) + (correction ? correction[e] : 0.f);
       if (c[i] != c[i]) c[i] = -INFINITY;         // a NaN takes the last places, its weight shows it
       if (e >= experts) c[i] = __builtin_nanf("");
     }
@@ -101,6 +105,7 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
     } else {
       w = mine ? 1.f / (1.f + expf(-zk)) : 0.f;
       if (normed) w *= weight_scale / (wave_sum(w) + 1e-20f);
+      else if (corrected) w *= weight_scale;
     }
     if (mine) {
       ids[lane] = ek;
@@ -114,7 +119,7 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
     for (int e = lane; e < experts; e += JV_WAVE) {
       float v = zt[e];
       // an expert already taken holds -inf and stays out; the others compete with their corrected sigmoid
-      if (normed && v != -INFINITY) v = 1.f / (1.f + expf(-v)) + (correction ? correction[e] : 0.f);
+      if (corrected && v != -INFINITY) v = 1.f / (1.f + expf(-v)) + (correction ? correction[e] : 0.f);
       if (v > bv || (bi == 0x7fffffff && v == v)) { bv = v; bi = e; }
     }
 #pragma unroll
@@ -126,7 +131,7 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
     if (bi == 0x7fffffff) { bi = kk; bv = __builtin_nanf(""); }      // a row of NaN: some expert, the NaN shows in the output
     if (lane == 0) {
       ids[kk] = bi;
-      const float z = normed ? zt[bi] : bv;          // the logit itself: the correction takes part in the choice only
+      const float z = corrected ? zt[bi] : bv;          // the logit itself: the correction takes part in the choice only
       weights[kk] = score == MOE_SCORE_SOFTMAX_CHOSEN ? bv : score == MOE_SCORE_SOFTMAX ? expf(z - zmax) * inv_sum
                                                                                         : 1.f / (1.f + expf(-z));
     }
@@ -144,6 +149,8 @@ __device__ __forceinline__ void moe_pick(float* zt, int experts, int top, int la
     const float inv = 1.f / sum;
     for (int kk = 0; kk < top; ++kk) weights[kk] *= inv;
   }
+  if (corrected && !normed && lane == 0)
+    for (int kk = 0; kk < top; ++kk) weights[kk] *= weight_scale;
   if (normed && lane == 0) {
     float sum = 0.f;
     for (int kk = 0; kk < top; ++kk) sum += weights[kk];
@@ -341,7 +348,7 @@ __global__ void __launch_bounds__(256)
 moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restrict__ Wg, const T* __restrict__ Wu,
                    const int* __restrict__ meta, const int* __restrict__ offsets, const int* __restrict__ tile_expert,
                    const int* __restrict__ tile_row0, const int* __restrict__ order, const float* __restrict__ weights,
-                   int top, int hidden, int ff, int act, int scale_input) {
+                   int top, int hidden, int ff, JvAct act, int scale_input) {
   if ((int)blockIdx.x >= meta[0]) return;
   __shared__ float As[MOE_BK][MOE_TM + 4];
   __shared__ float Gs[GATED ? MOE_BK : 1][MOE_TN + 4];
@@ -398,7 +405,7 @@ moe_gate_up_kernel(T* __restrict__ z, const T* __restrict__ x, const T* __restri
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
-      if (n < ff) z[(long long)(row0 + m) * ff + n] = from_f32<T>(GATED ? jv_gated(act, ag[i][j] * w, au[i][j] * w) : jv_act(act, au[i][j] * w));
+      if (n < ff) z[(long long)(row0 + m) * ff + n] = from_f32<T>(GATED ? jv_gated(act, ag[i][j] * w, au[i][j] * w) : jv_act(act.id, au[i][j] * w));
     }
   }
 }
@@ -501,7 +508,7 @@ extern "C" int jv_moe_route(const float* logits, const float* bias, int n, int e
                             float* weights, const float* correction, float weight_scale, int groups, int keep,
                             void* stream) {
   if (n <= 0) return 0;
-  if (experts <= 0 || top <= 0 || top > experts || score < 0 || score > MOE_SCORE_SOFTMAX)
+  if (experts <= 0 || top <= 0 || top > experts || score < 0 || score > MOE_SCORE_LAST)
     return (int)hipErrorInvalidValue;
   if (!moe_groups_ok(experts, top, groups, keep)) return (int)hipErrorInvalidValue;
   if (experts > 3840) return (int)hipErrorInvalidValue;
@@ -521,7 +528,7 @@ extern "C" int jv_moe_route_group(const float* logits, int parts, long long part
                                   int keep, int tile_rows, int* meta, int* offsets, int* tile_expert, int* tile_row0,
                                   int* order, void* stream) {
   if (n <= 0) return 0;
-  if (!jv_moe_route_group_fits(n, experts, top, always) || top > experts || score < 0 || score > MOE_SCORE_SOFTMAX ||
+  if (!jv_moe_route_group_fits(n, experts, top, always) || top > experts || score < 0 || score > MOE_SCORE_LAST ||
       !moe_groups_ok(experts, top, groups, keep) || tile_rows <= 0 || parts < 1)
     return (int)hipErrorInvalidValue;
   const size_t shmem = (16 * (size_t)experts + 2 * (size_t)n * (top + always) + 3 * (size_t)(experts + always) + 2) * 4;
@@ -548,7 +555,7 @@ extern "C" int jv_moe_group(const int* ids, int entries, int experts, int tile_r
                                      int keep, void* stream) {                                                    \
     if (n <= 0) return 0;                                                                                         \
     if (experts <= 0 || top <= 0 || top > experts || hidden <= 0 || (hidden + experts) > 15000 || score < 0 ||    \
-        score > MOE_SCORE_SOFTMAX || !moe_groups_ok(experts, top, groups, keep))                                  \
+        score > MOE_SCORE_LAST || !moe_groups_ok(experts, top, groups, keep))                                  \
       return (int)hipErrorInvalidValue;                                                                           \
     int tb = 15000 / (hidden + experts);             /* tokens of a block: their rows and logits in 60 KB */      \
     tb = tb > MOE_RT ? MOE_RT : tb;                                                                               \
@@ -575,14 +582,14 @@ extern "C" int jv_moe_group(const int* ids, int entries, int experts, int tile_r
   extern "C" int jv_moe_gate_up_##SUF(void* z, const void* x, const void* Wg, const void* Wu, const int* meta,    \
                                       const int* offsets, const int* tile_expert, const int* tile_row0,           \
                                       const int* order, const float* weights, int max_tiles, int top, int hidden, \
-                                      int ff, int act, int scale_input, void* stream) {                           \
+                                      int ff, int act, float act_limit, float act_slope, int scale_input, void* stream) {                           \
     if (max_tiles <= 0 || ff <= 0) return 0;                                                                      \
     if (!(Wg ? jv_act_known(act) : jv_plain_act_known(act)) || (ff + MOE_TN - 1) / MOE_TN > 65535)                \
       return (int)hipErrorInvalidValue;                                                                           \
     auto kernel = Wg ? moe_gate_up_kernel<T, true> : moe_gate_up_kernel<T, false>;                                \
     hipLaunchKernelGGL(kernel, dim3(max_tiles, (ff + MOE_TN - 1) / MOE_TN), dim3(256), 0,          \
                        (hipStream_t)stream, (T*)z, (const T*)x, (const T*)Wg, (const T*)Wu, meta, offsets,        \
-                       tile_expert, tile_row0, order, weights, top, hidden, ff, act, scale_input);                \
+                       tile_expert, tile_row0, order, weights, top, hidden, ff, JvAct{act, act_limit, act_slope}, scale_input);                \
     return JV_LAUNCH_CHECK();                                                                                     \
   }                                                                                                               \
   extern "C" int jv_moe_down_##SUF(float* y, const void* z, const void* Wd, const int* meta, const int* offsets,  \

@@ -27,7 +27,7 @@ __global__ void __launch_bounds__(256)
 moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const bf16_t* __restrict__ W0,
                 const bf16_t* __restrict__ W1, const int* __restrict__ meta, const int* __restrict__ offsets,
                 const int* __restrict__ tile_expert, const int* __restrict__ tile_row0, const int* __restrict__ order,
-                const float* __restrict__ weights, int top, int n_tokens, int K, int N, int act, int use_weight) {
+                const float* __restrict__ weights, int top, int n_tokens, int K, int N, JvAct act, int use_weight) {
   constexpr int TM = 16 * MT;
   constexpr bool GATED = MODE == MM_GATED, BY_TOKEN = MODE != MM_DOWN;
   // Blocks b, b + 8, b + 16, ... run on one XCD (with an L2 of its own): each of the 8 takes one run of the (tile, rows of W)
@@ -128,7 +128,7 @@ moe_mfma_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const
       bf16_t* z = (bf16_t*)out + (long long)(row0 + m) * N;
 #pragma unroll
       for (int c = 0; c < 4; ++c)
-        if (nb + c < N) z[nb + c] = from_f32<bf16_t>(jv_act(act, acc0[mt][c] * w));
+        if (nb + c < N) z[nb + c] = from_f32<bf16_t>(jv_act(act.id, acc0[mt][c] * w));
     } else {
       const int token = s / top, kk = s - token * top;
       float* y = (float*)out + ((long long)kk * n_tokens + token) * N;
@@ -143,7 +143,7 @@ template <int MODE>
 static int launch_moe_mfma(int tile_rows, int max_tiles, hipStream_t stream, void* out, const bf16_t* a, const bf16_t* W0,
                            const bf16_t* W1, const int* meta, const int* offsets, const int* tile_expert,
                            const int* tile_row0, const int* order, const float* weights, int top, int n_tokens, int K,
-                           int N, int act, int use_weight) {
+                           int N, JvAct act, int use_weight) {
   const long long pairs = (long long)max_tiles * ((N + MM_T - 1) / MM_T);
   if (pairs > 0x7ffffff0ll) return (int)hipErrorInvalidValue;
   const dim3 grid((unsigned)(pairs + 7));
@@ -163,16 +163,16 @@ static int launch_moe_mfma(int tile_rows, int max_tiles, hipStream_t stream, voi
 extern "C" int jv_moe_gate_up_mfma_bf16(void* z, const void* x, const void* Wg, const void* Wu, const int* meta,
                                         const int* offsets, const int* tile_expert, const int* tile_row0,
                                         const int* order, const float* weights, int max_tiles, int top, int hidden,
-                                        int ff, int act, int scale_input, int tile_rows, void* stream) {
+                                        int ff, int act, float act_limit, float act_slope, int scale_input, int tile_rows, void* stream) {
   if (max_tiles <= 0 || ff <= 0) return 0;
   if (!(Wg ? jv_act_known(act) : jv_plain_act_known(act)) || hidden < 8 || hidden % 8 || (ff + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
   if (!Wg)
     return launch_moe_mfma<MM_PLAIN>(tile_rows, max_tiles, (hipStream_t)stream, z,
                                      (const bf16_t*)x, (const bf16_t*)Wu, nullptr, meta, offsets, tile_expert, tile_row0,
-                                     order, weights, top, 0, hidden, ff, act, scale_input);
+                                     order, weights, top, 0, hidden, ff, JvAct{act, act_limit, act_slope}, scale_input);
   return launch_moe_mfma<MM_GATED>(tile_rows, max_tiles, (hipStream_t)stream, z, (const bf16_t*)x,
                                (const bf16_t*)Wg, (const bf16_t*)Wu, meta, offsets, tile_expert, tile_row0, order,
-                               weights, top, 0, hidden, ff, act, scale_input);
+                               weights, top, 0, hidden, ff, JvAct{act, act_limit, act_slope}, scale_input);
 }
 
 // down: z [entries, ff] by position, Wd [experts, hidden, ff] -> y [top, tokens, hidden] float
@@ -184,7 +184,7 @@ extern "C" int jv_moe_down_mfma_bf16(float* y, const void* z, const void* Wd, co
   if (ff < 8 || ff % 8 || (hidden + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
   return launch_moe_mfma<MM_DOWN>(tile_rows, max_tiles, (hipStream_t)stream, y,
                                 (const bf16_t*)z, (const bf16_t*)Wd, nullptr, meta, offsets, tile_expert, tile_row0, order,
-                                weights, top, n_tokens, ff, hidden, 0, scale_output);
+                                weights, top, n_tokens, ff, hidden, JvAct{}, scale_output);
 }
 
 // y [M, N] float = x [M, K] W[N, K]^T for bfloat16 x and W: the same kernel without a grouping (router logits
@@ -193,5 +193,5 @@ extern "C" int jv_gemm_rows_f32out_bf16(float* y, const void* x, const void* W, 
   if (M <= 0 || N <= 0) return 0;
   if (K < 8 || K % 8 || (N + MM_T - 1) / MM_T > 65535) return (int)hipErrorInvalidValue;
   return launch_moe_mfma<MM_DOWN>(128, (M + 127) / 128, (hipStream_t)stream, y, (const bf16_t*)x,
-                                (const bf16_t*)W, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 1, M, K, N, 0, 0);
+                                (const bf16_t*)W, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, 1, M, K, N, JvAct{}, 0);
 }

@@ -26,7 +26,7 @@ __global__ void __launch_bounds__(256)
 moe_skinny_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, const bf16_t* __restrict__ W0,
                   const bf16_t* __restrict__ W1, const int* __restrict__ meta, const int* __restrict__ offsets,
                   const int* __restrict__ tile_expert, const int* __restrict__ tile_row0, const int* __restrict__ order,
-                  const float* __restrict__ weights, int top, int n_tokens, int K, int N, int act, int use_weight) {
+                  const float* __restrict__ weights, int top, int n_tokens, int K, int N, JvAct act, int use_weight) {
   constexpr bool GATED = MODE == MS_GATED, BY_TOKEN = MODE != MS_DOWN;
   constexpr int STEPS = MS_STEPS, NB = 64 / WK;          // rows of W a block takes
   __shared__ float red[GATED ? 2 : 1][4][16][17];
@@ -104,7 +104,7 @@ moe_skinny_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, con
     if (MODE == MS_GATED) {
       ((bf16_t*)out)[(long long)(row0 + m) * N + n] = from_f32<bf16_t>(jv_gated(act, y0 * w, y1 * w));
     } else if (MODE == MS_PLAIN) {
-      ((bf16_t*)out)[(long long)(row0 + m) * N + n] = from_f32<bf16_t>(jv_act(act, y0 * w));
+      ((bf16_t*)out)[(long long)(row0 + m) * N + n] = from_f32<bf16_t>(jv_act(act.id, y0 * w));
     } else {
       const int token = s / top, kk = s - token * top;
       ((float*)out)[((long long)kk * n_tokens + token) * N + n] = y0 * w;
@@ -115,7 +115,7 @@ moe_skinny_kernel(void* __restrict__ out, const bf16_t* __restrict__ a_rows, con
 template <int MODE>
 static int launch_moe_skinny(void* out, const void* a, const void* W0, const void* W1, const int* meta, const int* offsets,
                              const int* tile_expert, const int* tile_row0, const int* order, const float* weights,
-                             int max_tiles, int top, int n_tokens, int K, int N, int act, int use_weight, void* stream) {
+                             int max_tiles, int top, int n_tokens, int K, int N, JvAct act, int use_weight, void* stream) {
   if (K < 8 || K % 8) return (int)hipErrorInvalidValue;
   const int wk = K >= 2048 ? 4 : 2;
   auto kernel = wk == 4 ? moe_skinny_kernel<MODE, 4> : moe_skinny_kernel<MODE, 2>;
@@ -135,14 +135,14 @@ extern "C" int jv_moe_skinny_rows() { return MS_ROWS; }
 extern "C" int jv_moe_gate_up_skinny_bf16(void* z, const void* x, const void* Wg, const void* Wu, const int* meta,
                                           const int* offsets, const int* tile_expert, const int* tile_row0,
                                           const int* order, const float* weights, int max_tiles, int top, int hidden,
-                                          int ff, int act, int scale_input, void* stream) {
+                                          int ff, int act, float act_limit, float act_slope, int scale_input, void* stream) {
   if (max_tiles <= 0 || ff <= 0) return 0;
   if (!(Wg ? jv_act_known(act) : jv_plain_act_known(act))) return (int)hipErrorInvalidValue;
   if (Wg)
     return launch_moe_skinny<MS_GATED>(z, x, Wg, Wu, meta, offsets, tile_expert, tile_row0, order, weights, max_tiles, top,
-                                       0, hidden, ff, act, scale_input, stream);
+                                       0, hidden, ff, JvAct{act, act_limit, act_slope}, scale_input, stream);
   return launch_moe_skinny<MS_PLAIN>(z, x, Wu, nullptr, meta, offsets, tile_expert, tile_row0, order, weights, max_tiles,
-                                     top, 0, hidden, ff, act, scale_input, stream);
+                                     top, 0, hidden, ff, JvAct{act, act_limit, act_slope}, scale_input, stream);
 }
 
 // down: z [entries, ff] by position, Wd [experts, hidden, ff] -> y [top, tokens, hidden] float
@@ -152,5 +152,5 @@ extern "C" int jv_moe_down_skinny_bf16(float* y, const void* z, const void* Wd, 
                                        int scale_output, void* stream) {
   if (max_tiles <= 0 || hidden <= 0) return 0;
   return launch_moe_skinny<MS_DOWN>(y, z, Wd, nullptr, meta, offsets, tile_expert, tile_row0, order, weights, max_tiles,
-                                    top, n_tokens, ff, hidden, 0, scale_output, stream);
+                                    top, n_tokens, ff, hidden, JvAct{}, scale_output, stream);
 }

@@ -72,6 +72,13 @@ __device__ __forceinline__ int first_key(int pos, int window) {
   return pos - window + 1 > 0 ? pos - window + 1 : 0;
 }
 
+// The score under a cap: cap * tanh(s / cap) of the scaled score, from the raw one (`in` = scale / cap).  Exact to a few
+// units of 2^-24 of the cap, which is what a score of that size is rounded to.
+__device__ __forceinline__ float capped_score(float raw, float in, float cap) {
+  const float e = fast_exp2(raw * in * 2.8853900817779268f);         // e^(2 s / cap); infinity gives cap, 0 gives -cap
+  return cap - 2.f * cap * __builtin_amdgcn_rcpf(e + 1.f);
+}
+
 struct AttnArgs {
   bf16_t* out;                // [tokens, nq * D]
   const bf16_t* q;            // row t at q + t * q_row_stride, head h at + h * D
@@ -87,6 +94,9 @@ struct AttnArgs {
   float scale_log2;           // softmax scale * log2(e)
   int window;                 // which keys a row sees, see first_key()
   const float* sinks;         // [nq] or null: exp(sinks[h]) joins every row's softmax denominator (no key, no value, unscaled)
+  // kernels with MORE only
+  float cap, cap_in;          // cap > 0: a score is capped (capped_score), cap_in = scale / cap and scale_log2 = log2(e)
+  int keep;                   // the first `keep` keys are seen by every row at or behind them, whatever its window
   // decode only
   int num_splits;
   float* part_acc;            // [n_work, nq, num_splits, D]
@@ -119,7 +129,8 @@ constexpr int NO_GAP = 0x7fffffff;
 #ifndef JV_PREFILL32
 // PAGES: 1 = the page size is 8, 16, 32 or 64 (pages tile the 64 keys: a thread's slot in its
 // page is the same in every tile), 2 = a larger power of two, 0 = any other multiple of 8.
-template <int PAGES>
+// MORE: capped scores and kept first keys (AttnArgs) are looked at.
+template <int PAGES, bool MORE>
 __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(AttnArgs p) {
   __shared__ __attribute__((aligned(16))) bf16_t Ks[BN * KS_STRIDE];
   __shared__ __attribute__((aligned(16))) bf16_t Vt[D * VT_STRIDE];
@@ -194,7 +205,18 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
     const int e0_up = (e0 + BN - 1) / BN * BN;
     if (b1 > e0_up) { gap_from = e0_up; gap_to = b1; }
   }
-  auto next_tile = [&](int j0) { return j0 + BN == gap_from ? gap_to : j0 + BN; };
+  // kept first keys: the walk begins at key 0 and jumps from behind them to the window's first tile
+  int keep_from = NO_GAP, keep_to = NO_GAP;
+  if (MORE && p.keep > 0 && kv_end > j_first) {
+    const int keep_up = (p.keep + BN - 1) / BN * BN;
+    if (keep_up < j_first) { keep_from = keep_up; keep_to = j_first; }
+    if (keep_up > gap_from) gap_from = keep_up < gap_to ? keep_up : NO_GAP;     // kept keys in the gap are not jumped over
+    j_first = 0;
+  }
+  auto next_tile = [&](int j0) {
+    if (MORE && j0 + BN == keep_from) return keep_to;
+    return j0 + BN == gap_from ? gap_to : j0 + BN;
+  };
   if (kv_end <= j_first) return;                    // nothing to do (the same in every thread)
 
   // A slice of the request's page table sits in LDS: a tile's loads then hang on one global
@@ -390,8 +412,14 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
 #pragma unroll
     for (int t = 0; t < RT; ++t) {
       if (!((MASK >> t) & 1)) continue;
+      if (MORE && p.cap > 0.f) {
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) s[t][kt][e] = capped_score(s[t][kt][e], p.cap_in, p.cap);
+      }
       // interior tile: every key visible to every row of the tile -> no per-element mask
-      const bool interior = (j0 + BN - 1 <= wave_min_pos[t]) && j0 >= wave_full_begin[t];
+      const bool interior = (j0 + BN - 1 <= wave_min_pos[t]) && (j0 >= wave_full_begin[t] || (MORE && j0 + BN <= p.keep));
       float tmax = -INFINITY;
       // the maximum is taken over raw scores (the scale is positive); the scale enters in the
       // exponent's multiply-add: p = exp2(s * scale_log2 - m * scale_log2)
@@ -406,7 +434,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
             const int j = j0 + kt * 16 + lc * 4 + e;
-            const bool ok = row_ok[t] && j <= pos[t] && j >= row_first[t];
+            const bool ok = row_ok[t] && j <= pos[t] && (j >= row_first[t] || (MORE && j < p.keep));
             const float v = ok ? s[t][kt][e] : -INFINITY;
             s[t][kt][e] = v;
             tmax = fmaxf(tmax, v);
@@ -470,7 +498,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_prefill_kernel(Att
     int mask = 0;
 #pragma unroll
     for (int t = 0; t < RT; ++t)
-      if (wave_live[t] && j0 < wave_kv_end[t] && j0 + BN > wave_kv_begin[t]) mask |= 1 << t;
+      if (wave_live[t] && j0 < wave_kv_end[t] && (j0 + BN > wave_kv_begin[t] || (MORE && j0 < p.keep))) mask |= 1 << t;
     if (RT > 1 && mask == 3) multiply(std::integral_constant<int, 3>{}, j0);
     else if (RT > 1 && mask == 2) multiply(std::integral_constant<int, 2>{}, j0);
     else if (mask == 1) multiply(std::integral_constant<int, 1>{}, j0);
@@ -537,7 +565,7 @@ constexpr int PCS = BN * CPK / 256;        // 16-byte pieces of a K tile (and of
 constexpr bool KB_ADDS = (32 * CPK / 16) % 16 == 0;   // the second key block's chunks are the first's plus a constant
 __device__ __forceinline__ int swizzle(int q) { return q ^ ((q >> 4) & 15); }   // chunk index -> chunk position
 
-template <int PAGES>
+template <int PAGES, bool MORE>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) attn_prefill32_kernel(AttnArgs p) {
   __shared__ __attribute__((aligned(16))) bf16_t Ks[2][BN * D];
   __shared__ __attribute__((aligned(16))) bf16_t Vs[2][D * BN];
@@ -608,7 +636,18 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     const int e0_up = (e0 + BN - 1) / BN * BN;
     if (b1 > e0_up) { gap_from = e0_up; gap_to = b1; }
   }
-  auto next_tile = [&](int j0) { return j0 + BN == gap_from ? gap_to : j0 + BN; };
+  // kept first keys: the walk begins at key 0 and jumps from behind them to the window's first tile
+  int keep_from = NO_GAP, keep_to = NO_GAP;
+  if (MORE && p.keep > 0 && kv_end > j_first) {
+    const int keep_up = (p.keep + BN - 1) / BN * BN;
+    if (keep_up < j_first) { keep_from = keep_up; keep_to = j_first; }
+    if (keep_up > gap_from) gap_from = keep_up < gap_to ? keep_up : NO_GAP;     // kept keys in the gap are not jumped over
+    j_first = 0;
+  }
+  auto next_tile = [&](int j0) {
+    if (MORE && j0 + BN == keep_from) return keep_to;
+    return j0 + BN == gap_from ? gap_to : j0 + BN;
+  };
   if (kv_end <= j_first) return;                    // nothing to do (the same in every thread)
 
   const int last_page = ps.index(kv_end - 1);
@@ -792,8 +831,14 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     };
     read_v(0, vf[0]);                    // on its way during the softmax
     __builtin_amdgcn_sched_barrier(0);
+    if (MORE && p.cap > 0.f) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) s[kb][e] = capped_score(s[kb][e], p.cap_in, p.cap);
+    }
     // interior tile: every key visible to every row of the tile -> no per-element mask
-    const bool interior = (j0 + BN - 1 <= wave_min_pos) && j0 >= wave_full_begin;
+    const bool interior = (j0 + BN - 1 <= wave_min_pos) && (j0 >= wave_full_begin || (MORE && j0 + BN <= p.keep));
     float tmax = -INFINITY;
     if (interior) {
 #pragma unroll
@@ -806,7 +851,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int j = j0 + kb * 32 + acc_key(e);
-          const bool ok = row_ok && j <= pos && j >= row_first;
+          const bool ok = row_ok && j <= pos && (j >= row_first || (MORE && j < p.keep));
           const float v = ok ? s[kb][e] : -INFINITY;
           s[kb][e] = v;
           tmax = fmaxf(tmax, v);
@@ -886,7 +931,13 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
     };
     // the row's maximum over the tile, the new reference if it has grown; returns whether any row of the wave moved
     auto row_max = [&](f32x16 (&sc)[2], int j0, float& alpha) -> bool {
-      const bool interior = (j0 + BN - 1 <= wave_min_pos) && j0 >= wave_full_begin;
+      if (MORE && p.cap > 0.f) {
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+          for (int e = 0; e < 16; ++e) sc[kb][e] = capped_score(sc[kb][e], p.cap_in, p.cap);
+      }
+      const bool interior = (j0 + BN - 1 <= wave_min_pos) && (j0 >= wave_full_begin || (MORE && j0 + BN <= p.keep));
       float tmax = -INFINITY;
       if (interior) {
 #pragma unroll
@@ -899,7 +950,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
 #pragma unroll
           for (int e = 0; e < 16; ++e) {
             const int j = j0 + kb * 32 + acc_key(e);
-            const bool ok = row_ok && j <= pos && j >= row_first;
+            const bool ok = row_ok && j <= pos && (j >= row_first || (MORE && j < p.keep));
             const float v = ok ? sc[kb][e] : -INFINITY;
             sc[kb][e] = v;
             tmax = fmaxf(tmax, v);
@@ -1074,7 +1125,7 @@ __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))
       const bool more = j_next < kv_end;
       if (more) fetch(j_next, b ^ 1);                 // in flight while this tile is multiplied; nobody reads that
                                                       // buffer: its tile was finished before the last barrier
-      if (wave_live && j0 < wave_kv_end && j0 + BN > wave_kv_begin) multiply(j0, b);
+      if (wave_live && j0 < wave_kv_end && (j0 + BN > wave_kv_begin || (MORE && j0 < p.keep))) multiply(j0, b);
       arrived();
       if (more && j_next + BN > kv_end) fix_tail(j_next, b ^ 1);   // own pieces only: no barrier needed before
       __syncthreads();
@@ -1116,6 +1167,7 @@ extern "C" int jv_attn_prefill_waves_split() { return 0; }
 constexpr int BND = 32;  // keys per wave iteration
 constexpr int DEC_TBL_MAX = 4096;  // page-table entries of a request that a decode block keeps in LDS
 
+template <bool MORE>
 __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(AttnArgs p) {
   extern __shared__ float smem[];  // per wave: m[16], l[16], acc[16][D]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -1162,27 +1214,48 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(Attn
     }
   }
   // tiles of this split, shared out to the 4 waves round-robin
-  const int t_first = kv_begin / BND, t_total = (kv_len + BND - 1) / BND - t_first;
+  // (with kept first keys the tiles in front of the window that hold them are shared out too: tile numbers are then
+  // counted without the gap, t_first - n_keep .. , and the first n_keep of them stand for tiles 0, 1, ...)
+  const int t_first = kv_begin / BND;
+  int n_keep = 0;
+  if (MORE) {
+    n_keep = (p.keep + BND - 1) / BND;
+    if (n_keep > t_first) n_keep = t_first;
+  }
+  const int t_total = (kv_len + BND - 1) / BND - t_first + n_keep;
   const int per_split = (t_total + p.num_splits - 1) / p.num_splits;
-  const int t_lo = t_first + split * per_split;
+  const int t_lo = t_first - n_keep + split * per_split;
   int t_hi = t_lo + per_split;
-  if (t_hi > t_first + t_total) t_hi = t_first + t_total;
+  if (t_hi > t_first - n_keep + t_total) t_hi = t_first - n_keep + t_total;
+  auto first_key_of = [&](int t) { return (MORE && t < t_first ? t - (t_first - n_keep) : t) * BND; };
 
   float m_run = -INFINITY, l_lane = 0.f;
   f32x4 acc[NDT];
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt) acc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  int tbl_first = 0;                      // table entry that tbl[0] holds
+  int tbl_first = 0;                      // table entry that tbl[0] holds (tbl[kept_entries] with kept first keys)
+  int kept_entries = 0;                   // entries of the kept first keys, in front of the split's own
   if (!whole_row && t_lo < t_hi) {
-    tbl_first = ps.index(t_lo * BND);
+    if (MORE && n_keep > 0) {
+      kept_entries = ps.index(n_keep * BND - 1) + 1;
+      for (int i = tid; i < kept_entries; i += 256) tbl[i] = gtable[i];
+    }
+    // (a split of kept keys alone has no entries of its own)
+    const int j_lo = (MORE && t_lo < t_first ? t_first : t_lo) * BND;
     const int j_last = (t_hi * BND < kv_len ? t_hi * BND : kv_len) - 1;
-    int n = ps.index(j_last) - tbl_first + 1;
-    if (n > DEC_TBL_MAX) n = DEC_TBL_MAX;             // never, by the entry point's check
-    for (int i = tid; i < n; i += 256) tbl[i] = gtable[tbl_first + i];
+    tbl_first = ps.index(j_lo);
+    int n = j_last >= j_lo ? ps.index(j_last) - tbl_first + 1 : 0;
+    if (n > DEC_TBL_MAX - kept_entries) n = DEC_TBL_MAX - kept_entries;       // never, by the entry point's check
+    for (int i = tid; i < n; i += 256) tbl[kept_entries + i] = gtable[tbl_first + i];
   }
   __syncthreads();   // the table entries are in LDS
-  auto page_at = [&](int idx) -> long long { return tbl[idx - tbl_first]; };
+  auto page_at = [&](int idx) -> long long {
+    if (MORE && idx < kept_entries) return tbl[idx];
+    return tbl[idx - tbl_first + kept_entries];
+  };
+  // an entry that is there whatever the split's keys are: what a lane without a key of its own looks up
+  const int some_entry = MORE && kept_entries > 0 ? 0 : tbl_first;
   // One tile's operands, global -> registers.  Nothing here looks at a loaded value, so a tile's
   // loads are in flight while the tile before it is multiplied.  Keys at or past kv_len read the
   // null page: their scores are masked by position, their V entries are zeroed before use.
@@ -1192,12 +1265,12 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(Attn
   // prefetch is never skipped: after a conditional one the compiler must assume that nothing younger is
   // in flight, and its waits for this tile's operands would wait for the prefetched tile as well.
   auto load_tile = [&](int t, bool real, bf16x8 (&kf)[2][NKS], bf16x4 (&vf)[2][NDT]) {
-    const int j0 = t * BND;
+    const int j0 = first_key_of(t);
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt) {
       const int j = j0 + kt * 16 + li;
       const bool ok = real && j < kv_len;
-      const long long looked = page_at(ok ? ps.index(j) : tbl_first);
+      const long long looked = page_at(ok ? ps.index(j) : some_entry);
       const long long page = ok ? looked : 0;
       const bf16_t* krow = p.k_pages + ((page * p.nkv + g) * P + (ok ? ps.slot(j) : 0)) * (long long)D;
 #pragma unroll
@@ -1210,7 +1283,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(Attn
     for (int kt = 0; kt < 2; ++kt) {
       const int j = j0 + kt * 16 + lc * 4;
       const bool ok = real && j < kv_len;
-      const long long looked = page_at(ok ? ps.index(j) : tbl_first);
+      const long long looked = page_at(ok ? ps.index(j) : some_entry);
       const long long page = ok ? looked : 0;
       const bf16_t* vbase = p.v_pages + (page * p.nkv + g) * (long long)D * P + (ok ? ps.slot(j) : 0);
 #pragma unroll
@@ -1218,7 +1291,7 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(Attn
     }
   };
   auto multiply = [&](int t, bf16x8 (&kf)[2][NKS], bf16x4 (&vf)[2][NDT]) {
-    const int j0 = t * BND;
+    const int j0 = first_key_of(t);
     if (DK != D) {                       // columns that pad the head size to the contraction step
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
@@ -1248,8 +1321,9 @@ __global__ void __launch_bounds__(256) PREFILL_OCCUPANCY attn_decode_kernel(Attn
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int j = j0 + kt * 16 + lc * 4 + e;
-        const bool ok = row_ok && j <= pos && j >= kv_begin;
-        const float v = ok ? s[kt][e] * p.scale_log2 : -INFINITY;
+        const bool ok = row_ok && j <= pos && (j >= kv_begin || (MORE && j < p.keep));
+        const float raw = MORE && p.cap > 0.f ? capped_score(s[kt][e], p.cap_in, p.cap) : s[kt][e];
+        const float v = ok ? raw * p.scale_log2 : -INFINITY;
         s[kt][e] = v;
         tmax = fmaxf(tmax, v);
       }
@@ -1389,8 +1463,18 @@ static int check_common(AttnArgs& a) {
   a.page_shift = -1;
   for (int sft = 3; sft < 31; ++sft)
     if ((1 << sft) == a.page_size) a.page_shift = sft;
-  if (a.nkv <= 0 || a.nq % a.nkv != 0) return (int)hipErrorInvalidValue;
+  if (a.nkv <= 0 || a.nq % a.nkv != 0 || a.keep < 0) return (int)hipErrorInvalidValue;
   return 0;
+}
+
+// Whether capped scores or kept first keys ask for the kernels with MORE; sets what those read.
+static bool set_more(AttnArgs& a, float scale) {
+  if (a.window == 0) a.keep = 0;            // every key is seen anyway
+  if (a.cap > 0.f) {
+    a.cap_in = scale / a.cap;
+    a.scale_log2 = 1.4426950408889634f;     // a capped score carries its scale
+  }
+  return a.cap > 0.f || a.keep > 0;
 }
 
 extern "C" int jv_attn_head_dim() { return D; }
@@ -1401,10 +1485,11 @@ extern "C" int jv_attn_prefill(void* out, const void* q, long long q_row_stride,
                                const void* v_pages, const int* block_tables, int table_stride,
                                const int* cu_seqlens, const int* context_lens, const int* work,
                                int n_work, int page_size, int nq, int nkv, float scale, int window,
-                               const float* sinks, void* stream) {
+                               const float* sinks, float cap, int keep, void* stream) {
   if (n_work <= 0) return 0;
   AttnArgs a{};
   a.sinks = sinks;
+  a.cap = cap; a.keep = keep;
   a.out = (bf16_t*)out; a.q = (const bf16_t*)q; a.q_row_stride = q_row_stride;
   a.k_pages = (const bf16_t*)k_pages; a.v_pages = (const bf16_t*)v_pages;
   a.block_tables = block_tables; a.table_stride = table_stride;
@@ -1412,17 +1497,25 @@ extern "C" int jv_attn_prefill(void* out, const void* q, long long q_row_stride,
   a.page_size = page_size; a.nq = nq; a.nkv = nkv;
   a.scale_log2 = scale * 1.4426950408889634f; a.window = window; a.num_splits = 1;
   if (int e = check_common(a)) return e;
+  const bool more = set_more(a, scale);
   if ((long long)nkv * page_size * D >= (1ll << 31)) return (int)hipErrorInvalidValue;   // offsets inside a page are 32-bit
   if ((long long)n_work * nkv >= (1ll << 31)) return (int)hipErrorInvalidValue;
   const int mode = (a.page_shift >= 3 && a.page_shift <= 6) ? 1 : (a.page_shift > 6 ? 2 : 0);
 #ifdef JV_PREFILL32
   constexpr bool pow2 = (D & (D - 1)) == 0;
-  void (*kernel)(AttnArgs) = (page_size == 16 && pow2) ? attn_prefill32_kernel<pow2 ? 16 : 1>
-                             : mode == 1 ? attn_prefill32_kernel<1>
-                             : mode == 2 ? attn_prefill32_kernel<2> : attn_prefill32_kernel<0>;
+  auto pick = [&](auto m) -> void (*)(AttnArgs) {
+    constexpr bool M = decltype(m)::value;
+    return (page_size == 16 && pow2) ? attn_prefill32_kernel<pow2 ? 16 : 1, M>
+           : mode == 1 ? attn_prefill32_kernel<1, M>
+           : mode == 2 ? attn_prefill32_kernel<2, M> : attn_prefill32_kernel<0, M>;
+  };
 #else
-  void (*kernel)(AttnArgs) = mode == 1 ? attn_prefill_kernel<1> : (mode == 2 ? attn_prefill_kernel<2> : attn_prefill_kernel<0>);
+  auto pick = [&](auto m) -> void (*)(AttnArgs) {
+    constexpr bool M = decltype(m)::value;
+    return mode == 1 ? attn_prefill_kernel<1, M> : (mode == 2 ? attn_prefill_kernel<2, M> : attn_prefill_kernel<0, M>);
+  };
 #endif
+  void (*kernel)(AttnArgs) = more ? pick(std::true_type{}) : pick(std::false_type{});
   hipLaunchKernelGGL(kernel, dim3(n_work * nkv), dim3(256), 0, (hipStream_t)stream, a);
   return JV_LAUNCH_CHECK();
 }
@@ -1436,10 +1529,12 @@ extern "C" int jv_attn_decode(void* out, const void* q, long long q_row_stride, 
                               const void* v_pages, const int* block_tables, int table_stride,
                               const int* cu_seqlens, const int* context_lens, const int* work,
                               int n_work, int page_size, int nq, int nkv, float scale, int window,
-                              int num_splits, float* scratch, const float* sinks, void* stream) {
+                              int num_splits, float* scratch, const float* sinks, float cap, int keep,
+                              void* stream) {
   if (n_work <= 0) return 0;
   AttnArgs a{};
   a.sinks = sinks;
+  a.cap = cap; a.keep = keep;
   a.out = (bf16_t*)out; a.q = (const bf16_t*)q; a.q_row_stride = q_row_stride;
   a.k_pages = (const bf16_t*)k_pages; a.v_pages = (const bf16_t*)v_pages;
   a.block_tables = block_tables; a.table_stride = table_stride;
@@ -1448,6 +1543,7 @@ extern "C" int jv_attn_decode(void* out, const void* q, long long q_row_stride, 
   a.scale_log2 = scale * 1.4426950408889634f; a.window = window;
   a.num_splits = num_splits < 1 ? 1 : num_splits;
   if (int e = check_common(a)) return e;
+  const bool more = set_more(a, scale);
   if (a.num_splits > 1) {
     if (!scratch) return (int)hipErrorInvalidValue;
     a.part_acc = scratch;
@@ -1460,16 +1556,18 @@ extern "C" int jv_attn_decode(void* out, const void* q, long long q_row_stride, 
   if (table_stride > DEC_TBL_MAX) {
     const long long tiles = ((long long)table_stride * page_size + BND - 1) / BND;
     const long long per_split = (tiles + a.num_splits - 1) / a.num_splits;
-    if (per_split * BND / page_size + 2 > DEC_TBL_MAX) return (int)hipErrorInvalidValue;
+    const long long kept = (a.keep + BND - 1) / BND * BND / page_size + 1;
+    if (per_split * BND / page_size + 2 + (a.keep > 0 ? kept : 0) > DEC_TBL_MAX) return (int)hipErrorInvalidValue;
   }
   const size_t shmem = 4 * (32 + 16 * D) * sizeof(float) +
                        (size_t)(table_stride <= DEC_TBL_MAX ? table_stride : DEC_TBL_MAX) * sizeof(int);
+  void (*kernel)(AttnArgs) = more ? attn_decode_kernel<true> : attn_decode_kernel<false>;
   if (shmem > 64 * 1024) {
-    hipError_t e = hipFuncSetAttribute((const void*)attn_decode_kernel,
+    hipError_t e = hipFuncSetAttribute((const void*)kernel,
                                        hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem);
     if (e != hipSuccess) return (int)e;
   }
-  hipLaunchKernelGGL(attn_decode_kernel, dim3(n_work, nkv * mt_per_head, a.num_splits), dim3(256),
+  hipLaunchKernelGGL(kernel, dim3(n_work, nkv * mt_per_head, a.num_splits), dim3(256),
                      shmem, (hipStream_t)stream, a);
   int e = JV_LAUNCH_CHECK();
   if (e) return e;

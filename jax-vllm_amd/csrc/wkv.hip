@@ -9,6 +9,10 @@
 //                       o_t = S^T r_t + (sum_d r_t[d] u[d] k_t[d]) v_t     (the bonus u counts for the current token only)
 //                       S   <- diag(w_t) S + k_t v_t^T
 //   wkv_chunks        the same by chunks of 32 tokens, for prompt portions (see below)
+// Both also run the form of gated linear attention (AFTER): the logarithms of the decays are given as floats (`rate`), r is
+// multiplied by a constant, and the output is read from the state AFTER the token's update, without a bonus:
+//                       S   <- diag(e^rate_t) S + k_t v_t^T;    o_t = S^T (r_scale r_t)
+//   low_rank_decay    those logarithms, log(sigmoid(z)) / tau with z = W low + b from a projection of small rank
 //
 // r, k, v and the decay's rate are products in the activation type; everything from there on is float.  The state of a
 // request lives in a row of `state` [slots + 1][heads][dim][vdim] between steps.  Columns of S never mix, so a block
@@ -87,11 +91,18 @@ token_shift_mix_vec_kernel(T* __restrict__ out, const T* __restrict__ x, const f
 // grid (requests, heads, column slices); block 256 = parts x cols threads, cols a power of two.
 // r, k, rate: [n][heads][dim] with row strides ldr, ldk, ldw; v [n][heads][vdim] with row stride ldv; w0, u [heads][dim]
 // float; out [n][heads * vdim] float.
-template <typename T>
+// The logarithm of a decay: given as a float, or -exp(rate + w0).
+template <typename T, bool AFTER>
+__device__ __forceinline__ float wkv_log_decay(const void* rate, long long at, const float* w0, int c) {
+  if (AFTER) return ((const float*)rate)[at];
+  return -expf(to_f32(((const T*)rate)[at]) + w0[c]);
+}
+
+template <typename T, bool AFTER>
 __global__ void __launch_bounds__(256)
 wkv_steps_kernel(float* __restrict__ out, const T* __restrict__ rr, long long ldr, const T* __restrict__ kk,
-                 long long ldk, const T* __restrict__ vv, long long ldv, const T* __restrict__ rate, long long ldw,
-                 const float* __restrict__ w0, const float* __restrict__ bonus, float* __restrict__ state,
+                 long long ldk, const T* __restrict__ vv, long long ldv, const void* __restrict__ rate, long long ldw,
+                 const float* __restrict__ w0, const float* __restrict__ bonus, float r_scale, float* __restrict__ state,
                  const int* __restrict__ slot_ids, const int* __restrict__ cu_seqlens, int heads, int dim, int vdim,
                  int cols) {
   extern __shared__ float lds[];          // 2 x (r[dim] | k[dim] | w[dim] | v[cols]) | partial sums [parts][cols]
@@ -109,14 +120,14 @@ wkv_steps_kernel(float* __restrict__ out, const T* __restrict__ rr, long long ld
   for (int i = 0; i < WKV_ROWS; ++i) {
     const int d = part + i * parts;
     s[i] = (live && d < dim) ? S[(long long)d * vdim] : 0.f;
-    ub[i] = d < dim ? bonus[h * dim + d] : 0.f;
+    ub[i] = !AFTER && d < dim ? bonus[h * dim + d] : 0.f;
   }
   for (int t = t0; t < t1; ++t) {
     float* buf = lds + ((t - t0) & 1) * stage;
     for (int d = threadIdx.x; d < dim; d += blockDim.x) {
-      buf[d] = to_f32(rr[(long long)t * ldr + h * dim + d]);
+      buf[d] = to_f32(rr[(long long)t * ldr + h * dim + d]) * (AFTER ? r_scale : 1.f);
       buf[dim + d] = to_f32(kk[(long long)t * ldk + h * dim + d]);
-      buf[2 * dim + d] = expf(-expf(to_f32(rate[(long long)t * ldw + h * dim + d]) + w0[h * dim + d]));
+      buf[2 * dim + d] = expf(wkv_log_decay<T, AFTER>(rate, (long long)t * ldw + h * dim + d, w0, h * dim + d));
     }
     if (threadIdx.x < cols)
       buf[3 * dim + threadIdx.x] = (c0 + threadIdx.x < vdim) ? to_f32(vv[(long long)t * ldv + h * vdim + c0 + threadIdx.x]) : 0.f;
@@ -128,8 +139,9 @@ wkv_steps_kernel(float* __restrict__ out, const T* __restrict__ rr, long long ld
       const int d = part + i * parts;
       if (d < dim) {
         const float kv = buf[dim + d] * v;
-        acc = fmaf(buf[d], fmaf(ub[i], kv, s[i]), acc);
+        if (!AFTER) acc = fmaf(buf[d], fmaf(ub[i], kv, s[i]), acc);
         s[i] = fmaf(buf[2 * dim + d], s[i], kv);
+        if (AFTER) acc = fmaf(buf[d], s[i], acc);
       }
     }
     red[part * cols + col] = acc;
@@ -155,7 +167,8 @@ wkv_steps_kernel(float* __restrict__ out, const T* __restrict__ rr, long long ld
 //     a[t][j] = sum_c r_t[c] k_j[c] exp(b_(t-1)[c] - b_j[c])  (j < t),     a[t][t] = sum_c r_t[c] u[c] k_t[c]
 //     S_end = diag(exp(b_(n-1))) S0 + sum_j (k_j * exp(b_(n-1) - b_j)) v_j^T
 // Only differences <= 0 are exponentiated, channel by channel (no product of a grown query with a shrunk key, which
-// would overflow).  Three launches, so that the chunks of a long prompt run side by side and only the cheap part is serial:
+// would overflow).  AFTER: the decay up to and with token t counts for its output, exp(b_t) and exp(b_t - b_j) in place of
+// exp(b_(t-1)) and exp(b_(t-1) - b_j), and a[t][t] = sum_c r_t[c] k_t[c].  Three launches, so that the chunks of a long prompt run side by side and only the cheap part is serial:
 //   local:  per (chunk, head)   out_t = sum_j a[t][j] v_j;  U = sum_j k'_j v_j^T -> scratch[chunk];  r_t * exp(b_(t-1)) -> rq;
 //                               exp(b_(n-1)) -> dtot[chunk]
 //   scan:   per (request, head) for its chunks in order: scratch[chunk] <- S (the state BEFORE the chunk),
@@ -169,12 +182,12 @@ wkv_steps_kernel(float* __restrict__ out, const T* __restrict__ rr, long long ld
 // below a hundred-millionth absolutely, which is the float rounding of the sums these weights enter.
 __device__ __forceinline__ float wkv_exp_neg(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
 
-template <typename T>
+template <typename T, bool AFTER>
 __global__ void __launch_bounds__(256)
 wkv_local_kernel(float* __restrict__ out, float* __restrict__ scratch, float* __restrict__ rq, float* __restrict__ dtot,
                  const T* __restrict__ rr, long long ldr, const T* __restrict__ kk, long long ldk,
-                 const T* __restrict__ vv, long long ldv, const T* __restrict__ rate, long long ldw,
-                 const float* __restrict__ w0, const float* __restrict__ bonus, const int* __restrict__ work,
+                 const T* __restrict__ vv, long long ldv, const void* __restrict__ rate, long long ldw,
+                 const float* __restrict__ w0, const float* __restrict__ bonus, float r_scale, const int* __restrict__ work,
                  const int* __restrict__ cu_seqlens, int heads, int dim, int vdim) {
   extern __shared__ float lds[];      // r [LC][dim + 1] | k [LC][dim + 1] | b [LC][dim + 1] | a [LC][LC + 1] | v [LC][CW] | u [dim]
   const int ld = dim + 1;
@@ -185,7 +198,7 @@ wkv_local_kernel(float* __restrict__ out, float* __restrict__ scratch, float* __
   float* vs = as + WKV_LC * (WKV_LC + 1);
   float* us = vs + WKV_LC * WKV_CW;
   const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
-  for (int c = tid; c < dim; c += 256) us[c] = bonus[h * dim + c];
+  for (int c = tid; c < dim; c += 256) us[c] = AFTER ? 1.f : bonus[h * dim + c];
   const int req = work[2 * ch], b0 = work[2 * ch + 1];
   const int n = min(WKV_LC, cu_seqlens[req + 1] - b0);
   for (int i = tid; i < WKV_LC * dim; i += 256) {
@@ -193,9 +206,9 @@ wkv_local_kernel(float* __restrict__ out, float* __restrict__ scratch, float* __
     float r = 0.f, k = 0.f, l = 0.f;
     if (t < n) {
       const long long row = b0 + t;
-      r = to_f32(rr[row * ldr + h * dim + c]);
+      r = to_f32(rr[row * ldr + h * dim + c]) * (AFTER ? r_scale : 1.f);
       k = to_f32(kk[row * ldk + h * dim + c]);
-      l = fmaxf(-expf(to_f32(rate[row * ldw + h * dim + c]) + w0[h * dim + c]), -WKV_MIN_LOG);
+      l = fmaxf(wkv_log_decay<T, AFTER>(rate, row * ldw + h * dim + c, w0, h * dim + c), -WKV_MIN_LOG);
     }
     rs[t * ld + c] = r;
     ks[t * ld + c] = k;
@@ -208,7 +221,7 @@ wkv_local_kernel(float* __restrict__ out, float* __restrict__ scratch, float* __
       const float before = run;
       run += bs[t * ld + c];
       bs[t * ld + c] = run;
-      if (t < n) rq[(long long)(b0 + t) * heads * dim + h * dim + c] = rs[t * ld + c] * wkv_exp_neg(before);
+      if (t < n) rq[(long long)(b0 + t) * heads * dim + h * dim + c] = rs[t * ld + c] * wkv_exp_neg(AFTER ? run : before);
     }
     dtot[((long long)ch * heads + h) * dim + c] = wkv_exp_neg(run);
   }
@@ -219,7 +232,7 @@ wkv_local_kernel(float* __restrict__ out, float* __restrict__ scratch, float* __
     if (j < t) {
 #pragma unroll 4
       for (int c = 0; c < dim; ++c)
-        a = fmaf(rs[t * ld + c] * ks[j * ld + c], wkv_exp_neg(bs[(t - 1) * ld + c] - bs[j * ld + c]), a);
+        a = fmaf(rs[t * ld + c] * ks[j * ld + c], wkv_exp_neg(bs[(t - (AFTER ? 0 : 1)) * ld + c] - bs[j * ld + c]), a);
     } else if (j == t) {
       for (int c = 0; c < dim; ++c) a = fmaf(rs[t * ld + c] * ks[t * ld + c], us[c], a);
     }
@@ -331,6 +344,38 @@ wkv_apply_kernel(float* __restrict__ out, const float* __restrict__ scratch, con
   }
 }
 
+// ---------------------------------------------------------------- decays from a projection of small rank
+// out[t][c] = log(sigmoid(z)) / tau,  z = sum_r W[c][r] low[t][r] + b[c]; W [channels][rank] and low (rows of stride ldl) in
+// the activation type, sums and logarithm float.  grid (channel blocks of 256, blocks of LD_TOKENS tokens).
+#define LD_TOKENS 8
+template <typename T>
+__global__ void __launch_bounds__(256)
+low_rank_decay_kernel(float* __restrict__ out, const T* __restrict__ low, long long ldl, const T* __restrict__ W,
+                      const float* __restrict__ b, long long n, int channels, int rank, float inv_tau) {
+  extern __shared__ float lows[];         // [LD_TOKENS][rank]
+  const long long t0 = (long long)blockIdx.y * LD_TOKENS;
+  for (int i = threadIdx.x; i < LD_TOKENS * rank; i += 256) {
+    const int t = i / rank;
+    lows[i] = t0 + t < n ? to_f32(low[(t0 + t) * ldl + (i - t * rank)]) : 0.f;
+  }
+  __syncthreads();
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= channels) return;
+  float z[LD_TOKENS];
+#pragma unroll
+  for (int t = 0; t < LD_TOKENS; ++t) z[t] = b[c];
+  const T* w = W + (long long)c * rank;
+#pragma unroll 8
+  for (int r = 0; r < rank; ++r) {
+    const float wv = to_f32(w[r]);
+#pragma unroll
+    for (int t = 0; t < LD_TOKENS; ++t) z[t] = fmaf(wv, lows[t * rank + r], z[t]);
+  }
+#pragma unroll
+  for (int t = 0; t < LD_TOKENS; ++t)
+    if (t0 + t < n) out[(t0 + t) * channels + c] = -(fmaxf(-z[t], 0.f) + log1pf(expf(-fabsf(z[t])))) * inv_tau;
+}
+
 extern "C" int jv_wkv_max_dim() { return WKV_ROWS * 256; }
 extern "C" int jv_wkv_chunk_tokens() { return WKV_LC; }
 extern "C" int jv_wkv_chunk_max_dim() { return 128; }
@@ -355,7 +400,8 @@ extern "C" int jv_wkv_chunk_max_dim() { return 128; }
   }                                                                                                             \
   extern "C" int jv_wkv_steps_##SUF(float* out, const void* r, long long ldr, const void* k, long long ldk,     \
                                     const void* v, long long ldv, const void* rate, long long ldw,              \
-                                    const float* w0, const float* bonus, float* state, const int* slot_ids,     \
+                                    const float* w0, const float* bonus, int after, float r_scale,              \
+                                    float* state, const int* slot_ids,                                          \
                                     const int* cu_seqlens, int n_requests, int heads, int dim, int vdim,        \
                                     void* stream) {                                                             \
     if (n_requests <= 0 || heads <= 0) return 0;                                                                \
@@ -366,9 +412,22 @@ extern "C" int jv_wkv_chunk_max_dim() { return 128; }
     const int parts = 256 / cols;                                                                               \
     const size_t shmem = (2 * (3 * dim + cols) + parts * cols) * sizeof(float);                                 \
     if (shmem > 64 * 1024 || (vdim + cols - 1) / cols > 65535) return (int)hipErrorInvalidValue;                \
-    hipLaunchKernelGGL(wkv_steps_kernel<T>, dim3(n_requests, heads, (vdim + cols - 1) / cols), dim3(256),       \
+    if (!after && (!w0 || !bonus)) return (int)hipErrorInvalidValue;                                            \
+    auto kernel = after ? wkv_steps_kernel<T, true> : wkv_steps_kernel<T, false>;                               \
+    hipLaunchKernelGGL(kernel, dim3(n_requests, heads, (vdim + cols - 1) / cols), dim3(256),       \
                        shmem, (hipStream_t)stream, out, (const T*)r, ldr, (const T*)k, ldk, (const T*)v, ldv,   \
-                       (const T*)rate, ldw, w0, bonus, state, slot_ids, cu_seqlens, heads, dim, vdim, cols);    \
+                       rate, ldw, w0, bonus, r_scale, state, slot_ids, cu_seqlens, heads, dim, vdim, cols);     \
+    return JV_LAUNCH_CHECK();                                                                                   \
+  }                                                                                                             \
+  extern "C" int jv_low_rank_decay_##SUF(float* out, const void* low, long long ldl, const void* W,             \
+                                         const float* b, long long n, int channels, int rank, float tau,        \
+                                         void* stream) {                                                        \
+    if (n <= 0 || channels <= 0) return 0;                                                                      \
+    if (rank <= 0 || rank > 2048 || !(tau > 0.f) || (n + LD_TOKENS - 1) / LD_TOKENS > 65535)                    \
+      return (int)hipErrorInvalidValue;                                                                         \
+    hipLaunchKernelGGL(low_rank_decay_kernel<T>, dim3((channels + 255) / 256, (n + LD_TOKENS - 1) / LD_TOKENS), \
+                       dim3(256), (size_t)LD_TOKENS * rank * sizeof(float), (hipStream_t)stream, out,           \
+                       (const T*)low, ldl, (const T*)W, b, n, channels, rank, 1.f / tau);                       \
     return JV_LAUNCH_CHECK();                                                                                   \
   }
 
@@ -377,7 +436,8 @@ extern "C" int jv_wkv_chunk_max_dim() { return 128; }
 #define DEFINE_WKV_CHUNKS(SUF, T)                                                                               \
   extern "C" int jv_wkv_chunks_##SUF(float* out, const void* r, long long ldr, const void* k, long long ldk,    \
                                      const void* v, long long ldv, const void* rate, long long ldw,             \
-                                     const float* w0, const float* bonus, float* state, const int* slot_ids,    \
+                                     const float* w0, const float* bonus, int after, float r_scale,             \
+                                     float* state, const int* slot_ids,                                         \
                                      const int* cu_seqlens, int n_requests, int heads, int dim, int vdim,       \
                                      int chunks, const int* work, const int* req_chunks, float* scratch,        \
                                      float* rq, float* dtot, void* stream) {                                    \
@@ -387,8 +447,10 @@ extern "C" int jv_wkv_chunk_max_dim() { return 128; }
     if (((long long)dim * vdim + 255) / 256 > 65535) return (int)hipErrorInvalidValue;                          \
     hipStream_t s = (hipStream_t)stream;                                                                        \
     const size_t lds_local = (3 * WKV_LC * (dim + 1) + WKV_LC * (WKV_LC + 1) + WKV_LC * WKV_CW + dim) * sizeof(float); \
-    hipLaunchKernelGGL(wkv_local_kernel<T>, dim3(chunks, heads), dim3(256), lds_local, s, out, scratch, rq, dtot, \
-                       (const T*)r, ldr, (const T*)k, ldk, (const T*)v, ldv, (const T*)rate, ldw, w0, bonus,    \
+    if (!after && (!w0 || !bonus)) return (int)hipErrorInvalidValue;                                            \
+    auto local = after ? wkv_local_kernel<T, true> : wkv_local_kernel<T, false>;                                \
+    hipLaunchKernelGGL(local, dim3(chunks, heads), dim3(256), lds_local, s, out, scratch, rq, dtot, \
+                       (const T*)r, ldr, (const T*)k, ldk, (const T*)v, ldv, rate, ldw, w0, bonus, r_scale,     \
                        work, cu_seqlens, heads, dim, vdim);                                                     \
     hipLaunchKernelGGL(wkv_scan_kernel, dim3(n_requests, heads, (dim * vdim + 255) / 256), dim3(256), 0, s,     \
                        scratch, state, dtot, slot_ids, req_chunks, heads, dim, vdim);                           \

@@ -319,18 +319,33 @@ def softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 # --------------------------------------------------------------------------- activation
-GATE_ACTIVATIONS = {"silu": 1, "gelu_tanh": 2}      # the kernels' ids of act in y = act(gate) * up
+# The kernels' ids of act in y = act(gate) * up; "clamped": y = g sigmoid(slope g) (u + 1) with g = min(gate, limit) and
+# u = up clamped to [-limit, limit], named with its constants: ("clamped", limit, slope).
+GATE_ACTIVATIONS = {"silu": 1, "gelu_tanh": 2, "clamped": 6}
 
 
-def _gate_act_id(name) -> int:
-    _need(name in GATE_ACTIVATIONS, f"no kernel for the gate activation {name!r}: there are {sorted(GATE_ACTIVATIONS)}")
-    return GATE_ACTIVATIONS[name]
+def gate_activation_known(activation) -> bool:
+    """Whether the kernels have this activation of a gated feed-forward: a name, or ("clamped", limit, slope)."""
+    if isinstance(activation, tuple):
+        return len(activation) == 3 and activation[0] == "clamped" and float(activation[1]) > 0
+    return activation in GATE_ACTIVATIONS and activation != "clamped"
+
+
+def _gate_act(activation) -> tuple:
+    """(id, limit, slope) of a gated feed-forward's activation as the entry points take it."""
+    _need(gate_activation_known(activation), f"no kernel for the gate activation {activation!r}: there are {sorted(GATE_ACTIVATIONS)}, "
+          "the clamped one as (\"clamped\", limit, slope)")
+    name, limit, slope = activation if isinstance(activation, tuple) else (activation, 0.0, 0.0)
+    return c_int(GATE_ACTIVATIONS[name]), c_float(limit), c_float(slope)
+
+
+_NO_ACT = (c_int(0), c_float(0.0), c_float(0.0))
 
 
 def gated_mul(gate_up: torch.Tensor, out=None, interleaved: bool = False, activation: str = "silu") -> torch.Tensor:
     """out[t, j] = act(gate) * up for gate_up of width 2 I: gate = gate_up[t, j], up =
     gate_up[t, I + j], or with ``interleaved`` gate = gate_up[t, 2j], up = gate_up[t, 2j + 1];
-    ``activation`` is one of ``GATE_ACTIVATIONS``, computed in float."""
+    ``activation`` is one of ``GATE_ACTIVATIONS`` (see ``gate_activation_known``), computed in float."""
     _dev(gate_up)
     n, two_i = gate_up.shape
     _need(two_i % 2 == 0, "gate_up must have an even width")
@@ -341,7 +356,7 @@ def gated_mul(gate_up: torch.Tensor, out=None, interleaved: bool = False, activa
     _need(out.shape == (n, inter) and out.dtype == gate_up.dtype, "out must be [tokens, I] of gate_up's type")
     fn = getattr(library.core(), f"jv_gated_mul_{_suffix(gate_up.dtype)}")
     _check(fn(_ptr(out), _ptr(gate_up), c_longlong(n), c_int(inter), c_int(1 if interleaved else 0),
-              c_int(_gate_act_id(activation)), _stream()), "gated_mul")
+              *_gate_act(activation), _stream()), "gated_mul")
     return out
 
 
@@ -429,7 +444,7 @@ def padded_head_dim(dk: int, dv: int) -> int:
 def attn_prepare_wide(qkv, bias, q_weight, k_weight, eps: float, cos_sin, rot_dims: int, slot_mapping, k_pages, v_pages,
                       page_size: int, nq: int, nkv: int, dk: int, dv: int, dp: int, v_scale: float = 1.0,
                       norm_per_head: bool = False, values_are_keys: bool = False, positions=None,
-                      q_temperature: "tuple | None" = None) -> torch.Tensor:
+                      q_temperature: "tuple | None" = None, v_first=None, v_mix: float = 0.0) -> torch.Tensor:
     """Attention input whose key and value sizes differ, whose q/k norm spans the whole projection, or whose rows
     carry more than q, k and v.  ``qkv`` rows
     begin with [q: nq * dk | k: nkv * dk | v: nkv * dv] (further columns are left alone); ``bias`` (float32, that width) is added first; with
@@ -438,7 +453,9 @@ def attn_prepare_wide(qkv, bias, q_weight, k_weight, eps: float, cos_sin, rot_di
     first ``rot_dims`` elements of every q and k head turn by ``cos_sin`` (``rope_table``); v is multiplied by
     ``v_scale``.  ``values_are_keys``: the rows hold [q | k] only and the values are the k columns as projected (before
     bias-free norm and rotation; needs dv == dk and no whole-projection norm).  ``q_temperature`` (coef, every) with
-    ``positions`` (int32 [n]): q at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  Returns q as [n, nq * dp] with every head padded with zeros to ``dp``; keys go to
+    ``positions`` (int32 [n]): q at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).  ``v_first`` (a
+    [n, nkv * dv] view of qkv's type with unit column stride): v becomes (1 - v_mix) v + v_mix v_first before it is stored
+    (not beside a norm over the whole projection).  Returns q as [n, nq * dp] with every head padded with zeros to ``dp``; keys go to
     [pages, nkv, page_size, dp], values to [pages, nkv, dp, page_size] (their pad is never written)."""
     _dev(qkv, bias, q_weight, k_weight, cos_sin, slot_mapping, k_pages, v_pages)
     n, ld = qkv.shape
@@ -467,13 +484,18 @@ def attn_prepare_wide(qkv, bias, q_weight, k_weight, eps: float, cos_sin, rot_di
     if k_pages is not None:
         _i32(slot_mapping, "slot_mapping", n)
         _check_pages(k_pages, v_pages, qkv.dtype, nkv, page_size, dp)
+    if v_first is not None:
+        _need(v_first.is_cuda and v_first.dtype == qkv.dtype and v_first.shape == (n, nkv * dv) and (n == 0 or v_first.stride(1) == 1),
+              "v_first must be a [n, nkv * dv] view of qkv's type with unit column stride")
+        _need(q_weight is None or norm_per_head, "values are blended beside a per-head norm or none")
     q = torch.empty((n, nq * dp), dtype=qkv.dtype, device=qkv.device)
     fn = getattr(library.core(), f"jv_attn_prepare_wide_{_suffix(qkv.dtype)}")
     _check(fn(_ptr(q), _ptr(qkv), c_longlong(ld), _ptr(bias), _ptr(q_weight), _ptr(k_weight), c_float(eps),
               _ptr(cos_sin if rot_dims else None), c_int(rot_dims), _ptr(slot_mapping if k_pages is not None else None),
               _ptr(k_pages), _ptr(v_pages), c_int(page_size), c_int(n), c_int(nq), c_int(nkv), c_int(dk), c_int(dv),
               c_int(dp), c_float(v_scale), c_int(1 if norm_per_head else 0), c_longlong(v_off),
-              _ptr(positions if q_temperature is not None else None), c_float(coef), c_int(every), _stream()), "attn_prepare_wide")
+              _ptr(positions if q_temperature is not None else None), c_float(coef), c_int(every), _ptr(v_first),
+              c_longlong(0 if v_first is None else v_first.stride(0)), c_float(v_mix), _stream()), "attn_prepare_wide")
     return q
 
 
@@ -605,9 +627,10 @@ def key_window(window: "int | None", chunk: "int | None") -> int:
 
 
 def paged_attention_generic(out, q, q_row_stride, k_pages, v_pages, block_tables, token_req, positions,
-                            nq, nkv, head_dim, scale, window=0, sinks=None) -> None:
+                            nq, nkv, head_dim, scale, window=0, sinks=None, cap: float = 0.0, keep: int = 0) -> None:
     """Causal attention of every token over its request's pages (generic float-math kernel).  ``window``: 0 all earlier
-    keys, > 0 the last so many, < 0 those of the query's own block of -window positions (``key_window``).
+    keys, > 0 the last so many, < 0 those of the query's own block of -window positions (``key_window``).  ``cap`` > 0: a
+    scaled score s becomes cap * tanh(s / cap).  ``keep``: the first so many keys are seen whatever the window.
 
     ``q`` is any tensor whose row t holds the q heads at [t * q_row_stride + h * D].  ``sinks`` (float32 [nq]):
     exp(sinks[h]) joins every row's softmax denominator (a term without key and value, not scaled)."""
@@ -629,7 +652,8 @@ def paged_attention_generic(out, q, q_row_stride, k_pages, v_pages, block_tables
     _check(
         fn(_ptr(out), _ptr(q), c_longlong(q_row_stride), _ptr(k_pages), _ptr(v_pages), _ptr(block_tables),
            c_int(block_tables.shape[1]), _ptr(token_req), _ptr(positions), c_int(page_size), c_int(n),
-           c_int(nq), c_int(nkv), c_int(head_dim), c_float(scale), c_int(window or 0), _ptr(sinks), _stream()),
+           c_int(nq), c_int(nkv), c_int(head_dim), c_float(scale), c_int(window or 0), _ptr(sinks), c_float(cap),
+           c_int(keep if window else 0), _stream()),
         "paged_attention_generic",
     )
 
@@ -661,7 +685,7 @@ PARTIAL_BLOCKS = 1024               # a streaming product wants about this many 
 PARTIAL_SHAPE = (-1, 4, 4)          # x resident in LDS, phases of 512 columns: for inner sizes the staying blocks do not cover
 
 
-def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate_pairs: "str | None" = None,
+def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate_pairs: "str | tuple | None" = None,
                 block_shape=(0, 0, 0), out=None, ksplit: int = 1, row_scale: "UnscaledRows | None" = None) -> torch.Tensor:
     """x @ w.T for at most 64 rows of bfloat16 x against bfloat16 w [N, K]: the weight-streaming
     product of decode steps.  With ``gate_pairs`` (one of ``GATE_ACTIVATIONS``) the rows of w alternate gate
@@ -699,7 +723,7 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate
     _need(out.shape == shape and out.dtype == out_dtype and out.is_contiguous(),
           "out must be [M, N] (or [M, N/2], or [ksplit, M, N]) of the output type")
     common = (_ptr(out), _ptr(x), _ptr(w), c_int(m), c_int(n), c_int(k), c_longlong(x.stride(0)), c_longlong(n_out),
-              c_int(1 if out_dtype == torch.float32 else 0), c_int(_gate_act_id(gate_pairs) if gate_pairs else 0),
+              c_int(1 if out_dtype == torch.float32 else 0), *(_gate_act(gate_pairs) if gate_pairs else _NO_ACT),
               c_int(block_shape[0]), c_int(block_shape[1]), c_int(block_shape[2]), c_int(ksplit))
     if row_scale is not None:
         _need(block_shape[0] == -2, "only the blocks that stay scale their output rows")
@@ -714,7 +738,7 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate
     return out
 
 
-def gemm_tile64(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate_pairs: "str | None" = None,
+def gemm_tile64(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate_pairs: "str | tuple | None" = None,
                 ksplit: int = 1, out=None) -> torch.Tensor:
     """x @ w.T for at most 64 rows of bfloat16 x against bfloat16 w [N, K] with blocks that take 64
     rows of w against all rows of x: the weight-streaming product of decode steps with 17..64
@@ -745,7 +769,7 @@ def gemm_tile64(x: torch.Tensor, w: torch.Tensor, out_dtype=torch.bfloat16, gate
     _check(
         library.core().jv_gemm_tile64_bf16(
             _ptr(out), _ptr(x), _ptr(w), c_int(m), c_int(n), c_int(k), c_longlong(x.stride(0)), c_longlong(n_out),
-            c_int(1 if out_dtype == torch.float32 else 0), c_int(_gate_act_id(gate_pairs) if gate_pairs else 0), c_int(ksplit), _stream()),
+            c_int(1 if out_dtype == torch.float32 else 0), *(_gate_act(gate_pairs) if gate_pairs else _NO_ACT), c_int(ksplit), _stream()),
         "gemm_tile64",
     )
     return out
@@ -862,7 +886,7 @@ def streaming_plan(m: int, n: int, k: int, gate_pairs: bool = False, partial_ok:
     return (0, 0, 0), 1
 
 
-def linear(x: torch.Tensor, w: torch.Tensor, out_dtype=None, partial_ok: bool = False, gate_pairs: "str | None" = None,
+def linear(x: torch.Tensor, w: torch.Tensor, out_dtype=None, partial_ok: bool = False, gate_pairs: "str | tuple | None" = None,
            partial_max_width: int | None = PARTIAL_SUM_MAX_WIDTH):
     """x @ w.T for w stored [out, in].
 
@@ -1007,12 +1031,13 @@ def _sinks_ok(sinks, nq: int) -> None:
 
 
 def attn_prefill_mfma(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_seqlens, context_lens, work, n_work,
-                      nq, nkv, head_dim, scale, window=0, sinks=None) -> None:
+                      nq, nkv, head_dim, scale, window=0, sinks=None, cap: float = 0.0, keep: int = 0) -> None:
     """Causal attention of prompt portions.  ``work`` is int32 [n_work, 3]: (request index, first row
     of a group, first row of a second group of the same request or -1), see ``attn_prefill_geometry``;
     every row of every request must be in exactly one group.  ``window``: see ``key_window``.  Pairing a group that sees many keys with
     one that sees few gives all blocks the same amount of work.  ``sinks`` (float32 [nq]): exp(sinks[h]) joins every
-    row's softmax denominator (a term without key and value, not scaled)."""
+    row's softmax denominator (a term without key and value, not scaled).  ``cap``, ``keep``: as for
+    ``paged_attention_generic``."""
     _sinks_ok(sinks, nq)
     page_size = _attn_common(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_seqlens, context_lens, work,
                              nq, nkv, head_dim)
@@ -1022,7 +1047,7 @@ def attn_prefill_mfma(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_s
         lib.jv_attn_prefill(_ptr(out), _ptr(q), c_longlong(q_row_stride), _ptr(k_pages), _ptr(v_pages),
                             _ptr(block_tables), c_int(block_tables.shape[1]), _ptr(cu_seqlens), _ptr(context_lens),
                             _ptr(work), c_int(n_work), c_int(page_size), c_int(nq), c_int(nkv), c_float(scale),
-                            c_int(window or 0), _ptr(sinks), _stream()),
+                            c_int(window or 0), _ptr(sinks), c_float(cap), c_int(keep if window else 0), _stream()),
         "attn_prefill_mfma",
     )
 
@@ -1031,14 +1056,16 @@ ATTN_DECODE_TABLE_ENTRIES = 4096    # page-table entries a block of the decode k
 ATTN_DECODE_TILE_KEYS = 32          # keys of one tile of the decode kernel
 
 
-def attn_decode_min_splits(table_width: int, page_size: int) -> int:
+def attn_decode_min_splits(table_width: int, page_size: int, keep: int = 0) -> int:
     """The fewest splits with which the decode kernel takes block tables of this width: a row of up to
     4,096 entries is kept in LDS whole; of a wider one a block keeps the entries of its own split's
-    keys, which must fit."""
+    keys, which must fit beside those of the ``keep`` first keys that are seen whatever the window."""
     if table_width <= ATTN_DECODE_TABLE_ENTRIES:
         return 1
     tiles = -(-table_width * page_size // ATTN_DECODE_TILE_KEYS)
-    tiles_per_split = (ATTN_DECODE_TABLE_ENTRIES - 2) * page_size // ATTN_DECODE_TILE_KEYS
+    kept = -(-keep // ATTN_DECODE_TILE_KEYS) * ATTN_DECODE_TILE_KEYS // page_size + 1 if keep else 0
+    _need(kept <= ATTN_DECODE_TABLE_ENTRIES // 2, "so many kept keys do not fit beside a split's own at this table width")
+    tiles_per_split = (ATTN_DECODE_TABLE_ENTRIES - 2 - kept) * page_size // ATTN_DECODE_TILE_KEYS
     return -(-tiles // tiles_per_split)
 
 
@@ -1047,13 +1074,15 @@ def attn_decode_scratch_floats(n_work: int, nq: int, num_splits: int, head_dim: 
 
 
 def attn_decode_mfma(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_seqlens, context_lens, work, n_work,
-                     nq, nkv, head_dim, scale, window=0, num_splits=1, scratch=None, sinks=None) -> None:
+                     nq, nkv, head_dim, scale, window=0, num_splits=1, scratch=None, sinks=None, cap: float = 0.0,
+                     keep: int = 0) -> None:
     """Attention of single decoded tokens.  ``work`` is int32 [n_work]: indices of the requests
     (each with exactly one token in this step); None: the step holds decoded tokens only, request
     r = 0 .. n_work-1 has its token in row r (the kernel then has nothing to look up before its
     loads start).  With ``num_splits`` > 1 a request's keys are shared out to that many blocks and
     ``scratch`` (float32, ``attn_decode_scratch_floats`` entries) holds their partial results.  ``sinks``: as for
-    ``attn_prefill_mfma`` (counted once, after the splits are merged)."""
+    ``attn_prefill_mfma`` (counted once, after the splits are merged).  ``cap``, ``keep``: as for ``paged_attention_generic``."""
+    keep = keep if window else 0
     _sinks_ok(sinks, nq)
     page_size = _attn_common(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_seqlens, context_lens, work,
                              nq, nkv, head_dim)
@@ -1061,9 +1090,8 @@ def attn_decode_mfma(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_se
         _need(n_work == context_lens.numel() == out.shape[0], "without a work list every request has one token")
     else:
         _need(work.numel() >= n_work, "work list shorter than n_work")
-    _need(num_splits >= attn_decode_min_splits(block_tables.shape[1], page_size),
-          f"block tables of {block_tables.shape[1]} pages need at least "
-          f"{attn_decode_min_splits(block_tables.shape[1], page_size)} splits")
+    least = attn_decode_min_splits(block_tables.shape[1], page_size, keep)
+    _need(num_splits >= least, f"block tables of {block_tables.shape[1]} pages need at least {least} splits")
     if num_splits > 1:
         _need(scratch is not None and scratch.is_cuda and scratch.dtype == torch.float32
               and scratch.numel() >= attn_decode_scratch_floats(n_work, nq, num_splits, head_dim),
@@ -1075,7 +1103,7 @@ def attn_decode_mfma(out, q, q_row_stride, k_pages, v_pages, block_tables, cu_se
                            _ptr(cu_seqlens if work is not None else None), _ptr(context_lens),
                            _ptr(work), c_int(n_work), c_int(page_size), c_int(nq), c_int(nkv), c_float(scale),
                            c_int(window or 0), c_int(num_splits), _ptr(scratch if num_splits > 1 else None),
-                           _ptr(sinks), _stream()),
+                           _ptr(sinks), c_float(cap), c_int(keep), _stream()),
         "attn_decode_mfma",
     )
 
@@ -1199,6 +1227,59 @@ def postnorm_add_rmsnorm(h, y, parts, post_weight, eps: float, weight=None, out=
               c_longlong(0 if parts is None else parts.stride(0)), _ptr(bias), _ptr(post_weight), _ptr(weight), _ptr(out),
               _ptr(rows), c_int(n_out), c_int(hidden), c_float(eps), c_float(eps if out_eps is None else out_eps), c_float(plain_scale), _stream()),
            "postnorm_add_rmsnorm")
+
+
+class PendingPair:
+    """Two outputs that join the residual stream together, each under an RMS norm of its own: h += norm(a; weight_a) +
+    norm(b; weight_b).  ``a`` and ``b`` are what two sublayers returned (rows, a float stack of partial results, or a pair
+    of both); constant factors of the shares are folded into the weights."""
+
+    def __init__(self, a, b, weight_a: torch.Tensor, weight_b: torch.Tensor, eps: float):
+        self.shares = (PendingNorm(*split_sublayer_output(a), weight_a, eps), PendingNorm(*split_sublayer_output(b), weight_b, eps))
+
+
+def add_layernorm(h, delta, weight, bias, eps: float, out, rows=None) -> None:
+    """The residual step and a layer norm in one pass: h += what ``delta`` owes the float stream (None; rows of out's type;
+    a float stack of partial results; a pair of both; a ``PendingNorm``; a ``PendingPair``), then out = (h - mean(h)) /
+    sqrt(mean((h - mean(h))^2) + eps) * weight + bias.  With ``rows`` (int32 indices) only those rows are computed and h is
+    left alone."""
+    if delta is None:
+        shares = ()
+    elif isinstance(delta, PendingPair):
+        shares = delta.shares
+    elif isinstance(delta, PendingNorm):
+        shares = (delta,)
+    else:
+        shares = (PendingNorm(*split_sublayer_output(delta), None, 0.0),)
+    _dev(h, weight, bias, out, rows)
+    _f32(h, "h")
+    hidden = h.shape[1]
+    _f32(weight, "weight", hidden)
+    _f32(bias, "bias", hidden)
+    _need(hidden <= 16384, "rows wider than 16,384 are not supported")
+    n_out = out.shape[0]
+    _need(out.shape == (h.shape[0] if rows is None else rows.numel(), hidden), "out must have one row per row asked for")
+    if rows is not None:
+        _i32(rows, "rows", n_out)
+    vec = hidden % 4 == 0 and all(t.data_ptr() % 16 == 0 for t in (h, weight, bias, out))
+    args = []
+    for s in shares:
+        _dev(s.y, s.parts, s.weight)
+        _need(s.bias is None and (s.y is not None or s.parts is not None), "an output without a bias that is still owed, and not an empty one")
+        _need(s.y is None or (s.y.shape == h.shape and s.y.dtype == out.dtype), "rows must match h's shape and out's type")
+        _need(s.parts is None or (s.parts.dtype == torch.float32 and s.parts.dim() == 3 and s.parts.shape[1:] == h.shape),
+              "parts must be float32 [P, *h.shape]")
+        if s.weight is not None:
+            _f32(s.weight, "weight of an output's norm", hidden)
+        stride = 0 if s.parts is None else s.parts.stride(0)
+        vec = vec and stride % 4 == 0 and all(t is None or t.data_ptr() % 16 == 0 for t in (s.y, s.parts, s.weight))
+        args += [_ptr(s.y), _ptr(s.parts), c_int(0 if s.parts is None else s.parts.shape[0]), c_longlong(stride),
+                 _ptr(s.weight), c_float(s.eps), c_float(s.scale)]
+    for _ in range(2 - len(shares)):
+        args += [_ptr(None), _ptr(None), c_int(0), c_longlong(0), _ptr(None), c_float(0.0), c_float(0.0)]
+    fn = getattr(library.core(), f"jv_add_layernorm_{_suffix(out.dtype)}")
+    _check(fn(_ptr(h), c_int(len(shares)), *args, _ptr(weight), _ptr(bias), _ptr(out), _ptr(rows), c_int(n_out), c_int(hidden),
+              c_float(eps), c_int(1 if vec else 0), _stream()), "add_layernorm")
 
 
 def gated_rmsnorm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
@@ -1583,20 +1664,25 @@ def wkv_chunk_plan(ctx, dim: int):
 
 
 def wkv_steps(r, k, v, rate, w0, bonus, state, slot_ids, cu_seqlens, heads: int, dim: int, vdim: int,
-              chunk_plan=None) -> torch.Tensor:
+              chunk_plan=None, after: bool = False, r_scale: float = 1.0) -> torch.Tensor:
     """The recurrence with a decay per key channel and a bonus for the current token, per head with S the request's
     float state [dim, vdim]:  w = exp(-exp(rate + w0));  o = S^T r + (sum_d r[d] bonus[d] k[d]) v;  S <- diag(w) S + k v^T.
     r, k, rate [n, heads * dim] and v [n, heads * vdim] are views (unit column stride) of the activation type; w0 and
     bonus float32 [heads * dim]; ``state`` float32 [slots + 1, heads, dim, vdim].  Returns float32 [n, heads * vdim].
     With ``chunk_plan`` (``wkv_chunk_plan``) the chunks of every request run side by side and only the states between
-    them are walked in order; the results differ from the token-by-token kernel's by rounding."""
+    them are walked in order; the results differ from the token-by-token kernel's by rounding.
+    ``after``: the form of gated linear attention, S <- diag(e^rate) S + k v^T;  o = S^T (r_scale r), where ``rate`` holds the
+    logarithms of the decays as float32 and w0 and bonus are None."""
     _dev(w0, bonus, state, slot_ids, cu_seqlens)
     n = r.shape[0]
     for name, t, width in (("r", r, heads * dim), ("k", k, heads * dim), ("rate", rate, heads * dim), ("v", v, heads * vdim)):
-        _need(t.is_cuda and t.dtype == r.dtype and t.shape == (n, width) and (n == 0 or t.stride(1) == 1),
-              f"{name} must be a [n, {width}] view with unit column stride of one type")
-    _f32(w0, "w0", heads * dim)
-    _f32(bonus, "bonus", heads * dim)
+        kind = torch.float32 if after and name == "rate" else r.dtype
+        _need(t.is_cuda and t.dtype == kind and t.shape == (n, width) and (n == 0 or t.stride(1) == 1),
+              f"{name} must be a [n, {width}] view with unit column stride of {kind}")
+    _need(after or r_scale == 1.0, "a constant on r belongs to the form that reads after the update")
+    if not after:
+        _f32(w0, "w0", heads * dim)
+        _f32(bonus, "bonus", heads * dim)
     _f32(state, "state")
     _need(state.dim() == 4 and tuple(state.shape[1:]) == (heads, dim, vdim), "the state must be [slots + 1, heads, dim, vdim]")
     _i32(slot_ids, "slot_ids")
@@ -1614,14 +1700,35 @@ def wkv_steps(r, k, v, rate, w0, bonus, state, slot_ids, cu_seqlens, heads: int,
         dtot = floats[scratch.numel() + rq.numel():]
         fn = getattr(library.core(), f"jv_wkv_chunks_{_suffix(r.dtype)}")
         _check(fn(_ptr(out), _ptr(r), c_longlong(r.stride(0)), _ptr(k), c_longlong(k.stride(0)), _ptr(v), c_longlong(v.stride(0)),
-                  _ptr(rate), c_longlong(rate.stride(0)), _ptr(w0), _ptr(bonus), _ptr(state), _ptr(slot_ids), _ptr(cu_seqlens),
+                  _ptr(rate), c_longlong(rate.stride(0)), _ptr(w0), _ptr(bonus), c_int(1 if after else 0), c_float(r_scale), _ptr(state), _ptr(slot_ids), _ptr(cu_seqlens),
                   c_int(slot_ids.numel()), c_int(heads), c_int(dim), c_int(vdim), c_int(chunks), _ptr(work), _ptr(req_chunks),
                   _ptr(scratch), _ptr(rq), _ptr(dtot), _stream()), "wkv_chunks")
         return out
     fn = getattr(library.core(), f"jv_wkv_steps_{_suffix(r.dtype)}")
     _check(fn(_ptr(out), _ptr(r), c_longlong(r.stride(0)), _ptr(k), c_longlong(k.stride(0)), _ptr(v), c_longlong(v.stride(0)),
-              _ptr(rate), c_longlong(rate.stride(0)), _ptr(w0), _ptr(bonus), _ptr(state), _ptr(slot_ids), _ptr(cu_seqlens),
+              _ptr(rate), c_longlong(rate.stride(0)), _ptr(w0), _ptr(bonus), c_int(1 if after else 0), c_float(r_scale), _ptr(state), _ptr(slot_ids), _ptr(cu_seqlens),
               c_int(slot_ids.numel()), c_int(heads), c_int(dim), c_int(vdim), _stream()), "wkv_steps")
+    return out
+
+
+LOW_RANK_DECAY_MAX_RANK = 2048
+
+
+def low_rank_decay(low: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
+    """Float32 [n, channels]: log(sigmoid(z)) / tau with z = w low + bias, the logarithms of decays sigmoid(z)^(1/tau) from a
+    projection of small rank.  ``low`` a [n, rank] view (unit column stride) and ``w`` [channels, rank] of one activation
+    type, ``bias`` float32 [channels]; sums and logarithm are float (z is never rounded to the activation type)."""
+    _dev(w, bias)
+    n, rank = low.shape
+    channels = w.shape[0]
+    _need(low.is_cuda and low.dtype == w.dtype and w.shape[1] == rank and (n == 0 or low.stride(1) == 1),
+          "low must be a [n, rank] view with unit column stride of w's type")
+    _need(0 < rank <= LOW_RANK_DECAY_MAX_RANK and tau > 0, "a rank of at most 2,048 and a positive tau")
+    _f32(bias, "bias", channels)
+    out = torch.empty((n, channels), dtype=torch.float32, device=low.device)
+    fn = getattr(library.core(), f"jv_low_rank_decay_{_suffix(w.dtype)}")
+    _check(fn(_ptr(out), _ptr(low), c_longlong(low.stride(0) if n else 0), _ptr(w), _ptr(bias), c_longlong(n), c_int(channels),
+              c_int(rank), c_float(tau), _stream()), "low_rank_decay")
     return out
 
 
@@ -1764,7 +1871,9 @@ class MoePlan:
         self.tile_rows = tile_rows
 
 
-ROUTER_SCORES = {"sigmoid": 0, "softmax_chosen": 1, "sigmoid_normed": 2, "softmax": 3}      # the kernels' ids of how a chosen logit becomes a weight
+ROUTER_SCORES = {"sigmoid": 0, "softmax_chosen": 1, "sigmoid_normed": 2, "softmax": 3,
+                 "sigmoid_corrected": 4}      # the kernels' ids of how a chosen logit becomes a weight
+CORRECTED_SCORES = ("sigmoid_normed", "sigmoid_corrected")     # chosen by sigmoid(logit) + correction, a constant on the weights
 ROUTER_MAX_GROUPS = 64
 
 
@@ -1776,7 +1885,8 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     to the logits before the choice; ``score``: a chosen expert's weight is "sigmoid" of its logit, or
     "softmax_chosen": the softmax over the token's chosen logits alone, or "sigmoid_normed": the experts with the
     largest sigmoid(logit) + ``correction`` (float32 [experts] or None) are chosen, and a chosen expert's weight is its
-    sigmoid(logit) (without the correction) over the sum of the chosen ones' (+ 1e-20), times ``weight_scale``;
+    sigmoid(logit) (without the correction) over the sum of the chosen ones' (+ 1e-20), times ``weight_scale``
+    ("sigmoid_corrected": sigmoid(logit) times ``weight_scale``, not over the sum);
     or "softmax": the softmax over ALL of the token's logits.  ``groups`` (count, keep): the experts form ``count`` equal
     groups of neighbours, and only those of the ``keep`` groups with the largest logits can be chosen.
     ``always`` (few tokens: ``moe_always_possible``): every token also gets the ``always`` experts behind the routed ones
@@ -1817,8 +1927,8 @@ def moe_route(logits: "torch.Tensor | None", top: int, x=None, w_router=None, lo
     if bias is not None:
         _dev(bias)
         _f32(bias, "bias", experts)
-    _need(score == "sigmoid_normed" or (correction is None and weight_scale == 1.0),
-          "a correction of the choice and a constant on the weights belong to the score 'sigmoid_normed'")
+    _need(score in CORRECTED_SCORES or (correction is None and weight_scale == 1.0),
+          f"a correction of the choice and a constant on the weights belong to the scores {CORRECTED_SCORES}")
     if correction is not None:
         _dev(correction)
         _f32(correction, "correction", experts)
@@ -1892,10 +2002,10 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
     _need((w_gate is None or w_gate.shape == w_up.shape) and w_up.shape == (experts, ff, hidden) and w_down.shape == (experts, hidden, ff),
           "expert weights must be [experts, ff, hidden] and [experts, hidden, ff]")
     if w_gate is not None:
-        act = _gate_act_id(activation)
+        act = _gate_act(activation)
     else:
         _need(activation in PLAIN_ACTIVATIONS and activation is not None, f"no kernel for the activation {activation!r}")
-        act = PLAIN_ACTIVATIONS[activation]
+        act = (c_int(PLAIN_ACTIVATIONS[activation]), c_float(0.0), c_float(0.0))
     _need(w_gate is None or w_gate.dtype == x.dtype, "x and the weights must have one type")
     _need(x.dtype == w_up.dtype == w_down.dtype, "x and the weights must have one type")
     _need(out.dtype == torch.float32 and tuple(out.shape) == (plan.top, n, hidden), "out must be float32 [top, n, hidden]")
@@ -1913,7 +2023,7 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
         _check(lib.jv_moe_gate_up_skinny_bf16(
             _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),
             _ptr(p.tile_row0), _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(hidden), c_int(ff),
-            c_int(act), c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
+            *act, c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
         _check(lib.jv_moe_down_skinny_bf16(
             _ptr(out), _ptr(z), _ptr(w_down), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert), _ptr(p.tile_row0),
             _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(n), c_int(hidden), c_int(ff),
@@ -1923,7 +2033,7 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
         _check(lib.jv_moe_gate_up_mfma_bf16(
             _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),
             _ptr(p.tile_row0), _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(hidden), c_int(ff),
-            c_int(act), c_int(1 if weight_on_input else 0), c_int(p.tile_rows), _stream()), "moe_gate_up")
+            *act, c_int(1 if weight_on_input else 0), c_int(p.tile_rows), _stream()), "moe_gate_up")
         _check(lib.jv_moe_down_mfma_bf16(
             _ptr(out), _ptr(z), _ptr(w_down), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert), _ptr(p.tile_row0),
             _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(n), c_int(hidden), c_int(ff),
@@ -1932,7 +2042,7 @@ def moe_experts(x, plan: MoePlan, w_gate, w_up, w_down, activation: str, out: to
     _check(getattr(lib, f"jv_moe_gate_up_{suf}")(
         _ptr(z), _ptr(x), _ptr(w_gate), _ptr(w_up), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert),
         _ptr(p.tile_row0), _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(hidden), c_int(ff),
-        c_int(act), c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
+        *act, c_int(1 if weight_on_input else 0), _stream()), "moe_gate_up")
     _check(getattr(lib, f"jv_moe_down_{suf}")(
         _ptr(out), _ptr(z), _ptr(w_down), _ptr(p.meta), _ptr(p.offsets), _ptr(p.tile_expert), _ptr(p.tile_row0),
         _ptr(p.order), _ptr(p.weights), c_int(p.max_tiles), c_int(p.top), c_int(n), c_int(hidden), c_int(ff),

@@ -20,6 +20,9 @@ from .spec import (LayerMemory, PagedCacheSpec, PartSpec, StateSpec, StepContext
                    kv_cache_spec, register_part)
 
 
+FIRST_VALUES = "first_values"      # in ``StepContext.extras``: the step's values of the first layer that blends them
+
+
 class GroupedQueryAttention:
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int,
                  qk_norm_eps: Optional[float] = None, position: Optional[PartSpec] = None,
@@ -27,7 +30,8 @@ class GroupedQueryAttention:
                  o_bias: bool = False, v_head_dim: Optional[int] = None, qk_norm: str = "head", v_scale: float = 1.0,
                  output_gate: bool = False, values_are_keys: bool = False, q_temperature: Optional[tuple] = None,
                  chunk: Optional[int] = None, filter_taps: Optional[int] = None, value_position: Optional[PartSpec] = None,
-                 softmax_plus_one: bool = False):
+                 softmax_plus_one: bool = False, softcap: Optional[float] = None, keep_first: int = 0, sinks: bool = False,
+                 qk_norm_weight: bool = True, value_blend: Optional[str] = None):
         """``v_head_dim``: a value size that differs from the key size; ``qk_norm`` "whole": the q/k norm spans all
         of q's (and all of k's) columns at once, with weights of that size, instead of every head on its own;
         ``v_scale``: a constant on the values (and so on the mixer's result before its output projection);
@@ -41,8 +45,15 @@ class GroupedQueryAttention:
         y_t = sum_j w[:, j] u_(t - taps + 1 + j) (the last taps - 1 projected rows are the request's state ``filter``);
         ``value_position``: a rotation of the whole value heads by their token's position, cached so, and every head's
         result turned back by the query's position (before the gate): the weighted sum sees the values at their
-        distance from the query; ``softmax_plus_one``: one is added to the softmax denominator (a sink of score 0).
-        Any of these but ``chunk`` and ``softmax_plus_one`` takes the ``wide`` path: heads cached
+        distance from the query; ``softmax_plus_one``: one is added to the softmax denominator (a sink of score 0);
+        ``softcap`` c: a scaled score s becomes c tanh(s / c); ``keep_first``: beside a window the first so many keys of the
+        sequence stay in sight; ``sinks``: a learned number per q head whose exponential joins the softmax denominator (no
+        key, no value, neither scaled nor capped); ``qk_norm_weight`` False: the per-head q/k norm has no weight (it is then
+        the same before and behind the rotation, which keeps a head's length); ``value_blend`` "first": the layer's values
+        are kept for the step; "later": the values become (1 - l) v + l v_first with v_first those of the same token and l a
+        learned number, before they are cached.
+        Any of these but ``chunk``, ``softmax_plus_one``, ``softcap``, ``keep_first`` and ``sinks`` takes the ``wide`` path (so does
+        ``qkv_bias`` beside one of the last three): heads cached
         under one padded size (``K.padded_head_dim``), prepared by ``K.attn_prepare_wide``, read by the same paged
         attention kernels."""
         if num_heads % num_kv_heads:
@@ -65,6 +76,19 @@ class GroupedQueryAttention:
             raise ValueError("a window or blocks, not both")
         self.taps = int(filter_taps) if filter_taps else 0
         self.plus_one = bool(softmax_plus_one)
+        self.softcap = float(softcap) if softcap else None
+        self.keep_first = int(keep_first or 0)
+        if self.keep_first and not window:
+            raise ValueError("kept first keys belong to a window")
+        self.learned_sinks = bool(sinks)
+        if self.plus_one and self.learned_sinks:
+            raise ValueError("one is added to the denominator, or a learned sink, not both")
+        self.qk_norm_weight = bool(qk_norm_weight)
+        if not self.qk_norm_weight and qk_norm != "head":
+            raise ValueError("a q/k norm without a weight is per head")
+        if value_blend not in (None, "first", "later"):
+            raise ValueError(f"value_blend is 'first' or 'later', not {value_blend!r}")
+        self.value_blend = value_blend
         self.value_position = build_part("position", value_position) if value_position is not None else None
         self.filtered = bool(self.taps or self.value_position is not None)
         if self.filtered and (self.values_are_keys or self.q_temperature is not None or qk_norm_eps is not None or qkv_bias
@@ -76,7 +100,10 @@ class GroupedQueryAttention:
             if turn is None or turn != (self.dv, True):
                 raise ValueError("values turn whole, in pairs (2m, 2m + 1)")
         self.wide = (self.filtered or self.values_are_keys or self.q_temperature is not None or self.dv != self.dk or (qk_norm == "whole" and qk_norm_eps is not None) or self.v_scale != 1.0
-                     or self.output_gate)
+                     or self.output_gate or not self.qk_norm_weight or self.value_blend is not None
+                     or (bool(qkv_bias) and (self.softcap is not None or self.keep_first > 0 or self.learned_sinks)))
+        if self.value_blend is not None and (self.filtered or qkv_bias or values_are_keys or qk_norm == "whole"):
+            raise ValueError("blended values: without filters, biases, values taken from the keys or a norm over the whole projection")
         # what the paged attention kernels see
         self.d = K.padded_head_dim(self.dk, self.dv) if self.wide else self.dk
         if self.wide:
@@ -110,7 +137,7 @@ class GroupedQueryAttention:
         }
         if self.values_are_keys:
             del t["v_proj.weight"]
-        if self.qk_norm_eps is not None:
+        if self.qk_norm_eps is not None and self.qk_norm_weight:
             whole = self.qk_norm == "whole"
             t["q_norm.weight"] = TensorSpec((self.nq * self.dk if whole else self.dk,), role="vector", init="norm")
             t["k_norm.weight"] = TensorSpec((self.nkv * self.dk if whole else self.dk,), role="vector", init="norm")
@@ -122,6 +149,10 @@ class GroupedQueryAttention:
             t["o_proj.bias"] = TensorSpec((self.hidden_size,), role="vector")
         if self.output_gate:
             t["gate.weight"] = TensorSpec((self.nq * self.dv, self.hidden_size))
+        if self.learned_sinks:
+            t["sinks"] = TensorSpec((self.nq,), role="vector", init="small")
+        if self.value_blend is not None:      # stored in every blending layer, the first one's has no effect
+            t["value_blend"] = TensorSpec((), role="vector", init="fraction")
         if self.taps:
             t["q_filter.weight"] = TensorSpec((self.nq * self.dk, self.taps), role="vector")
             t["k_filter.weight"] = TensorSpec((self.nkv * self.dk, self.taps), role="vector")
@@ -129,7 +160,7 @@ class GroupedQueryAttention:
         return t
 
     def cache_spec(self) -> Optional[PagedCacheSpec]:
-        return kv_cache_spec(self.nkv, self.d, self.window, self.chunk)
+        return kv_cache_spec(self.nkv, self.d, self.window, self.chunk, self.keep_first)
 
     def state_spec(self):
         if not self.taps:
@@ -145,12 +176,15 @@ class GroupedQueryAttention:
         if self.output_gate:
             blocks.append(tensors["gate.weight"])
         rows = sum(b.shape[0] for b in blocks)
-        if self.filtered and rows % 8:      # rows of the product stay 16-byte aligned for the kernels that read heads out of them
+        if self.wide and rows % 8:      # rows of the product stay 16-byte aligned for the kernels that read heads out of them
             blocks.append(blocks[0].new_zeros((8 - rows % 8, self.hidden_size)))
         self.w_qkv = torch.cat(blocks, dim=0).contiguous()
         self.filters = (torch.cat([tensors[f"{s}_filter.weight"] for s in "qkv"], dim=0).t().contiguous()
                         if self.taps else None)       # [taps, channels]
         self.sinks = torch.zeros((self.nq,), dtype=torch.float32, device=self.w_qkv.device) if self.plus_one else None
+        if self.learned_sinks:
+            self.sinks = tensors["sinks"].contiguous()
+        self.blend = float(tensors["value_blend"].reshape(())) if self.value_blend is not None else 0.0
         self.qkv_width = self.nq * self.dk + self.nkv * (self.dk + (0 if self.values_are_keys else self.dv))
         self.w_o = tensors["o_proj.weight"]
         if self.wide and self.d != self.dv:
@@ -158,8 +192,10 @@ class GroupedQueryAttention:
             w = self.w_o.new_zeros((self.hidden_size, self.nq, self.d))
             w[:, :, :self.dv] = self.w_o.view(self.hidden_size, self.nq, self.dv)
             self.w_o = w.view(self.hidden_size, self.nq * self.d).contiguous()
-        if self.qk_norm_eps is not None:
+        if self.qk_norm_eps is not None and self.qk_norm_weight:
             self.q_norm, self.k_norm = tensors["q_norm.weight"], tensors["k_norm.weight"]
+        elif self.qk_norm_eps is not None:
+            self.q_norm = self.k_norm = torch.ones((self.dk,), dtype=torch.float32, device=self.w_qkv.device)
         if self.qkv_bias:
             self.b_qkv = torch.cat([tensors["q_proj.bias"], tensors["k_proj.bias"], tensors["v_proj.bias"]]).contiguous()
         if self.o_bias:
@@ -240,18 +276,29 @@ class GroupedQueryAttention:
         if interleaved:
             raise ValueError("heads of two sizes and a norm over the whole projection rotate half-split pairs only")
         writes = mem.writes
+        values = None
+        if self.value_blend is not None:
+            at = (self.nq + self.nkv) * self.dk
+            own = qkv[:, at:at + self.nkv * self.dv]
+            if self.value_blend == "first":
+                ctx.extras[FIRST_VALUES] = own
+            else:
+                values = ctx.extras.get(FIRST_VALUES)
+                if values is None:
+                    raise ValueError("values are blended with those of an earlier layer, and none kept them")
         q = K.attn_prepare_wide(
             qkv, self.b_qkv, self.q_norm, self.k_norm, self.qk_norm_eps or 0.0, cos_sin, rotary_dim,
             ctx.slot_mappings[mem.group] if writes else None, mem.pages["k"] if writes else None,
             mem.pages["v"] if writes else None, ctx.page_size, self.nq, self.nkv, self.dk, self.dv, self.d, self.v_scale,
             norm_per_head=self.qk_norm == "head", values_are_keys=self.values_are_keys,
-            positions=ctx.positions if self.q_temperature is not None else None, q_temperature=self.q_temperature)
+            positions=ctx.positions if self.q_temperature is not None else None, q_temperature=self.q_temperature,
+            v_first=values, v_mix=self.blend)
         out = torch.empty((qkv.shape[0], self.nq * self.d), dtype=qkv.dtype, device=qkv.device)
         from . import attention_backend
 
         attention_backend.run(self, out, q, ctx, mem)
         if self.output_gate:
-            K.sigmoid_gate_heads(out, qkv[:, self.qkv_width:], self.nq, self.dv, self.d)
+            K.sigmoid_gate_heads(out, qkv[:, self.qkv_width:self.qkv_width + self.nq * self.dv], self.nq, self.dv, self.d)
         y = K.linear(out, self.w_o, partial_ok=True)
         if self.b_o is not None:
             K.add_bias(y, self.b_o)

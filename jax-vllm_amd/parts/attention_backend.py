@@ -36,9 +36,10 @@ class MfmaPlan:
     scratch: Optional[torch.Tensor]
 
 
-def keys_seen(kv_len: int, window: int) -> int:
-    """The most keys a query sees that has ``kv_len`` keys up to itself (``K.key_window``'s number)."""
-    return min(kv_len, abs(window)) if window else kv_len
+def keys_seen(kv_len: int, window: int, keep: int = 0) -> int:
+    """The most keys a query sees that has ``kv_len`` keys up to itself (``K.key_window``'s number, and the first keys
+    that are kept whatever the window)."""
+    return min(kv_len, abs(window) + keep) if window else kv_len
 
 
 def decode_splits(n_decode: int, blocks_per_request: int, max_kv_len: int) -> int:
@@ -52,10 +53,10 @@ KEY_TILE = 64                # keys of one tile of the prefill kernel
 
 
 def prefill_work_items(q_lens, context_lens, g: int, window: int, group_rows: int, groups_per_item: int,
-                       balance: bool = True):
+                       balance: bool = True, keep: int = 0):
     """Work items (request, first row of group 0, first row of group 1 or -1) of the prefill kernel
     for the requests with more than one token, heaviest first.  Rows are (query, head-in-group)
-    pairs.  ``window``: see ``K.key_window``.  With ``balance`` and no window the i-th lightest group of a request is paired with its
+    pairs.  ``window``: see ``K.key_window``; ``keep``: first keys every query sees besides.  With ``balance`` and no window the i-th lightest group of a request is paired with its
     i-th heaviest: every pair then walks about the same number of (row tile, key tile) products,
     which matters when the items are so few that the heaviest one decides the time.  Otherwise
     neighbours are paired: they share nearly all their keys, so every fragment read feeds both."""
@@ -69,7 +70,7 @@ def prefill_work_items(q_lens, context_lens, g: int, window: int, group_rows: in
             end = cl + last_row // g + 1
             first = cl + m0 // g
             begin = max(0, first - window + 1) if window > 0 else first - first % -window if window else 0
-            groups.append((-(-end // KEY_TILE) - begin // KEY_TILE, m0))
+            groups.append((-(-end // KEY_TILE) - begin // KEY_TILE + min(begin // KEY_TILE, -(-keep // KEY_TILE)), m0))
         if groups_per_item < 2:
             items.extend((t, r, m0, -1) for t, m0 in groups)
         elif window or not balance:
@@ -120,23 +121,23 @@ def prefill_item_shape(rows: int, nkv: int, group_rows: int, kernel_groups: int,
     return kernel_groups, blocks <= RESIDENT_BLOCKS * compute_units
 
 
-def plan_mfma(ctx, nq: int, nkv: int, head_dim: int, window: int, device) -> MfmaPlan:
+def plan_mfma(ctx, nq: int, nkv: int, head_dim: int, window: int, device, keep: int = 0) -> MfmaPlan:
     g = nq // nkv
     group_rows, kernel_groups = K.attn_prefill_geometry(head_dim)
     rows = sum(ql * g for ql in ctx.q_lens_host if ql > 1)
     groups_per_item, balance = prefill_item_shape(rows, nkv, group_rows, kernel_groups, K.compute_units(device),
                                                   K.attn_prefill_waves_split(head_dim))
     prefill = prefill_work_items(ctx.q_lens_host, ctx.context_lens_host, g, window, group_rows, groups_per_item,
-                                 balance=balance)
+                                 balance=balance, keep=keep)
     cus = K.compute_units(device)
     if cus < len(prefill) * nkv <= RESIDENT_BLOCKS * cus:
         prefill = pair_up_resident_items(prefill, cus // nkv)
     decode = [r for r, ql in enumerate(ctx.q_lens_host) if ql == 1]
     max_kv_decode = max([ctx.context_lens_host[r] + 1 for r in decode], default=1)
-    splits = decode_splits(len(decode), nkv * (-(-g // 16)), keys_seen(max_kv_decode, window)) if decode else 1
+    splits = decode_splits(len(decode), nkv * (-(-g // 16)), keys_seen(max_kv_decode, window, keep)) if decode else 1
     if decode:      # a very wide block table is taken split by split
         widest = max(t.shape[1] for t in ctx.block_tables)
-        splits = max(splits, K.attn_decode_min_splits(widest, ctx.page_size))
+        splits = max(splits, K.attn_decode_min_splits(widest, ctx.page_size, keep))
     decode_only = len(decode) == len(ctx.q_lens_host)       # requests 0, 1, ...: the kernel needs no list
     flat = [x for item in prefill for x in item] + ([] if decode_only else decode)
     dev = torch.tensor(flat, dtype=torch.int32).pin_memory().to(device, non_blocking=True) if flat else None
@@ -154,22 +155,24 @@ def run(att, out, qkv, ctx, mem) -> None:
     q_row_stride = getattr(att, "q_row_stride", None) or (att.nq + 2 * att.nkv) * att.d
     window = K.key_window(att.window, getattr(att, "chunk", None))
     sinks = getattr(att, "sinks", None)      # float [nq] or None: one more term exp(sink) in every softmax denominator
+    cap = getattr(att, "softcap", None) or 0.0                       # scores under a soft cap
+    keep = (getattr(att, "keep_first", 0) or 0) if window else 0     # first keys seen whatever the window
     if not K.mfma_attention_supported(qkv.dtype, att.d, ctx.page_size):
         K.paged_attention_generic(
             out, qkv, q_row_stride, mem.pages["k"], mem.pages["v"], ctx.block_tables[mem.group], ctx.token_req,
-            ctx.positions, att.nq, att.nkv, att.d, att.scale, window, sinks=sinks,
+            ctx.positions, att.nq, att.nkv, att.d, att.scale, window, sinks=sinks, cap=cap, keep=keep,
         )
         return
-    key = ("mfma_attention_plan", att.nq, att.nkv, att.d, window)
+    key = ("mfma_attention_plan", att.nq, att.nkv, att.d, window, keep)
     plan = ctx.plans.get(key)
     if plan is None:
-        plan = ctx.plans[key] = plan_mfma(ctx, att.nq, att.nkv, att.d, window, qkv.device)
+        plan = ctx.plans[key] = plan_mfma(ctx, att.nq, att.nkv, att.d, window, qkv.device, keep)
     tables = ctx.block_tables[mem.group]
     if plan.n_prefill:
         K.attn_prefill_mfma(out, qkv, q_row_stride, mem.pages["k"], mem.pages["v"], tables, ctx.cu_seqlens,
                             ctx.context_lens, plan.prefill_work, plan.n_prefill, att.nq, att.nkv, att.d, att.scale,
-                            window, sinks=sinks)
+                            window, sinks=sinks, cap=cap, keep=keep)
     if plan.n_decode:
         K.attn_decode_mfma(out, qkv, q_row_stride, mem.pages["k"], mem.pages["v"], tables, ctx.cu_seqlens,
                            ctx.context_lens, plan.decode_work, plan.n_decode, att.nq, att.nkv, att.d, att.scale,
-                           window, plan.num_splits, plan.scratch, sinks=sinks)
+                           window, plan.num_splits, plan.scratch, sinks=sinks, cap=cap, keep=keep)

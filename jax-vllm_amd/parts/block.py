@@ -2,7 +2,7 @@
 
     h = h + mixer(norm_1(h));   h = h + feed_forward(norm_2(h))
 
-The residual stream ``h`` is float.  Each sublayer's output is not added at once:
+(the norm part is a parameter: an RMS norm or a layer norm).  The residual stream ``h`` is float.  Each sublayer's output is not added at once:
 it is handed on as ``delta`` and added inside the next norm's kernel (one pass over
 ``h`` instead of two), so a block takes and returns ``(h, delta)``.
 
@@ -47,6 +47,10 @@ class PreNormBlock:
 
     def _share(self, out):
         """What a sublayer returned, as the next norm takes it."""
+        if isinstance(out, K.PendingPair):                             # two outputs under norms of their own
+            if self.residual_scale != 1.0:
+                raise ValueError("a residual constant on a pair of normed outputs belongs into their norms' weights")
+            return out
         if self.residual_scale != 1.0 or isinstance(out, tuple):       # a pair (rows, float shares) is added there too
             return K.pending_scale(out, self.residual_scale)
         return out.settled() if isinstance(out, K.BiasedOutput) else out

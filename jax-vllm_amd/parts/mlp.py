@@ -1,6 +1,6 @@
 """Gated feed-forward.  Reference: ``jllm/model/common.py:69-76``:
 ``down( silu(gate(x)) * up(x) )``, no biases (SwiGLU); the gate's activation is a parameter, one
-of ``ops.kernels.GATE_ACTIVATIONS``.  gate and up are one matrix product against
+of ``ops.kernels.GATE_ACTIVATIONS`` (the clamped one with its constants, ``("clamped", limit, slope)``).  gate and up are one matrix product against
 one weight whose rows alternate gate row j, up row j, so that a gate value and its up value
 come out next to each other: for few rows the activation is that product's epilogue, for
 many rows a kernel over adjacent pairs.  The activation runs in float."""
@@ -16,7 +16,8 @@ class GatedMLP:
     replayable = True
 
     def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu"):
-        if activation not in K.GATE_ACTIVATIONS:
+        activation = tuple(activation) if isinstance(activation, list) else activation
+        if not K.gate_activation_known(activation):
             raise ValueError(f"GatedMLP has kernels for {sorted(K.GATE_ACTIVATIONS)}, not for {activation!r}")
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.activation = activation

@@ -4,7 +4,8 @@
     z = W_router x (+ b)  (float);   the ``top`` experts with the largest z are chosen;
     s = sigmoid(z), or (``score`` "softmax_chosen") the softmax over the chosen z alone, or (``score``
     "sigmoid_normed") the experts with the largest sigmoid(z) + correction are chosen and
-    s = sigmoid(z) / (sum of the chosen sigmoids + 1e-20) * ``weight_scale``, or (``score`` "softmax") the
+    s = sigmoid(z) / (sum of the chosen sigmoids + 1e-20) * ``weight_scale`` (``score`` "sigmoid_corrected": chosen
+    alike, s = sigmoid(z) * ``weight_scale``), or (``score`` "softmax") the
     softmax over ALL z, as it is; with ``groups`` (count, keep) the experts form equal groups of neighbours
     and only those of the ``keep`` groups with the largest z can be chosen
     out = sum over the chosen e of  expert_e(s_e * x)   [+ shared(x)  or  + sigmoid(w_sg . x) shared(x)]
@@ -39,8 +40,9 @@ class RoutedExperts:
                  expert_names=("gate", "up", "down"), router_bias: bool = False, score: str = "sigmoid",
                  choice_correction: bool = False, weight_scale: float = 1.0, shared_gate: bool = False,
                  gated: bool = True, groups: Optional[tuple] = None):
-        known = K.GATE_ACTIVATIONS if gated else {a: i for a, i in K.PLAIN_ACTIVATIONS.items() if a}
-        if activation not in known:
+        activation = tuple(activation) if isinstance(activation, list) else activation
+        if not (K.gate_activation_known(activation) if gated else activation in K.PLAIN_ACTIVATIONS and activation):
+            known = K.GATE_ACTIVATIONS if gated else [a for a in K.PLAIN_ACTIVATIONS if a]
             raise ValueError(f"the expert kernels have {sorted(known)}, not {activation!r}")
         self.gated = bool(gated)
         self.groups = (int(groups[0]), int(groups[1])) if groups else None
@@ -52,8 +54,8 @@ class RoutedExperts:
         self.activation, self.weight_on_input = activation, bool(weight_on_input)
         self.router_bias, self.score = bool(router_bias), score
         self.choice_correction, self.weight_scale = bool(choice_correction), float(weight_scale)
-        if (self.choice_correction or self.weight_scale != 1.0) and score != "sigmoid_normed":
-            raise ValueError("a correction of the choice and a constant on the weights belong to the score 'sigmoid_normed'")
+        if (self.choice_correction or self.weight_scale != 1.0) and score not in K.CORRECTED_SCORES:
+            raise ValueError(f"a correction of the choice and a constant on the weights belong to the scores {K.CORRECTED_SCORES}")
         if self.groups is not None:
             count, keep = self.groups
             if not (0 < keep <= count <= K.ROUTER_MAX_GROUPS) or self.experts % count or keep * (self.experts // count) < self.top:

@@ -1,4 +1,4 @@
-"""RMSNorm part.  Reference: ``jllm/model/common.py:44-48``.
+"""RMSNorm and layer norm parts.  Reference: ``jllm/model/common.py:44-48``.
 
 ``y = x * rsqrt(mean(x^2, last axis) + eps) * weight`` with the mean square, the
 inverse root and both products in float.  (The reference rounds the normalised value
@@ -63,4 +63,32 @@ class RMSNorm:
         return out
 
 
+class LayerNorm:
+    """``y = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * weight + bias`` over the last axis, all in float."""
+
+    replayable = True
+
+    def __init__(self, size: int, eps: float):
+        self.size, self.eps = int(size), float(eps)
+        self.weight = self.bias = None
+
+    def tensors(self) -> dict:
+        return {"weight": TensorSpec((self.size,), role="vector", init="norm"),
+                "bias": TensorSpec((self.size,), role="vector", init="small")}
+
+    def bind(self, tensors: dict, dtype: torch.dtype) -> None:
+        self.weight, self.bias = tensors["weight"], tensors["bias"]
+        self.dtype = dtype
+
+    def add_norm(self, h: torch.Tensor, delta, rows=None):
+        """The residual step fused with the norm: ``h += delta`` in the float residual stream, returns ``norm(h)`` in the
+        activation type.  ``delta`` is whatever a block hands on: rows, float partial results, a ``K.PendingNorm``, a
+        ``K.PendingPair`` or None.  With ``rows`` only those rows are normed and ``h`` is left alone."""
+        n_out = h.shape[0] if rows is None else rows.numel()
+        out = torch.empty((n_out, self.size), dtype=self.dtype, device=h.device)
+        K.add_layernorm(h, delta, self.weight, self.bias, self.eps, out, rows)
+        return out
+
+
 register_part("norm", "rmsnorm", RMSNorm)
+register_part("norm", "layernorm", LayerNorm)

@@ -15,7 +15,8 @@ and differ in what q, k, v, the decay g and the write strength w are made of:
                    weight shared by the heads, times silu(gate).
 
 A fourth mixer, ``time_mix`` (below), has a recurrence of its own, ``K.wkv_steps``: a decay per key channel instead of
-one per head, the output read from the state BEFORE the token's update, and a bonus on the token's own key.
+one per head, the output read from the state BEFORE the token's update, and a bonus on the token's own key.  A fifth,
+``gated_linear_attention``, runs the same kernels in the form that reads the state AFTER the update, without a bonus.
 
 Everything that enters the recurrence is float (the products and the convolutions' results are in the activation
 type).  The state, and the last taps - 1 inputs of every convolution, live in the request's state slot between steps.
@@ -180,8 +181,7 @@ class GatedDeltaMixer:
     def bind(self, tensors: dict, dtype: torch.dtype) -> None:
         self.dtype = dtype
         # one product for everything that reads the input: [q | k | v | gate | decay | beta]
-        self.w_in = torch.cat([tensors[k + ".weight"] for k in ("q_proj", "k_proj", "v_proj", "gate", "decay_proj", "beta_proj")],
-                              dim=0).contiguous()
+        self.w_in = _stacked([tensors[k + ".weight"] for k in ("q_proj", "k_proj", "v_proj", "gate", "decay_proj", "beta_proj")])
         self.conv_w = torch.cat([tensors[k + "_conv.weight"] for k in ("q", "k", "v")], dim=0).contiguous()
         self.dt_bias, self.a_log, self.norm_weight = tensors["dt_bias"], tensors["A_log"], tensors["norm.weight"]
         self.w_o = tensors["o_proj.weight"]
@@ -272,12 +272,100 @@ class TimeMix:
         return K.linear(y, self.w_o, partial_ok=True)
 
 
+class GatedLinearAttention:
+    """Linear attention with a data-dependent decay per key channel, read after the token's update:
+
+        q, k = W_q h / sqrt(dim), W_k h  [heads, dim];   v = W_v h  [heads, vdim]
+        log a = log(sigmoid(W_up (W_down h) + b)) / tau       per head and key channel, float
+        S <- diag(a_t) S + k_t v_t^T;   o_t = S^T q_t         per head, S [dim, vdim] float
+        out = W_o ( concat_h( o_t / rms(o_t) * norm ) * silu(W_g h) )      (norm [vdim], shared by the heads)
+
+    The state S lives in the request's state slot between steps."""
+
+    replayable = True     # slots, request borders and tokens come from the device; the kernel choice does not depend on values
+
+    def __init__(self, hidden_size: int, num_heads: int, head_dim: int, v_dim: int, tau: float, norm_eps: float,
+                 decay_rank: Optional[int] = None):
+        """``decay_rank`` None: the inner size of the decay's two products is whatever the checkpoint's tensors have."""
+        self.hidden_size, self.heads, self.dim, self.vdim = int(hidden_size), int(num_heads), int(head_dim), int(v_dim)
+        self.tau, self.eps = float(tau), float(norm_eps)
+        self.decay_rank = int(decay_rank) if decay_rank else None
+        if self.dim > K.WKV_MAX_DIM:
+            raise ValueError(f"the recurrence keeps heads of at most {K.WKV_MAX_DIM} channels, not {self.dim}")
+        if not self.tau > 0:
+            raise ValueError("tau must be positive")
+
+    def tensors(self) -> dict:
+        H, hid = self.heads, self.hidden_size
+        return {
+            "q_proj.weight": TensorSpec((H * self.dim, hid)),
+            "k_proj.weight": TensorSpec((H * self.dim, hid)),
+            "v_proj.weight": TensorSpec((H * self.vdim, hid)),
+            "gate.weight": TensorSpec((H * self.vdim, hid)),
+            "decay_down.weight": TensorSpec((self.decay_rank, hid)),
+            "decay_up.weight": TensorSpec((H * self.dim, self.decay_rank)),
+            "decay_up.bias": TensorSpec((H * self.dim,), role="vector", init="norm"),
+            "norm.weight": TensorSpec((self.vdim,), role="vector", init="norm"),
+            "o_proj.weight": TensorSpec((hid, H * self.vdim)),
+        }
+
+    def cache_spec(self):
+        return None
+
+    def state_spec(self):
+        return StateSpec((self.heads, self.dim, self.vdim), "float32", "S")
+
+    def bind(self, tensors: dict, dtype: torch.dtype) -> None:
+        self.dtype = dtype
+        # one product for everything that reads the input: [q | k | v | gate | the decay's inner size]
+        blocks = [tensors[k + ".weight"] for k in ("q_proj", "k_proj", "v_proj", "gate", "decay_down")]
+        self.rank = blocks[-1].shape[0]
+        if tensors["decay_up.weight"].shape[1] != self.rank:
+            raise ValueError(f"the decay's products disagree: {self.rank} and {tensors['decay_up.weight'].shape[1]}")
+        self.w_in = _stacked(blocks)
+        self.w_decay_up, self.b_decay = tensors["decay_up.weight"].contiguous(), tensors["decay_up.bias"].contiguous()
+        self.norm_weight, self.w_o = tensors["norm.weight"], tensors["o_proj.weight"]
+
+    def forward(self, x, ctx: StepContext, mem: LayerMemory):
+        H, d, dv = self.heads, self.dim, self.vdim
+        proj = K.linear(x, self.w_in)
+        v_at, gate_at = 2 * H * d, 2 * H * d + H * dv
+        low_at = gate_at + H * dv
+        log_decay = K.low_rank_decay(proj[:, low_at:low_at + self.rank], self.w_decay_up, self.b_decay, self.tau)
+        o = K.wkv_steps(proj[:, :H * d], proj[:, H * d:v_at], proj[:, v_at:gate_at], log_decay, None, None, mem.states["S"],
+                        ctx.slot_ids, ctx.cu_seqlens, H, d, dv, chunk_plan=K.wkv_chunk_plan(ctx, d), after=True,
+                        r_scale=d ** -0.5)
+        y = K.group_gated_norm(o, proj[:, gate_at:low_at], self.norm_weight, dv, self.eps, "silu")
+        return K.linear(y, self.w_o, partial_ok=True)
+
+
+def _stacked(blocks) -> torch.Tensor:
+    """Weights that read one input as one matrix, with rows of zeros up to a multiple of 8 (rows of the product then stay
+    16-byte aligned)."""
+    rows = sum(b.shape[0] for b in blocks)
+    if rows % 8:
+        blocks = list(blocks) + [blocks[0].new_zeros((8 - rows % 8, blocks[0].shape[1]))]
+    return torch.cat(blocks, dim=0).contiguous()
+
+
+OUT_NORM = "out.weight"      # below ``left.`` and ``right.``
+
+
 class ParallelMixer:
     """Two mixers side by side on the same input: ``left_scale * left(x) + right_scale * right(x)``.  Either may keep
     pages, either may keep state (their state tensors are declared under ``left.`` and ``right.``); their results
-    go on as a float stack of two weighed shares that the next norm adds."""
+    go on as a float stack of two weighed shares that the next norm adds.
 
-    def __init__(self, left: PartSpec, right: PartSpec, left_scale: float = 1.0, right_scale: float = 1.0):
+    With ``out_norm_eps`` every result first goes through an RMS norm of its own over the width (weights ``left.out`` and
+    ``right.out``): the results then travel as a ``K.PendingPair``, and the next norm's kernel norms both, adds them to the
+    stream and norms the stream."""
+
+    def __init__(self, left: PartSpec, right: PartSpec, left_scale: float = 1.0, right_scale: float = 1.0,
+                 out_norm_eps: Optional[float] = None, hidden_size: Optional[int] = None):
+        self.out_norm_eps = float(out_norm_eps) if out_norm_eps is not None else None
+        self.hidden_size = int(hidden_size) if hidden_size else None
+        if self.out_norm_eps is not None and not self.hidden_size:
+            raise ValueError("norms on the results need the width")
         self.sides = (("left.", build_part("mixer", left), float(left_scale)),
                       ("right.", build_part("mixer", right), float(right_scale)))
         if sum(part.cache_spec() is not None for _, part, _ in self.sides) > 1:
@@ -288,7 +376,10 @@ class ParallelMixer:
         return all(is_replayable(part) for _, part, _ in self.sides)
 
     def tensors(self) -> dict:
-        return {prefix + name: ts for prefix, part, _ in self.sides for name, ts in part.tensors().items()}
+        out = {prefix + name: ts for prefix, part, _ in self.sides for name, ts in part.tensors().items()}
+        if self.out_norm_eps is not None:
+            out.update({prefix + OUT_NORM: TensorSpec((self.hidden_size,), role="vector", init="norm") for prefix, _, _ in self.sides})
+        return out
 
     def cache_spec(self):
         return next((part.cache_spec() for _, part, _ in self.sides if part.cache_spec() is not None), None)
@@ -302,9 +393,14 @@ class ParallelMixer:
 
     def bind(self, tensors: dict, dtype: torch.dtype) -> None:
         for prefix, part, _ in self.sides:
-            part.bind({k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)}, dtype)
+            part.bind({k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix) and k != prefix + OUT_NORM}, dtype)
+        if self.out_norm_eps is not None:      # the constant on a side's share is part of its norm's weight
+            self.out_weights = [(tensors[prefix + OUT_NORM] * scale).contiguous() for prefix, _, scale in self.sides]
 
     def forward(self, x, ctx: StepContext, mem: LayerMemory):
+        if self.out_norm_eps is not None:
+            a, b = (part.forward(x, ctx, mem.below(prefix)) for prefix, part, _ in self.sides)
+            return K.PendingPair(a, b, *self.out_weights, self.out_norm_eps)
         out = torch.empty((len(self.sides), x.shape[0], x.shape[1]), dtype=torch.float32, device=x.device)
         for i, (prefix, part, scale) in enumerate(self.sides):
             K.scaled_sum(out[i], part.forward(x, ctx, mem.below(prefix)), scale)
@@ -315,4 +411,5 @@ register_part("mixer", "retention", Retention)
 register_part("mixer", "state_space", StateSpaceMixer)
 register_part("mixer", "gated_delta", GatedDeltaMixer)
 register_part("mixer", "time_mix", TimeMix)
+register_part("mixer", "gated_linear_attention", GatedLinearAttention)
 register_part("mixer", "parallel", ParallelMixer)

@@ -22,7 +22,7 @@ class RotaryEncoding:
     replayable = True      # the table is computed on the device from the step's positions
 
     def __init__(self, head_dim: int, theta: float, rotary_dim: int | None = None, interleaved: bool = False,
-                 rescale: dict | None = None, by_wavelength: dict | None = None):
+                 rescale: dict | None = None, by_wavelength: dict | None = None, linear_factor: float | None = None):
         self.head_dim = int(head_dim)
         self.theta = float(theta)
         self.rotary_dim = int(rotary_dim) if rotary_dim is not None else self.head_dim
@@ -34,7 +34,9 @@ class RotaryEncoding:
         self.amplitude = 0.1 * math.log(float(self.rescale["factor"])) + 1.0 if self.rescale else 1.0
         # frequencies slowed down by wavelength (the Llama 3.1 rule): see ``inverse_frequencies``
         self.by_wavelength = dict(by_wavelength) if by_wavelength else None
-        if self.rescale and self.by_wavelength:
+        # every frequency slowed down by one factor (1: as they are, computed in double)
+        self.linear_factor = float(linear_factor) if linear_factor is not None else None
+        if sum(rule is not None for rule in (self.rescale, self.by_wavelength, self.linear_factor)) > 1:
             raise ValueError("one rule for the frequencies, not two")
         self.inv_freq = None
 
@@ -44,6 +46,8 @@ class RotaryEncoding:
     def inverse_frequencies(self) -> torch.Tensor:
         """float32 table of rotary_dim/2 entries, computed as the reference does."""
         d = self.rotary_dim
+        if self.linear_factor is not None:      # computed in double, rounded once
+            return (self.theta ** (-2.0 * torch.arange(d // 2, dtype=torch.float64) / d) / self.linear_factor).to(torch.float32)
         if self.by_wavelength is not None:
             # ``by_wavelength`` = {factor, low, high, original}: a pair whose wavelength 2 pi / f is below original / high
             # keeps f, one above original / low turns ``factor`` times slower, and between the two f is blended with
@@ -85,7 +89,7 @@ class RotaryEncoding:
     def rotation_table(self, ctx):
         """Float cos/sin table of the step's positions for the attention-input kernel."""
         key = ("rope_table", self.theta, self.rotary_dim, tuple(sorted(self.rescale.items())) if self.rescale else None,
-               tuple(sorted(self.by_wavelength.items())) if self.by_wavelength else None)
+               tuple(sorted(self.by_wavelength.items())) if self.by_wavelength else None, self.linear_factor)
         table = ctx.extras.get(key)
         if table is None:
             if self.rescale is None:

@@ -78,12 +78,14 @@ class PagedCacheSpec:
     page id) and which earlier tokens it reads.  ``window`` None: every earlier token is read
     ("full"); otherwise only the last ``window`` are, and older pages are given back.  ``chunk``: a token
     reads those of its own block of ``chunk`` positions (counted from position 0), and the pages of a
-    finished block are given back.  Mixers with
+    finished block are given back.  ``keep_first``: beside a window or a block the first so many tokens are read by every
+    later one, and their pages stay.  Mixers with
     the same need share a page pool and a block table (a *group*), whatever tensors they keep."""
 
     tensors: tuple
     window: Optional[int] = None
     chunk: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self):
         names = [t.name for t in self.tensors]
@@ -94,7 +96,8 @@ class PagedCacheSpec:
 
     @property
     def group_key(self) -> tuple:
-        return ("window", self.window) if self.window else ("chunk", self.chunk) if self.chunk else ("full",)
+        key = ("window", self.window) if self.window else ("chunk", self.chunk) if self.chunk else ("full",)
+        return key + (self.keep_first,) if self.keep_first and key != ("full",) else key
 
 
 def widest_need(keys) -> tuple:
@@ -104,17 +107,20 @@ def widest_need(keys) -> tuple:
     if len(keys) == 1:
         return keys.pop()
     if all(k[0] == "window" for k in keys):
-        return ("window", max(k[1] for k in keys))
+        kept = max(k[2] if len(k) > 2 else 0 for k in keys)
+        return ("window", max(k[1] for k in keys)) + ((kept,) if kept else ())
     return ("full",)
 
 
-def kv_cache_spec(num_kv_heads: int, head_dim: int, window: Optional[int] = None, chunk: Optional[int] = None) -> PagedCacheSpec:
+def kv_cache_spec(num_kv_heads: int, head_dim: int, window: Optional[int] = None, chunk: Optional[int] = None,
+                  keep_first: int = 0) -> PagedCacheSpec:
     """Keys and values of grouped-query attention in the layout its kernels read: a key page is
     ``[kv_heads, page_size, head_dim]`` (one head's keys of a page are contiguous), a value page
     is transposed, ``[kv_heads, head_dim, page_size]`` (8 consecutive keys of one head element are
     16 aligned bytes)."""
     shape = (int(num_kv_heads), int(head_dim))
-    return PagedCacheSpec((PagedTensorSpec("k", shape, slot_axis=1), PagedTensorSpec("v", shape, slot_axis=2)), window, chunk)
+    return PagedCacheSpec((PagedTensorSpec("k", shape, slot_axis=1), PagedTensorSpec("v", shape, slot_axis=2)), window, chunk,
+                          keep_first)
 
 
 @dataclass(frozen=True)
