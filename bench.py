@@ -130,6 +130,27 @@ def fezuzen_shape(width, layers, heads, experts, top, expert_ff, shared_ff, grou
             "logit_scale": 0.5, "layers": out}
 
 
+def kuditar_shape(width, layers, heads, ff, experts, top, expert_ff, vocab=32000, window=1024, block=2048):
+    """Layers in the order attention (half of a head rotated, blended values, an output gate), window attention (the first
+    16 tokens kept, sinks) beside the gated delta rule, block attention beside gated linear attention (a decay from a rank
+    of 16), window attention beside the delta rule again; heads of 128 everywhere, a quarter as many kv heads, capped
+    scores; a clamped gated feed-forward in every fourth layer, routed experts (top * expert_ff = ff) in the others."""
+    kv = max(1, heads // 4)
+    own = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    att = {"type": "attention", "mixer": dict(own, rot={"base": 1e6, "dims": 64, "scaling": {"factor": 4.0}}, softcap=50.0, v_mix=True)}
+    par = {"type": "parallel", "mixer": {
+        "left": dict(own, rot={"base": 1e4, "dims": 128}, softcap=50.0, mask={"size": window, "keep_first": 16}),
+        "right": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}}}
+    par2 = {"type": "parallel_2", "mixer": {
+        "left": dict(own, mask={"size": block}),
+        "right": {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0, "decay_rank": 16}}}
+    order = (att, par, par2, par)
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top, "scale": 2.0}, "expert": {"ff": expert_ff, "limit": 7.0}}
+    return {"architecture": "Kuditar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 2.0},
+            "layers": [dict(order[i % 4], mlp=moe if i % 4 else dense) for i in range(layers)]}
+
+
 # --only design: Lomozen beside the dense model of the same width, depth, vocabulary and feed-forward
 # parameters per token (top * expert + shared = intermediate)
 DESIGN_SHAPES = {
@@ -164,6 +185,13 @@ ZERIPEL_SHAPES = {
 FEZUZEN_SHAPES = {
     "2k": (fezuzen_shape(2048, 8, 16, 32, 4, 768, 1536, 8),) + DESIGN_SHAPES["2k"],
     "4k": (fezuzen_shape(4096, 8, 32, 64, 6, 1536, 3072, 8),) + DESIGN_SHAPES["4k"],
+}
+# --only design --design kuditar: Kuditar beside Dumazen (the closest kin of its mixers: window attention side by side with the
+# gated delta rule), Zeripel (the closest kin of its feed-forwards and of the decay per key channel) and the dense model, all
+# of one width, depth, vocabulary and feed-forward parameters per token (top * expert = intermediate)
+KUDITAR_SHAPES = {
+    "2k": (kuditar_shape(2048, 8, 16, 3072, 32, 4, 768), DUMAZEN_SHAPES["2k"][0], ZERIPEL_SHAPES["2k"][0], DESIGN_SHAPES["2k"][1]),
+    "4k": (kuditar_shape(4096, 8, 32, 8192, 64, 8, 1024), DUMAZEN_SHAPES["4k"][0], ZERIPEL_SHAPES["4k"][0], DESIGN_SHAPES["4k"][1]),
 }
 PROMPT_LEN = 1024
 MAX_CONTEXT = 8192
@@ -293,6 +321,7 @@ def measure_design(args, rng):
               else zip(("bozisun", "lomozen", "dense"), BOZISUN_SHAPES[args.design_shape]) if args.design == "bozisun"
               else zip(("zeripel", "lomozen", "dense"), ZERIPEL_SHAPES[args.design_shape]) if args.design == "zeripel"
               else zip(("fezuzen", "lomozen", "dense"), FEZUZEN_SHAPES[args.design_shape]) if args.design == "fezuzen"
+              else zip(("kuditar", "dumazen", "zeripel", "dense"), KUDITAR_SHAPES[args.design_shape]) if args.design == "kuditar"
               else zip(("lomozen", "dense"), DESIGN_SHAPES[args.design_shape]))
     out["design"] = args.design
     for name, cfg in models:
@@ -462,7 +491,7 @@ def main():
     ap.add_argument("--no-kernel-share", action="store_true", help="leave out the per-kernel time shares")
     ap.add_argument("--design-shape", choices=sorted(DESIGN_SHAPES), default="2k",
                     help="with --only design: the width of both models (2,048 or 4,096), 8 layers each")
-    ap.add_argument("--design", choices=["lomozen", "dumazen", "bozisun", "zeripel", "fezuzen"], default="lomozen",
+    ap.add_argument("--design", choices=["lomozen", "dumazen", "bozisun", "zeripel", "fezuzen", "kuditar"], default="lomozen",
                     help="with --only design: the architecture that is measured beside its kin of equal size")
     ap.add_argument("--design-models", default="", help="with --only design: only these of the models, with commas between them")
     ap.add_argument("--only", choices=["prefill", "decode", "mixed", "long-prompt", "ttft", "calibrate", "design"], default=None,

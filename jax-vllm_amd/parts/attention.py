@@ -53,7 +53,7 @@ class GroupedQueryAttention:
         are kept for the step; "later": the values become (1 - l) v + l v_first with v_first those of the same token and l a
         learned number, before they are cached.
         Any of these but ``chunk``, ``softmax_plus_one``, ``softcap``, ``keep_first`` and ``sinks`` takes the ``wide`` path (so does
-        ``qkv_bias`` beside one of the last three): heads cached
+        ``qkv_bias``, unless pairs (2i, 2i + 1) turn): heads cached
         under one padded size (``K.padded_head_dim``), prepared by ``K.attn_prepare_wide``, read by the same paged
         attention kernels."""
         if num_heads % num_kv_heads:
@@ -99,9 +99,14 @@ class GroupedQueryAttention:
             turn = self.value_position.as_rotation()
             if turn is None or turn != (self.dv, True):
                 raise ValueError("values turn whole, in pairs (2m, 2m + 1)")
+        self.position = build_part("position", position) if position is not None else None
+        # what the position part asks of this mixer's kernels: a rotation of q and k by position
+        # (rotary_dim, interleaved), or nothing (a part that acts elsewhere, or no part at all)
+        self.rotation = self.position.as_rotation() if self.position is not None else None
         self.wide = (self.filtered or self.values_are_keys or self.q_temperature is not None or self.dv != self.dk or (qk_norm == "whole" and qk_norm_eps is not None) or self.v_scale != 1.0
                      or self.output_gate or not self.qk_norm_weight or self.value_blend is not None
-                     or (bool(qkv_bias) and (self.softcap is not None or self.keep_first > 0 or self.learned_sinks)))
+                     # biases are added where the heads are prepared; only pairs (2i, 2i + 1) need a pass of their own
+                     or (bool(qkv_bias) and not (self.rotation is not None and self.rotation[1])))
         if self.value_blend is not None and (self.filtered or qkv_bias or values_are_keys or qk_norm == "whole"):
             raise ValueError("blended values: without filters, biases, values taken from the keys or a norm over the whole projection")
         # what the paged attention kernels see
@@ -111,10 +116,6 @@ class GroupedQueryAttention:
         self.qk_norm_eps = qk_norm_eps
         self.window = int(window) if window else None
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.dk)
-        self.position = build_part("position", position) if position is not None else None
-        # what the position part asks of this mixer's kernels: a rotation of q and k by position
-        # (rotary_dim, interleaved), or nothing (a part that acts elsewhere, or no part at all)
-        self.rotation = self.position.as_rotation() if self.position is not None else None
         if self.filtered and (self.dk % 2 or self.dv % 2 or (self.rotation is not None and not self.rotation[1])):
             raise ValueError("the filtered attention input takes even head sizes and turns pairs (2i, 2i + 1)")
         self.qkv_bias, self.o_bias = bool(qkv_bias), bool(o_bias)

@@ -99,7 +99,7 @@ def write_safetensors(path, tensors: Iterable, metadata: dict | None = None) -> 
             t = make().contiguous()
             if tuple(t.shape) != tuple(shape) or t.dtype != dtype:
                 raise ValueError(f"tensor {name!r} was produced as {tuple(t.shape)} {t.dtype}, declared {shape} {dtype}")
-            f.write(t.view(torch.uint8).numpy().tobytes() if t.numel() else b"")
+            f.write(t.reshape(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b"")
 
 
 def open_shards(folder) -> Iterator[SafetensorsFile]:

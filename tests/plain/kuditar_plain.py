@@ -145,6 +145,11 @@ def heads_of(y, count: int):
     return y.view(y.shape[0], count, -1).transpose(0, 1)
 
 
+def seen_by(shared: dict, seen):
+    """The layer's own mask, or the one a test puts in its place."""
+    return seen if shared.get("mask") is None else shared["mask"]
+
+
 def attention(w: dict, p: str, m: dict, h, eps: float, shared: dict):
     H, G = int(m["heads"]), int(m["kv_heads"])
     q, k = heads_of(linear(h, w[p + "q"]), H), heads_of(linear(h, w[p + "k"]), G)
@@ -158,7 +163,7 @@ def attention(w: dict, p: str, m: dict, h, eps: float, shared: dict):
             v = rounded((1 - lam) * v + lam * shared["v_first"])
         else:
             shared["v_first"] = v
-    o = weigh(q, k, v, visible_window(h.shape[0]), float(m["scale"]), m.get("softcap"))
+    o = weigh(q, k, v, seen_by(shared, visible_window(h.shape[0])), float(m["scale"]), m.get("softcap"))
     return linear(rounded(o * torch.sigmoid(linear(h, w[p + "g"]))), w[p + "o"])
 
 
@@ -173,13 +178,14 @@ def side_attention(w: dict, p: str, m: dict, h, eps: float, seen):
     return linear(o, w[p + "o"])
 
 
-def kept_window_attention(w, p, m, h, eps):
+def kept_window_attention(w, p, m, h, eps, shared):
     mask = m.get("mask") or {}
-    return side_attention(w, p, m, h, eps, visible_window(h.shape[0], mask.get("size"), int(mask.get("keep_first") or 0)))
+    seen = visible_window(h.shape[0], mask.get("size"), int(mask.get("keep_first") or 0))
+    return side_attention(w, p, m, h, eps, seen_by(shared, seen))
 
 
-def chunked_attention(w, p, m, h, eps):
-    return side_attention(w, p, m, h, eps, visible_chunk(h.shape[0], (m.get("mask") or {}).get("size")))
+def chunked_attention(w, p, m, h, eps, shared):
+    return side_attention(w, p, m, h, eps, seen_by(shared, visible_chunk(h.shape[0], (m.get("mask") or {}).get("size"))))
 
 
 # --------------------------------------------------------------------------- recurrences
@@ -234,7 +240,7 @@ def gated_linear(w: dict, p: str, m: dict, h, eps: float):
 
 def side_by_side(left, right):
     def run(w, p, m, h, eps, shared):
-        a = by_rms(left(w, p + "left.", m["left"], h, eps), eps) * w[p + "left.out"]
+        a = by_rms(left(w, p + "left.", m["left"], h, eps, shared), eps) * w[p + "left.out"]
         b = by_rms(right(w, p + "right.", m["right"], h, eps), eps) * w[p + "right.out"]
         return (a + b) / 2
     return run
@@ -275,14 +281,15 @@ def feed_forward(w: dict, p: str, f: dict, h):
 
 
 # --------------------------------------------------------------------------- the model
-def forward(w: dict, cfg: dict, tokens, layers_out: list | None = None):
+def forward(w: dict, cfg: dict, tokens, layers_out: list | None = None, masks: dict | None = None):
     """Logits [n, vocab] of one sequence from position 0; with ``layers_out`` the residual stream after
-    every layer is appended to it."""
+    every layer is appended to it; ``masks`` {layer: [n, n]} replaces what some layers' queries see."""
     eps = float(cfg["norm"]["eps"])
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)] * float((cfg.get("embedding") or {}).get("scale", 1.0))
     shared: dict = {}
     for i, layer in enumerate(cfg["layers"]):
         p = f"l{i}."
+        shared["mask"] = (masks or {}).get(i)
         h = layer_norm(x, w[p + "norm1"], w[p + "norm1.b"], eps)
         x = x + MIXERS[layer["type"]](w, p + "mix.", layer["mixer"], h, eps, shared)
         if layer.get("mlp") is not None:
