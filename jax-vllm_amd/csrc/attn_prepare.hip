@@ -183,10 +183,13 @@ attn_prepare_heads_vec_kernel(T* __restrict__ q_out, const T* __restrict__ qkv, 
   const bool store = sm >= 0 && k_pages != nullptr;
   const tv xv = *(const tv*)(qkv + t * ld + (long long)head * dk + e0);
   const float* w = is_q ? q_w : k_w;
-  float a[EP], ss = 0.f;
+  float a[EP], bv[EP], ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < EP; ++e) bv[e] = 0.f;
+  if (bias) load_floats<EP>(bias + head * dk + e0, bv);
 #pragma unroll
   for (int e = 0; e < EP; ++e) {
-    a[e] = to_f32<T>(xv[e]) + (bias ? bias[head * dk + e0 + e] : 0.f);
+    a[e] = to_f32<T>(xv[e]) + bv[e];
     ss = fmaf(a[e], a[e], ss);
   }
   if (w) {

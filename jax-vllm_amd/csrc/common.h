@@ -94,4 +94,15 @@ __device__ __forceinline__ float jv_act(int act, float z) {
   return z;
 }
 
+// N consecutive floats (a multiple of 4) in pieces of 16 bytes, from any address of a float.
+template <int N> __device__ __forceinline__ void load_floats(const float* p, float (&v)[N]) {
+  typedef float f4 __attribute__((ext_vector_type(4), aligned(4)));
+#pragma unroll
+  for (int i = 0; i < N; i += 4) {
+    const f4 x = *(const f4*)(p + i);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[i + e] = x[e];
+  }
+}
+
 #define JV_LAUNCH_CHECK() ((int)hipGetLastError())

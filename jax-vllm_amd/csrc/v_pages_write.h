@@ -31,8 +31,10 @@ __global__ void __launch_bounds__(256) v_pages_write_kernel(
     typedef T tv __attribute__((ext_vector_type(EP)));
     tv v = *(const tv*)(src + (t0 + j) * row_stride + c);
     if (bias) {
+      float b[EP];
+      load_floats<EP>(bias + kvh * D + c, b);
 #pragma unroll
-      for (int e = 0; e < EP; ++e) v[e] = from_f32<T>(to_f32<T>(v[e]) + bias[kvh * D + c + e]);
+      for (int e = 0; e < EP; ++e) v[e] = from_f32<T>(to_f32<T>(v[e]) + b[e]);
     }
     if (first) {
       const T* f = first + (t0 + j) * first_stride + (long long)kvh * D + c;

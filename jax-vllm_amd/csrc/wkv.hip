@@ -345,18 +345,26 @@ wkv_apply_kernel(float* __restrict__ out, const float* __restrict__ scratch, con
 }
 
 // ---------------------------------------------------------------- decays from a projection of small rank
+// log(1 + e^-a) for a >= 0: u = 1 + e rounded, and log(u) e / (u - 1) takes that rounding back (Kahan's log1p), so the
+// hardware's logarithm and exponential give the result to a few units in the last place.
+__device__ __forceinline__ float softplus_of_negative(float a) {
+  const float e = __builtin_amdgcn_exp2f(-a * 1.4426950408889634f);
+  const float u = 1.f + e, d = u - 1.f;
+  return d > 0.f ? __builtin_amdgcn_logf(u) * 0.6931471805599453f * (e * __builtin_amdgcn_rcpf(d)) : e;
+}
+
 // out[t][c] = log(sigmoid(z)) / tau,  z = sum_r W[c][r] low[t][r] + b[c]; W [channels][rank] and low (rows of stride ldl) in
 // the activation type, sums and logarithm float.  grid (channel blocks of 256, blocks of LD_TOKENS tokens).
 #define LD_TOKENS 8
 template <typename T>
 __global__ void __launch_bounds__(256)
 low_rank_decay_kernel(float* __restrict__ out, const T* __restrict__ low, long long ldl, const T* __restrict__ W,
-                      const float* __restrict__ b, long long n, int channels, int rank, float inv_tau) {
-  extern __shared__ float lows[];         // [LD_TOKENS][rank]
+                      const float* __restrict__ b, long long n, int channels, int rank, float inv_tau, int vec) {
+  extern __shared__ __attribute__((aligned(16))) float lows[];         // [rank][LD_TOKENS]: a thread reads its tokens' numbers 16 bytes at a time
   const long long t0 = (long long)blockIdx.y * LD_TOKENS;
   for (int i = threadIdx.x; i < LD_TOKENS * rank; i += 256) {
-    const int t = i / rank;
-    lows[i] = t0 + t < n ? to_f32(low[(t0 + t) * ldl + (i - t * rank)]) : 0.f;
+    const int t = i / rank, r = i - t * rank;
+    lows[r * LD_TOKENS + t] = t0 + t < n ? to_f32(low[(t0 + t) * ldl + r]) : 0.f;
   }
   __syncthreads();
   const int c = blockIdx.x * 256 + threadIdx.x;
@@ -365,15 +373,27 @@ low_rank_decay_kernel(float* __restrict__ out, const T* __restrict__ low, long l
 #pragma unroll
   for (int t = 0; t < LD_TOKENS; ++t) z[t] = b[c];
   const T* w = W + (long long)c * rank;
-#pragma unroll 8
-  for (int r = 0; r < rank; ++r) {
-    const float wv = to_f32(w[r]);
+  if (vec) {      // rows of W in pieces of 16 bytes, a piece's sums in the same order
+    constexpr int EP = 16 / (int)sizeof(T);
+    typedef T tv __attribute__((ext_vector_type(EP)));
+#pragma unroll 2
+    for (int r = 0; r < rank; r += EP) {
+      const tv wv = *(const tv*)(w + r);
 #pragma unroll
-    for (int t = 0; t < LD_TOKENS; ++t) z[t] = fmaf(wv, lows[t * rank + r], z[t]);
+      for (int e = 0; e < EP; ++e)
+#pragma unroll
+        for (int t = 0; t < LD_TOKENS; ++t) z[t] = fmaf(to_f32<T>(wv[e]), lows[(r + e) * LD_TOKENS + t], z[t]);
+    }
+  } else {
+    for (int r = 0; r < rank; ++r) {
+      const float wv = to_f32(w[r]);
+#pragma unroll
+      for (int t = 0; t < LD_TOKENS; ++t) z[t] = fmaf(wv, lows[r * LD_TOKENS + t], z[t]);
+    }
   }
 #pragma unroll
   for (int t = 0; t < LD_TOKENS; ++t)
-    if (t0 + t < n) out[(t0 + t) * channels + c] = -(fmaxf(-z[t], 0.f) + log1pf(expf(-fabsf(z[t])))) * inv_tau;
+    if (t0 + t < n) out[(t0 + t) * channels + c] = -(fmaxf(-z[t], 0.f) + softplus_of_negative(fabsf(z[t]))) * inv_tau;
 }
 
 extern "C" int jv_wkv_max_dim() { return WKV_ROWS * 256; }
@@ -427,7 +447,8 @@ extern "C" int jv_wkv_chunk_max_dim() { return 128; }
       return (int)hipErrorInvalidValue;                                                                         \
     hipLaunchKernelGGL(low_rank_decay_kernel<T>, dim3((channels + 255) / 256, (n + LD_TOKENS - 1) / LD_TOKENS), \
                        dim3(256), (size_t)LD_TOKENS * rank * sizeof(float), (hipStream_t)stream, out,           \
-                       (const T*)low, ldl, (const T*)W, b, n, channels, rank, 1.f / tau);                       \
+                       (const T*)low, ldl, (const T*)W, b, n, channels, rank, 1.f / tau,                        \
+                       rank % (16 / (int)sizeof(T)) == 0 && (uintptr_t)W % 16 == 0 ? 1 : 0);                    \
     return JV_LAUNCH_CHECK();                                                                                   \
   }
 

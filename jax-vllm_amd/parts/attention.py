@@ -219,9 +219,26 @@ class GroupedQueryAttention:
         """x goes into the qkv product and nowhere else: the norm before may leave its scale to that product."""
         return K.linear_takes_unscaled_rows(n_rows, self.w_qkv, partial_ok=self._qkv_parts_ok(), partial_max_width=None)
 
+    # ---- one product with what else reads the same input (``parts/recurrent.py: ParallelMixer``)
+    def input_weight(self):
+        """The matrix of the one product this mixer begins with, or None where it has to make that product itself."""
+        return self.w_qkv if self.wide and not self.filtered else None
+
+    def share_input(self, weight: torch.Tensor) -> None:
+        self.w_qkv = weight
+
+    def forward_projected(self, proj, at: int, ctx: StepContext, mem: LayerMemory) -> torch.Tensor:
+        """The rest of the mixer behind its input product, whose columns begin at ``at`` (0: the heads are read from the
+        rows' beginning)."""
+        if at:
+            raise ValueError("the attention's heads begin its rows")
+        return self._forward_wide(proj, ctx, mem)
+
     # ---- one step
     def forward(self, x, ctx: StepContext, mem: LayerMemory) -> torch.Tensor:
         n = x.shape[0]
+        if self.wide and not self.filtered:
+            return self._forward_wide(K.linear(x, self.w_qkv), ctx, mem)
         rotary_dim, interleaved = self.rotation if self.rotation is not None else (0, False)
         cos_sin = self.position.rotation_table(ctx) if self.rotation is not None else None
         # at few rows the projection may come as float partial products, which the next kernel adds
@@ -229,8 +246,6 @@ class GroupedQueryAttention:
                        partial_ok=self._qkv_parts_ok())
         if self.filtered:
             return self._forward_filtered(qkv, ctx, mem, cos_sin, rotary_dim)
-        if self.wide:
-            return self._forward_wide(qkv, ctx, mem, cos_sin, rotary_dim, interleaved)
         if self.b_qkv is not None:
             K.add_bias(qkv, self.b_qkv)
         parts = None
@@ -273,7 +288,9 @@ class GroupedQueryAttention:
             K.add_bias(y, self.b_o)
         return y
 
-    def _forward_wide(self, qkv, ctx: StepContext, mem: LayerMemory, cos_sin, rotary_dim: int, interleaved: bool):
+    def _forward_wide(self, qkv, ctx: StepContext, mem: LayerMemory):
+        rotary_dim, interleaved = self.rotation if self.rotation is not None else (0, False)
+        cos_sin = self.position.rotation_table(ctx) if self.rotation is not None else None
         if interleaved:
             raise ValueError("heads of two sizes and a norm over the whole projection rotate half-split pairs only")
         writes = mem.writes
