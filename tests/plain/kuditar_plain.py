@@ -14,7 +14,7 @@ The design in this file's notation (n tokens, width w):
                first tokens, a sink] and [gated delta rule] side by side
 * parallel_2:  [attention with biases, weighted head norm, no rotation, blocks of positions] and [linear attention whose
                decay sigmoid(z)^(1/tau) acts per key channel, read after the write] side by side
-               either pair: half the sum of the two outputs, each by its root mean square over the width times a weight
+               either pair gives (a + b) / 2, a and b the sides' results under RMS norms of their own
 * feed-forward: W_down (g sigmoid(1.702 g) (u + 1)) with g = min(gate, c), u = clamp(up, -c, c), dense or as experts: the
                ``top`` experts by sigmoid(z) + correction, weighed by sigmoid(z) times a constant
 * output:      L(x), logits = embed @ that
